@@ -3,8 +3,8 @@
 ``ARCHITECTURES`` maps the string in config.json's ``architectures`` list to an
 architecture (a typed configuration class plus a function that turns such a
 configuration into a ``ModelSpec``).  ``MIXERS``, ``FEED_FORWARDS``, ``NORMS``,
-``POSITION_ENCODINGS``, ``BLOCKS``, ``EMBEDDINGS``, ``HEADS``, ``FILTERS`` and ``STREAM_SHIFTS`` map a
-``PartSpec.kind`` to a part class.
+``POSITION_ENCODINGS``, ``BLOCKS``, ``EMBEDDINGS``, ``HEADS``, ``FILTERS``, ``STREAM_SHIFTS`` and
+``STREAM_ENTRIES`` map a ``PartSpec.kind`` to a part class.
 Code outside this package (a test, a plug-in) adds an entry with
 ``@REGISTRY.register("name")`` and needs no change to the package's files.
 
@@ -70,6 +70,7 @@ EMBEDDINGS = Registry("embedding")
 HEADS = Registry("output head")
 FILTERS = Registry("input filter")
 STREAM_SHIFTS = Registry("stream shift")
+STREAM_ENTRIES = Registry("stream entry")
 
 
 def register_architecture(name: str, config_class: Any, to_spec: Callable[[Any], Any], *, replace: bool = False):

@@ -65,7 +65,9 @@ class LayerCall:
     ``shift``   a row of the model's stream shift (``ModelSpec.stream_shift``)
                 that is added to the residual stream right before this call;
     ``reinject`` true: the embedding's output (the stream's first value, row by
-                row) is added to the residual stream right before this call.
+                row) is added to the residual stream right before this call;
+    ``enter``   true: the model's stream entry (``ModelSpec.stream_entry``) makes the
+                residual stream anew right before this call.
     """
 
     layer: int
@@ -73,6 +75,7 @@ class LayerCall:
     writes: bool = True
     shift: Optional[int] = None
     reinject: bool = False
+    enter: bool = False
 
 
 @dataclass(frozen=True)
@@ -99,6 +102,9 @@ class ModelSpec:
     # (``LayerCall.shift``), and the tensor-name prefix it is found under.
     stream_shift: Optional[PartSpec] = None
     stream_shift_prefix: str = ""
+    # What makes the residual stream anew for calls that say so (``LayerCall.enter``), and its tensors' prefix.
+    stream_entry: Optional[PartSpec] = None
+    stream_entry_prefix: str = ""
     eos_token_ids: tuple = ()
     ignorable_tensors: tuple = ()    # shell-style patterns of tensor names a file may hold unused
     init_std: float = 0.02           # random-weights mode: normal(0, init_std) matrices

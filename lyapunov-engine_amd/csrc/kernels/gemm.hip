@@ -15,7 +15,7 @@
 #include <algorithm>
 #include <type_traits>
 
-#include "common.h"
+#include "stream_map.h"
 
 namespace lyp {
 
@@ -327,6 +327,8 @@ __global__ __launch_bounds__(512) void gemm_bf16_wide_kernel(const bf16_t* __res
 enum SkinnyEpilogue : int {
   kEpiAct = 0, kEpiF32 = 1, kEpiSwiglu = 2, kEpiParts = 3, kEpiRope = 4,
   kEpiResidual = 5,  // C is the float residual stream: C += A . W^T
+  kEpiStream = 6,    // C = base + A . W^T (float), and the next branch's input map(C) with it (StreamTail)
+  kEpiRelu2 = 7,     // stored in the operands' type as max(y, 0)^2
 };
 
 // The residual epilogue's by-products for the RMS norm that follows: with
@@ -339,6 +341,17 @@ struct ResidualTail {
   void* xs;            // [M][ldx]
   int ldx;
   float* ssq_part;     // [workgroups][16]: rows past M get zeros
+};
+
+// kEpiStream: the sum v = base + A . W^T is the residual stream's new value, and the branch that
+// follows reads it feature by feature (stream_map.h): both are written here, and neither the sum
+// nor the map needs a kernel of its own.  base may be the stream itself (C) or another tensor.
+struct StreamTail {
+  const float* base;   // [M][ldb]
+  int ldb;
+  void* xs;            // [M][ldx] of the operands' type
+  int ldx;
+  StreamMap map;
 };
 
 // For a product whose activations are such an xs: the sums are scaled by the
@@ -385,16 +398,17 @@ template <typename T, int MB, int EPI, bool NORMED = false, int ROWS = 16, bool 
 __global__ __launch_bounds__(1024) void gemm_skinny_kernel(const T* __restrict__ A, const T* __restrict__ W,
                                                            void* __restrict__ Cv, int M, int N, int K, int lda,
                                                            int ldw, int ldc, RopeTail tail, NormHead head,
-                                                           ResidualTail res) {
+                                                           ResidualTail res, StreamTail stm) {
+  constexpr bool JOINS = EPI == kEpiResidual || EPI == kEpiStream;   // the sum goes onto the residual stream
   using MM = Mma16Wide<T>;
   using Frag = typename MM::Frag;
   constexpr int NF = 16 / MM::kElems;  // fragments per lane per 64 values of K
   static_assert(ROWS == 16 || ROWS == 8, "a workgroup owns 16 rows of W, or 8 (the tile's lower half repeats them)");
   // With 16 rows of W a paired wave keeps two tiles, rows 0-7 and 8-15, over the same tokens: MB counts them.
-  static_assert(!PAIRED || (EPI == kEpiResidual && ((ROWS == 8 && MB == 1) || (ROWS == 16 && MB == 2))),
+  static_assert(!PAIRED || (JOINS && ((ROWS == 8 && MB == 1) || (ROWS == 16 && MB == 2))),
                 "two chunks per tile: 8 rows (or twice 8), 8 tokens");
   static_assert(TB == 1 || (TB == 2 && PAIRED && MB == 1), "blocks of 8 tokens: for the paired tile of 8 rows");
-  static_assert(RT == 1 || (!PAIRED && !NORMED && ROWS == 16 && EPI != kEpiResidual), "several row tiles: the plain tile only");
+  static_assert(RT == 1 || (!PAIRED && !NORMED && ROWS == 16 && !JOINS), "several row tiles: the plain tile only");
   constexpr int NT = MB * TB * RT;           // tiles (accumulators) a wave keeps: tile rt * MB + b is row tile rt, token block b
   constexpr int NB = PAIRED ? TB : MB;       // blocks of tokens whose activations it loads
   constexpr int CHUNK = PAIRED ? 128 : 64;  // values of K per step of a wave
@@ -446,16 +460,24 @@ __global__ __launch_bounds__(1024) void gemm_skinny_kernel(const T* __restrict__
       for (int i = 0; i < 4; ++i) sq[i] += __shfl_xor(sq[i], off, kWave);
     if (lane < 4) *reinterpret_cast<f32x4*>(row_val + wave * 16 + 4 * lane) = sq;
   }
-  float h_first = 0.f, nw_first = 0.f;  // kEpiResidual: what the thread's first element adds to and is weighted by
-  if constexpr (EPI == kEpiResidual) {
+  float h_first = 0.f, nw_first = 0.f, nb_first = 0.f;  // JOINS: what the thread's first element adds to and is weighted by
+  if constexpr (JOINS) {
     const int e = threadIdx.x, l = (e % 256) / 4, in_tile = 4 * (l / 16) + e % 4;
     const int row = PAIRED ? 8 * (e / 256 / TB) + in_tile : in_tile;
     const int m = (PAIRED ? 8 * (e / 256 % TB) : (e / 256) * 16) + l % 16, n = n0 + row;
     if (e < NT * 256 && in_tile < (PAIRED ? 8 : ROWS) && (!PAIRED || l % 16 < 8) && m < M && n < N) {
-      h_first = static_cast<const float*>(Cv)[static_cast<size_t>(m) * ldc + n];
-      if (res.next_w)
-        nw_first = res.next_w_f32 ? static_cast<const float*>(res.next_w)[n]
-                                  : to_f32(static_cast<const bf16_t*>(res.next_w)[n]);
+      if constexpr (EPI == kEpiStream) {
+        h_first = stm.base[static_cast<size_t>(m) * stm.ldb + n];
+        if (stm.map.kind == kMapTanh) {
+          nw_first = stm.map.w[n];
+          nb_first = stm.map.b[n];
+        }
+      } else {
+        h_first = static_cast<const float*>(Cv)[static_cast<size_t>(m) * ldc + n];
+        if (res.next_w)
+          nw_first = res.next_w_f32 ? static_cast<const float*>(res.next_w)[n]
+                                    : to_f32(static_cast<const bf16_t*>(res.next_w)[n]);
+      }
     }
   }
 
@@ -674,6 +696,20 @@ __global__ __launch_bounds__(1024) void gemm_skinny_kernel(const T* __restrict__
         static_cast<T*>(res.xs)[static_cast<size_t>(m) * res.ldx + n] = from_f32<T>(v * nw);
         sq_el[e] = v * v;
       }
+    } else if constexpr (EPI == kEpiStream) {
+      const bool first = e == static_cast<int>(threadIdx.x);
+      const float v = (first ? h_first : stm.base[static_cast<size_t>(m) * stm.ldb + n]) + total(e);
+      if (Cv != nullptr) static_cast<float*>(Cv)[static_cast<size_t>(m) * ldc + n] = v;
+      float w = nw_first, bias = nb_first;
+      if (!first && stm.map.kind == kMapTanh) {
+        w = stm.map.w[n];
+        bias = stm.map.b[n];
+      }
+      static_cast<T*>(stm.xs)[static_cast<size_t>(m) * stm.ldx + n] =
+          from_f32<T>(map_feature(stm.map.kind, stm.map.alpha, v, w, bias));
+    } else if constexpr (EPI == kEpiRelu2) {
+      const float y = fmaxf(total(e), 0.f);
+      static_cast<T*>(Cv)[static_cast<size_t>(m) * ldc + n] = from_f32<T>(y * y);
     } else if constexpr (EPI == kEpiParts) {
       static_cast<float*>(Cv)[(static_cast<size_t>(blockIdx.y) * M + m) * ldc + n] = total(e);
     } else if constexpr (EPI == kEpiF32) {
@@ -711,10 +747,11 @@ __global__ __launch_bounds__(1024) void gemm_skinny_kernel(const T* __restrict__
 // With `cand` every workgroup also leaves, per token, the largest logit among the rows it computed
 // and the first place it stands at: cand[token][workgroup].  The sampler then needs no pass over
 // the row to find the maximum.
-template <typename T, int MB>
+// SHAPED: every logit is scaled and capped (stream_map.h) before it is stored and compared.
+template <typename T, int MB, bool SHAPED = false>
 __global__ __launch_bounds__(256) void lm_head_kernel(const T* __restrict__ A, const T* __restrict__ W,
                                                       float* __restrict__ C, int M, int N, int K, int lda, int ldw,
-                                                      int ldc, ArgMax* __restrict__ cand) {
+                                                      int ldc, ArgMax* __restrict__ cand, float scale, float cap) {
   using MM = Mma16Wide<T>;
   using Frag = typename MM::Frag;
   constexpr int NF = 16 / MM::kElems;
@@ -766,6 +803,10 @@ __global__ __launch_bounds__(256) void lm_head_kernel(const T* __restrict__ A, c
     for (int b = 0; b < MB; ++b) {
       const int m = 16 * b + r, n = n0 + 4 * j;
       ArgMax mine{LYP_NEG_INF, 0x7fffffff};
+      if constexpr (SHAPED) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc[b][i] = shaped_logit(acc[b][i], scale, cap);
+      }
       if (m < M) {
         float* crow = C + static_cast<size_t>(m) * ldc + n;
         if (n + 3 < N && ldc % 4 == 0) {
@@ -810,10 +851,10 @@ __global__ __launch_bounds__(256) void lm_head_kernel(const T* __restrict__ A, c
 // (8 tokens on 128256 x 2048: 256 workgroups 106.5 us, 512 107.0, 1024 111.5, against 115.7 of
 // lm_head_kernel; 16 tokens 114 against 131, one token 100 against 105).
 // MB blocks of 16 tokens (what LDS holds of them: 32 tokens of 2,048 values): a fragment of weights is then used MB times.
-template <int RING, int MB>
+template <int RING, int MB, bool SHAPED = false>
 __global__ __launch_bounds__(256) void lm_head_stream_kernel(const bf16_t* __restrict__ A, const bf16_t* __restrict__ W,
                                                              float* __restrict__ C, int M, int N, int K, int lda, int ldw,
-                                                             int ldc, ArgMax* __restrict__ cand) {
+                                                             int ldc, ArgMax* __restrict__ cand, float scale, float cap) {
   using MM = Mma16Wide<bf16_t>;
   constexpr int kWaves = 4;
   extern __shared__ __attribute__((aligned(16))) unsigned char x_lds[];   // [16 MB][2 K + 16] bytes
@@ -874,6 +915,10 @@ __global__ __launch_bounds__(256) void lm_head_stream_kernel(const bf16_t* __res
     for (int b = 0; b < MB; ++b) {
       const int m = 16 * b + r;
       ArgMax mine{LYP_NEG_INF, 0x7fffffff};
+      if constexpr (SHAPED) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc[b][i] = shaped_logit(acc[b][i], scale, cap);
+      }
       if (m < M) {
         float* crow = C + static_cast<size_t>(m) * ldc + n;
         if (n + 3 < N && ldc % 4 == 0) {
@@ -953,7 +998,8 @@ static int skinny_row_tiles(int M, int N, int slices) {
 template <typename T, int EPI, bool NORMED = false, int ROWS = 16, bool PAIRED = false, int RT = 1>
 static void launch_skinny(const T* A, const T* W, void* C, int M, int N, int K, int lda, int ldw, int ldc,
                           int slices, hipStream_t stream, const RopeTail& tail = RopeTail{},
-                          const NormHead& head = NormHead{}, const ResidualTail& res = ResidualTail{}) {
+                          const NormHead& head = NormHead{}, const ResidualTail& res = ResidualTail{},
+                          const StreamTail& stm = StreamTail{}) {
   // tiles a wave keeps: paired, 8 rows of W each for 8 tokens each; else 16 rows of W for 16 tokens each
   const int MB = PAIRED ? (ROWS / 8) * ((M + 7) / 8) : (M + 15) / 16;
   const int waves = skinny_waves(N, K, MB * RT, slices, ROWS * RT, PAIRED ? 128 : 64);
@@ -971,7 +1017,7 @@ static void launch_skinny(const T* A, const T* W, void* C, int M, int N, int K, 
         asked = true;                                                                                                  \
       }                                                                                                                \
     }                                                                                                                  \
-    kernel<<<grid, block, lds, stream>>>(A, W, C, M, N, K, lda, ldw, ldc, tail, head, res);                            \
+    kernel<<<grid, block, lds, stream>>>(A, W, C, M, N, K, lda, ldw, ldc, tail, head, res, stm);                       \
   } while (0)
 #define LYP_SKINNY(MBV) LYP_SKINNY_TB(MBV, 1)
   if constexpr (PAIRED && ROWS == 16) {
@@ -1142,8 +1188,11 @@ constexpr int kHeadRing = 8;   // chunks a wave of lm_head_stream_kernel asks fo
 // cand (optional): [M][blocks] pairs of (float, int32) that receive every workgroup's largest logit
 // per row and its index.  Returns the number of workgroups used (the stride of cand), 0 when the
 // kernel does not take the operands (then use lyp_gemm_nt), negative on error.
+// scale, cap: every logit is cap * tanh(scale * z / cap) (cap 0: scale * z), also where the largest is looked for.
 extern "C" int lyp_lm_head(const void* A, const void* W, float* C, int dtype, int M, int N, int K, int lda, int ldw,
-                           int ldc, void* cand, int blocks, hipStream_t stream) {
+                           int ldc, void* cand, int blocks, float scale, float cap, hipStream_t stream) {
+  const bool shaped = scale != 1.0f || cap != 0.0f;
+  LYP_REQUIRE(cap >= 0.f, "lm_head: cap %f", static_cast<double>(cap));
   LYP_REQUIRE(N > 0 && K > 0 && ldc >= N && blocks >= 0 && blocks <= 4096, "lm_head: N=%d K=%d stride %d blocks %d", N, K,
               ldc, blocks);
   if (!skinny_ok(M, K, lda, ldw, A, W, dtype)) return 0;
@@ -1156,27 +1205,27 @@ extern "C" int lyp_lm_head(const void* A, const void* W, float* C, int dtype, in
   const size_t staged = static_cast<size_t>(16) * token_blocks * (2 * K + 16);
   if (dtype == kBF16 && token_blocks <= 2 && staged <= kHeadStageBytes) {
     blocks = std::min(blocks, compute_units());
-    auto kernel = token_blocks == 1 ? lm_head_stream_kernel<kHeadRing, 1> : lm_head_stream_kernel<kHeadRing, 2>;
-    static bool asked[2] = {false, false};
-    if (!asked[token_blocks - 1]) {
+    auto kernel = shaped ? (token_blocks == 1 ? lm_head_stream_kernel<kHeadRing, 1, true> : lm_head_stream_kernel<kHeadRing, 2, true>)
+                         : (token_blocks == 1 ? lm_head_stream_kernel<kHeadRing, 1> : lm_head_stream_kernel<kHeadRing, 2>);
+    static bool asked[4] = {false, false, false, false};
+    const int which = token_blocks - 1 + (shaped ? 2 : 0);
+    if (!asked[which]) {
       (void)hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize,
                                 static_cast<int>(kHeadStageBytes));
-      asked[token_blocks - 1] = true;
+      asked[which] = true;
     }
     kernel<<<blocks, 256, staged, stream>>>(static_cast<const bf16_t*>(A), static_cast<const bf16_t*>(W), C, M, N, K, lda,
-                                            ldw, ldc, cd);
+                                            ldw, ldc, cd, scale, cap);
     LYP_LAUNCH_CHECK("lm_head_stream");
     return blocks;
   }
   if (M > 16) return 0;   // beyond that the general products are ahead of lm_head_kernel
-#define LYP_HEAD(T, MB) \
-  lm_head_kernel<T, MB><<<blocks, 256, 0, stream>>>(static_cast<const T*>(A), static_cast<const T*>(W), C, M, N, K, lda, ldw, ldc, cd)
-#define LYP_HEAD_T(T)                  \
-  do {                                 \
-    if (M <= 16) LYP_HEAD(T, 1);       \
-    else if (M <= 32) LYP_HEAD(T, 2);  \
-    else if (M <= 48) LYP_HEAD(T, 3);  \
-    else LYP_HEAD(T, 4);               \
+#define LYP_HEAD(T, MB, SH) \
+  lm_head_kernel<T, MB, SH><<<blocks, 256, 0, stream>>>(static_cast<const T*>(A), static_cast<const T*>(W), C, M, N, K, lda, ldw, ldc, cd, scale, cap)
+#define LYP_HEAD_T(T)                        \
+  do {                                       \
+    if (shaped) LYP_HEAD(T, 1, true);        \
+    else LYP_HEAD(T, 1, false);              \
   } while (0)
   if (dtype == kF32) LYP_HEAD_T(float);
   else if (dtype == kBF16) LYP_HEAD_T(bf16_t);
@@ -1324,6 +1373,54 @@ extern "C" int lyp_gemm_residual(const void* A, const void* W, float* h, int dty
     LYP_REQUIRE(false, "gemm_residual: unknown dtype %d", dtype);
 #undef LYP_RESIDUAL
   LYP_LAUNCH_CHECK("gemm_residual");
+  return 0;
+}
+
+// The residual stream's next value and what the branch after it reads, from a product of few rows:
+// v = base + A . W^T goes to h (float [M, N]; null: not kept; base may be h), map(v) to xs in the
+// operands' type.  kind, alpha, w, b: stream_map.h.  Returns 1 (and does nothing) when the few-rows
+// kernel does not apply.
+extern "C" int lyp_gemm_stream(const void* A, const void* W, const float* base, int ldb, float* h, int ldh, int dtype, int M,
+                               int N, int K, int lda, int ldw, int kind, float alpha, const float* w, const float* b,
+                               void* xs, int ldx, hipStream_t stream) {
+  const StreamTail stm{base, ldb, xs, ldx, StreamMap{kind, alpha, w, b}};
+  LYP_REQUIRE(N > 0 && K > 0 && base && ldb >= N && (!h || ldh >= N) && xs && ldx >= N, "gemm_stream: N=%d K=%d", N, K);
+  LYP_REQUIRE(stream_map_ok(stm.map), "gemm_stream: map %d needs its vectors", kind);
+  if (!skinny_ok(M, K, lda, ldw, A, W, dtype)) return 1;
+  const bool paired = M <= 16 && K % 128 == 0;
+  const bool wide = residual_rows(M, N, K) == 16;
+#define LYP_STREAM(T, ROWS, PAIRED)                                                                             \
+  launch_skinny<T, kEpiStream, false, ROWS, PAIRED>(static_cast<const T*>(A), static_cast<const T*>(W), h, M, N, \
+                                                    K, lda, ldw, ldh, 1, stream, RopeTail{}, NormHead{},        \
+                                                    ResidualTail{}, stm)
+  if (dtype == kF32) {
+    if (wide) LYP_STREAM(float, 16, true);
+    else if (paired) LYP_STREAM(float, 8, true);
+    else LYP_STREAM(float, 8, false);
+  } else if (dtype == kBF16) {
+    if (wide) LYP_STREAM(bf16_t, 16, true);
+    else if (paired) LYP_STREAM(bf16_t, 8, true);
+    else LYP_STREAM(bf16_t, 8, false);
+  } else
+    LYP_REQUIRE(false, "gemm_stream: unknown dtype %d", dtype);
+#undef LYP_STREAM
+  LYP_LAUNCH_CHECK("gemm_stream");
+  return 0;
+}
+
+// out[M, N] = max(A . W^T, 0)^2 in the operands' type, for few rows; returns 1 (and does nothing) when
+// the few-rows kernel does not apply.
+extern "C" int lyp_gemm_relu2(const void* A, const void* W, void* out, int dtype, int M, int N, int K, int lda, int ldw,
+                              int ldo, hipStream_t stream) {
+  LYP_REQUIRE(N > 0 && K > 0 && ldo >= N, "gemm_relu2: N=%d K=%d stride %d", N, K, ldo);
+  if (!skinny_ok(M, K, lda, ldw, A, W, dtype)) return 1;
+  if (dtype == kF32)
+    launch_skinny_rows<float, kEpiRelu2>(static_cast<const float*>(A), static_cast<const float*>(W), out, M, N, K, lda, ldw, ldo, 1, stream);
+  else if (dtype == kBF16)
+    launch_skinny_rows<bf16_t, kEpiRelu2>(static_cast<const bf16_t*>(A), static_cast<const bf16_t*>(W), out, M, N, K, lda, ldw, ldo, 1, stream);
+  else
+    LYP_REQUIRE(false, "gemm_relu2: unknown dtype %d", dtype);
+  LYP_LAUNCH_CHECK("gemm_relu2");
   return 0;
 }
 

@@ -20,7 +20,8 @@
 //     O^T += V^T P^T       (latent dimensions x rows; a lane's accumulators all belong
 //                           to its one row, so rescaling needs no exchange)
 // with the softmax in 32-bit between them (running maximum and sum per row).
-// With one partition the kernel finishes the softmax itself, the sink included;
+// With one partition the kernel finishes the softmax itself, the sink included (a model without sinks
+// passes none: sink == nullptr);
 // with several it leaves (maximum, sum, unnormalised sums) per partition for
 // latent_combine_kernel.  The order of additions for a row depends on the
 // partition size and on the row's place in its tile only through rounding.
@@ -287,7 +288,7 @@ __global__ __launch_bounds__(256, KV <= 256 ? 2 : 1) void latent_attn_kernel(
     T* orow = out + grow * KV;
     float inv = 0.f, w = 0.f;
     if (valid) {
-      const float sk = sink[head];
+      const float sk = sink != nullptr ? sink[head] : LYP_NEG_INF;   // no sinks: nothing but the keys' weights
       const float mx = fmaxf(m, sk);
       w = expf(m - mx);
       inv = 1.0f / (l * w + expf(sk - mx));
@@ -319,7 +320,7 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(const float* __rest
   __shared__ float weight[256];   // at most 256 partitions (lyp_latent_attn checks)
   const size_t row = blockIdx.x;
   const int head = static_cast<int>(row % H);
-  const float sk = sink[head];
+  const float sk = sink != nullptr ? sink[head] : LYP_NEG_INF;
   __shared__ float denom_s;
   // the first wave, a lane a partition: maxima, weights and the denominator (partitions added in
   // lane order); then a thread a dimension
@@ -335,7 +336,8 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(const float* __rest
       part += part_ml[(row * n_parts + p) * 2 + 1] * w;
     }
     part = wave_sum(part);
-    if (threadIdx.x == 0) denom_s = part + expf(sk - mx);
+    // (a padded row without a sink has nothing at all in its denominator)
+    if (threadIdx.x == 0) denom_s = mx > LYP_NEG_INF ? part + expf(sk - mx) : 1.0f;
   }
   __syncthreads();
   const float inv = 1.0f / denom_s;
@@ -366,7 +368,7 @@ __global__ __launch_bounds__(256) void latent_heads_out_kernel(const float* __re
   if (mixed) {
     for (int d = threadIdx.x; d < KV; d += blockDim.x) rowv[d] = to_f32(mixed[row * KV + d]);
   } else {
-    const float sk = sink[head];
+    const float sk = sink != nullptr ? sink[head] : LYP_NEG_INF;
     if (threadIdx.x < kWave) {
       float mx = sk;
       for (int p = threadIdx.x; p < n_parts; p += kWave) mx = fmaxf(mx, part_ml[(row * n_parts + p) * 2]);
@@ -379,7 +381,7 @@ __global__ __launch_bounds__(256) void latent_heads_out_kernel(const float* __re
         part += part_ml[(row * n_parts + p) * 2 + 1] * wgt;
       }
       part = wave_sum(part);
-      if (threadIdx.x == 0) denom_s = part + expf(sk - mx);
+      if (threadIdx.x == 0) denom_s = mx > LYP_NEG_INF ? part + expf(sk - mx) : 1.0f;
     }
     __syncthreads();
     const float inv = 1.0f / denom_s;
@@ -445,7 +447,7 @@ int lyp_latent_heads_out(const float* part_o, const float* part_ml, const float*
                          const void* w, void* out, int dtype, int rows, int H, int n_parts, int vdim,
                          hipStream_t stream) {
   LYP_REQUIRE(rows >= 0 && H > 0 && vdim > 0 && n_parts >= 1 && n_parts <= 256, "latent_heads_out: bad sizes");
-  LYP_REQUIRE((part_o != nullptr && part_ml != nullptr && sink != nullptr) != (mixed != nullptr),
+  LYP_REQUIRE((part_o != nullptr && part_ml != nullptr) != (mixed != nullptr),
               "latent_heads_out: either the partitions or the merged rows");
   if (rows == 0) return 0;
   if (dtype == kF32)

@@ -13,8 +13,10 @@
 //              from memory for few).  GATED: rows are gathered from
 //              the step's activations by token, the gate's and the up
 //              projection's columns are computed side by side and the epilogue
-//              writes  min(g, limit) * sigmoid(alpha * min(g, limit)) * (clamp(u, -limit, limit) + 1).
+//              writes  min(g, limit) * sigmoid(alpha * min(g, limit)) * (clamp(u, -limit, limit) + plus).
 //              Otherwise rows are read by place and the product is stored.
+//   table      instead of route: a table [vocab, top] names every token id's experts, so that all layers'
+//              pairs can be sorted before the first of them runs (one launch, a workgroup a layer).
 //   combine    out[t] = addend[t] + shared[t] + sum_k weight[t, k] * y[place(t, k)],
 //              in 32-bit, in the order of k.
 //
@@ -23,7 +25,7 @@
 // the batch.
 #include <algorithm>
 
-#include "common.h"
+#include "stream_map.h"
 
 namespace lyp {
 
@@ -247,10 +249,34 @@ struct RouteFirst {
   int parts, rows, experts, top, always;
 };
 
+// TABLE: pair p is the (p % top)-th expert that a table names for token id tokens[p / top]; a workgroup
+// a layer, every layer with a table and results of its own (table_stride and out_stride numbers apart).
+struct TableChoice {
+  const int32_t* table;
+  const int32_t* tokens;
+  long long table_stride, out_stride;
+  int top;
+};
+
+template <bool TABLE>
 __global__ __launch_bounds__(kSortThreads) void moe_sort_kernel(
     int32_t* __restrict__ idx, int P, int E, int tile_rows, int32_t* __restrict__ expert_off,
     int32_t* __restrict__ sorted_pair, int32_t* __restrict__ place_of, int32_t* __restrict__ tile_expert,
-    int32_t* __restrict__ tile_row0, int32_t* __restrict__ n_tiles, RouteFirst first) {
+    int32_t* __restrict__ tile_row0, int32_t* __restrict__ n_tiles, RouteFirst first, TableChoice choice) {
+  if constexpr (TABLE) {
+    const size_t at = static_cast<size_t>(blockIdx.x) * choice.out_stride;
+    expert_off += at;
+    sorted_pair += at;
+    place_of += at;
+    tile_expert += at;
+    tile_row0 += at;
+    n_tiles += at;
+    choice.table += static_cast<size_t>(blockIdx.x) * choice.table_stride;
+  }
+  auto expert_of = [&](int p) -> int {
+    if constexpr (TABLE) return choice.table[static_cast<size_t>(choice.tokens[p / choice.top]) * choice.top + p % choice.top];
+    else return idx[p];
+  };
   extern __shared__ int32_t s_sort[];
   int32_t* cnt = s_sort;               // [E]
   int32_t* base = cnt + E;             // [E]
@@ -259,7 +285,7 @@ __global__ __launch_bounds__(kSortThreads) void moe_sort_kernel(
   const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
   int bits = 1;                       // bits that tell the experts (and -1) apart
   while ((1 << bits) <= E) ++bits;
-  if (first.part != nullptr) {
+  if (!TABLE && first.part != nullptr) {
     const int per = first.top + (first.always >= 0 ? 1 : 0);
     for (int row = wave; row < first.rows; row += kSortWaves)
       route_row(first.part + static_cast<size_t>(row) * first.experts, first.bias, first.experts, first.top,
@@ -274,7 +300,7 @@ __global__ __launch_bounds__(kSortThreads) void moe_sort_kernel(
   // places one by one is what this pass would otherwise wait for)
   for (int p0 = 0; p0 < P; p0 += kSortThreads) {
     const int p = p0 + tid;
-    const int e = p < P ? idx[p] : -1;                       // (-1: all bits set, a value no expert has)
+    const int e = p < P ? expert_of(p) : -1;                       // (-1: all bits set, a value no expert has)
     const unsigned long long mates = wave_same(e, bits);
     const bool last = (mates >> lane) == 1ull;               // no later lane holds the same expert
     if (e >= 0 && last) atomicAdd(&cnt[e], __builtin_popcountll(mates));
@@ -309,7 +335,7 @@ __global__ __launch_bounds__(kSortThreads) void moe_sort_kernel(
 #pragma unroll
       for (int a = 0; a < kAhead; ++a) {
         const int pa = p0 + a * kSortThreads + tid;
-        mine[a] = pa < P ? idx[pa] : -1;
+        mine[a] = pa < P ? expert_of(pa) : -1;
       }
     }
     __syncthreads();
@@ -530,7 +556,7 @@ __global__ __launch_bounds__(256) void moe_gemm_few_kernel(
     T* __restrict__ out, int ldo, const int32_t* __restrict__ tile_expert, const int32_t* __restrict__ tile_row0,
     const int32_t* __restrict__ n_tiles, const int32_t* __restrict__ expert_off,
     const int32_t* __restrict__ sorted_pair, int top, int N, int K, int up_offset, float limit, float alpha,
-    int vec_ok, int flags) {
+    float plus, int vec_ok, int flags) {
   using MW = Mma16Wide<T>;
   constexpr int KE = MW::kElems, STEP = 4 * KE;
   __shared__ float s_red[4][2][kWave][4];
@@ -597,7 +623,7 @@ __global__ __launch_bounds__(256) void moe_gemm_few_kernel(
       const float up = s_red[0][1][lane][i] + s_red[1][1][lane][i] + s_red[2][1][lane][i] + s_red[3][1][lane][i];
       const float g = fminf(y, limit);
       const float u = fminf(fmaxf(up, -limit), limit);
-      y = g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+      y = g / (1.0f + expf(-alpha * g)) * (u + plus);
     } else if (flags & kMoeRelu2) {
       y = fmaxf(y, 0.f);
       y *= y;
@@ -625,7 +651,7 @@ __global__ __launch_bounds__(NW * 64) void moe_gemm_wide_kernel(
     T* __restrict__ out, int ldo, const int32_t* __restrict__ tile_expert, const int32_t* __restrict__ tile_row0,
     const int32_t* __restrict__ n_tiles, const int32_t* __restrict__ expert_off,
     const int32_t* __restrict__ sorted_pair, int top, int N, int K, int up_offset, float limit, float alpha,
-    int vec_ok, int flags) {
+    float plus, int vec_ok, int flags) {
   using MW = Mma32<T>;
   constexpr int VEC = 16 / sizeof(T);
   constexpr int KT = MoeWide<T, NW>::kKT;             // inner values a round: 128 bytes of every row
@@ -785,7 +811,7 @@ __global__ __launch_bounds__(NW * 64) void moe_gemm_wide_kernel(
         if (col >= N) continue;
         const float g = fminf(acc[i][0][v], limit);
         const float u = fminf(fmaxf(acc[i][1][v], -limit), limit);
-        orow[col] = from_f32<T>(g / (1.0f + expf(-alpha * g)) * (u + 1.0f));
+        orow[col] = from_f32<T>(g / (1.0f + expf(-alpha * g)) * (u + plus));
       } else {
 #pragma unroll
         for (int j = 0; j < 2; ++j) {
@@ -818,6 +844,7 @@ __global__ void glu_clamped_kernel(const T* __restrict__ gate_up, T* __restrict_
 }
 
 // out [rows, H] float = addend + shared + sum_k wgt[row, k] * y[place_of[row * top + k]]
+// (no weights given: 1 / top each)
 // One workgroup a row; the row's places and weights are read once; a thread takes V neighbouring
 // columns at a time (V = 4 where rows are whole multiples of that, else 1), two such groups in flight.
 template <typename T, int V>
@@ -831,7 +858,7 @@ __global__ void moe_combine_kernel(const T* __restrict__ y, const int32_t* __res
   const int row = blockIdx.x;
   if (threadIdx.x < top) {
     s_at[threadIdx.x] = place_of[static_cast<size_t>(row) * top + threadIdx.x];
-    s_w[threadIdx.x] = wgt[static_cast<size_t>(row) * top + threadIdx.x];
+    s_w[threadIdx.x] = wgt != nullptr ? wgt[static_cast<size_t>(row) * top + threadIdx.x] : 1.0f / static_cast<float>(top);
   }
   __syncthreads();
   constexpr int U = 2;
@@ -875,6 +902,55 @@ __global__ void moe_combine_kernel(const T* __restrict__ y, const int32_t* __res
       else *reinterpret_cast<VecF*>(out + static_cast<size_t>(row) * H + c) = v[u];
     }
   }
+}
+
+// The weighted sum straight onto the residual stream, with what the next branch reads of it
+// (stream_map.h): v = base[row] + sum_k wgt[row, k] * y[place_of[row * top + k]], v to h (where given),
+// map(v) to out.  A thread takes V neighbouring columns; blockIdx.y walks the row.
+template <typename T, int V>
+__global__ __launch_bounds__(256) void moe_combine_stream_kernel(const T* __restrict__ y, const int32_t* __restrict__ place_of,
+                                                                 const float* __restrict__ wgt, int top, float* h,
+                                                                 const float* base, StreamMap map, T* __restrict__ out,
+                                                                 int H) {
+  typedef T VecT __attribute__((ext_vector_type(V)));
+  typedef float VecF __attribute__((ext_vector_type(V)));
+  const int row = blockIdx.x;
+  const int c = (blockIdx.y * blockDim.x + threadIdx.x) * V;
+  if (c >= H) return;
+  const size_t at = static_cast<size_t>(row) * H + c;
+  const VecF x = *reinterpret_cast<const VecF*>(base + at);
+  VecF w, b, sum;
+#pragma unroll
+  for (int i = 0; i < V; ++i) w[i] = b[i] = sum[i] = 0.f;
+  if (map.kind == kMapTanh) {
+    w = *reinterpret_cast<const VecF*>(map.w + c);
+    b = *reinterpret_cast<const VecF*>(map.b + c);
+  }
+  constexpr int U = 4;   // choices whose loads are in flight together; added in their order
+  for (int k0 = 0; k0 < top; k0 += U) {
+    VecT v[U];
+    float wk[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int k = min(k0 + u, top - 1);
+      wk[u] = wgt != nullptr ? wgt[static_cast<size_t>(row) * top + k] : 1.0f / static_cast<float>(top);
+      v[u] = *reinterpret_cast<const VecT*>(y + static_cast<size_t>(place_of[static_cast<size_t>(row) * top + k]) * H + c);
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      if (k0 + u >= top) continue;
+#pragma unroll
+      for (int i = 0; i < V; ++i) sum[i] += wk[u] * to_f32(v[u][i]);
+    }
+  }
+  VecF s;
+#pragma unroll
+  for (int i = 0; i < V; ++i) s[i] = x[i] + sum[i];
+  if (h != nullptr) *reinterpret_cast<VecF*>(h + at) = s;
+  VecT o;
+#pragma unroll
+  for (int i = 0; i < V; ++i) o[i] = from_f32<T>(map_feature(map.kind, map.alpha, s[i], w[i], b[i]));
+  *reinterpret_cast<VecT*>(out + at) = o;
 }
 
 }  // namespace lyp
@@ -996,9 +1072,10 @@ int lyp_moe_sort(const int32_t* idx, int pairs, int E, int tile_rows, int32_t* e
   LYP_REQUIRE(pairs >= 0 && E > 0 && E <= kMostExperts && (tile_rows == 16 || tile_rows == 128),
               "moe_sort: %d pairs, %d experts, tiles of %d rows", pairs, E, tile_rows);
   const size_t lds = sizeof(int32_t) * (3 * E + 1 + kSortWaves * E);
-  moe_sort_kernel<<<1, kSortThreads, lds, stream>>>(const_cast<int32_t*>(idx), pairs, E, tile_rows, expert_off,
-                                                    sorted_pair, place_of, tile_expert, tile_row0, n_tiles,
-                                                    RouteFirst{nullptr, nullptr, nullptr, 0, 0, 0, 0, -1});
+  moe_sort_kernel<false><<<1, kSortThreads, lds, stream>>>(const_cast<int32_t*>(idx), pairs, E, tile_rows, expert_off,
+                                                           sorted_pair, place_of, tile_expert, tile_row0, n_tiles,
+                                                           RouteFirst{nullptr, nullptr, nullptr, 0, 0, 0, 0, -1},
+                                                           TableChoice{});
   LYP_LAUNCH_CHECK("moe_sort");
   return 0;
 }
@@ -1016,10 +1093,32 @@ int lyp_moe_route_sort(const float* part, int parts, const float* bias, int rows
   LYP_REQUIRE(E >= experts && E <= kMostExperts && (tile_rows == 16 || tile_rows == 128),
               "moe_route_sort: %d matrices, tiles of %d rows", E, tile_rows);
   const size_t lds = sizeof(int32_t) * (3 * E + 1 + kSortWaves * E);
-  moe_sort_kernel<<<1, kSortThreads, lds, stream>>>(idx, pairs, E, tile_rows, expert_off, sorted_pair, place_of,
-                                                    tile_expert, tile_row0, n_tiles,
-                                                    RouteFirst{part, bias, wgt, parts, rows, experts, top, always});
+  moe_sort_kernel<false><<<1, kSortThreads, lds, stream>>>(idx, pairs, E, tile_rows, expert_off, sorted_pair, place_of,
+                                                           tile_expert, tile_row0, n_tiles,
+                                                           RouteFirst{part, bias, wgt, parts, rows, experts, top, always},
+                                                           TableChoice{});
   LYP_LAUNCH_CHECK("moe_route_sort");
+  return 0;
+}
+
+// The same for `layers` layers at once whose experts a table names by token id: tables [layers][vocab][top],
+// tokens [rows] (ids below vocab; the tables hold experts below E: the caller has checked both).  Every
+// result is the first layer's; layer i's stand i * out_stride numbers further on.
+int lyp_moe_sort_tables(const int32_t* tables, long long table_stride, const int32_t* tokens, int layers, int rows, int top,
+                        int E, int tile_rows, int32_t* expert_off, int32_t* sorted_pair, int32_t* place_of,
+                        int32_t* tile_expert, int32_t* tile_row0, int32_t* n_tiles, long long out_stride,
+                        hipStream_t stream) {
+  LYP_REQUIRE(layers >= 0 && rows >= 0 && top > 0 && top <= E && top <= kMostTop && E <= kMostExperts &&
+                  (tile_rows == 16 || tile_rows == 128),
+              "moe_sort_tables: %d layers, %d rows, %d of %d experts, tiles of %d rows", layers, rows, top, E, tile_rows);
+  const long long pairs = static_cast<long long>(rows) * top;
+  LYP_REQUIRE(pairs < (1LL << 31) && out_stride >= 0 && table_stride >= 0, "moe_sort_tables: %lld pairs", pairs);
+  if (layers == 0 || rows == 0) return 0;
+  const size_t lds = sizeof(int32_t) * (3 * E + 1 + kSortWaves * E);
+  moe_sort_kernel<true><<<layers, kSortThreads, lds, stream>>>(
+      nullptr, static_cast<int>(pairs), E, tile_rows, expert_off, sorted_pair, place_of, tile_expert, tile_row0, n_tiles,
+      RouteFirst{nullptr, nullptr, nullptr, 0, 0, 0, 0, -1}, TableChoice{tables, tokens, table_stride, out_stride, top});
+  LYP_LAUNCH_CHECK("moe_sort_tables");
   return 0;
 }
 
@@ -1029,7 +1128,7 @@ int lyp_moe_route_sort(const float* part, int parts, const float* bias, int rows
 int lyp_moe_gemm(const void* a, int lda, const void* w, long long w_expert_stride, int ldw, void* out, int ldo,
                  int dtype, int gated, const int32_t* tile_expert, const int32_t* tile_row0, const int32_t* n_tiles,
                  int most_tiles, int tile_rows, const int32_t* expert_off, const int32_t* sorted_pair, int top, int N,
-                 int K, float limit, float alpha, int flags, hipStream_t stream) {
+                 int K, float limit, float alpha, float plus, int flags, hipStream_t stream) {
   LYP_REQUIRE(N > 0 && K > 0 && lda >= K && ldw >= K && ldo >= N && top > 0 && most_tiles >= 0,
               "moe_gemm: bad sizes N=%d K=%d lda=%d ldw=%d ldo=%d", N, K, lda, ldw, ldo);
   LYP_REQUIRE(tile_rows == 16 || tile_rows == 128, "moe_gemm: tiles of %d rows", tile_rows);
@@ -1060,11 +1159,11 @@ int lyp_moe_gemm(const void* a, int lda, const void* w, long long w_expert_strid
   }                                                                                                             \
   moe_gemm_wide_kernel<T, G, NWV><<<grid, NWV * 64, MoeWide<T, NWV>::kBytes, stream>>>(                         \
       static_cast<const T*>(a), lda, static_cast<const T*>(w), w_expert_stride, ldw, static_cast<T*>(out), ldo, \
-      tile_expert, tile_row0, n_tiles, expert_off, sorted_pair, top, N, K, N, limit, alpha, vec_ok, flags)
+      tile_expert, tile_row0, n_tiles, expert_off, sorted_pair, top, N, K, N, limit, alpha, plus, vec_ok, flags)
 #define LYP_MOE_FEW(T, G)                                                                                       \
   moe_gemm_few_kernel<T, G><<<grid, 256, 0, stream>>>(                                                          \
       static_cast<const T*>(a), lda, static_cast<const T*>(w), w_expert_stride, ldw, static_cast<T*>(out), ldo, \
-      tile_expert, tile_row0, n_tiles, expert_off, sorted_pair, top, N, K, N, limit, alpha, vec_ok, flags)
+      tile_expert, tile_row0, n_tiles, expert_off, sorted_pair, top, N, K, N, limit, alpha, plus, vec_ok, flags)
 #define LYP_MOE_T(T)                                 \
   do {                                               \
     if (few) {                                       \
@@ -1127,6 +1226,36 @@ int lyp_moe_combine(const void* y, const int32_t* place_of, const float* wgt, in
   }
 #undef LYP_COMBINE
   LYP_LAUNCH_CHECK("moe_combine");
+  return 0;
+}
+
+// y [pairs, H] of dtype by place; wgt float [rows, top] or null (1 / top each); base float [rows, H];
+// h float [rows, H] (may be base) or null; out [rows, H] of dtype; kind, alpha, w, b: stream_map.h.
+int lyp_moe_combine_stream(const void* y, const int32_t* place_of, const float* wgt, int top, float* h, const float* base,
+                           int kind, float alpha, const float* w, const float* b, void* out, int dtype, int rows, int H,
+                           hipStream_t stream) {
+  const StreamMap map{kind, alpha, w, b};
+  LYP_REQUIRE(rows >= 0 && H > 0 && top > 0 && top <= kMostTop && base != nullptr && out != nullptr && stream_map_ok(map),
+              "moe_combine_stream: %d rows of %d, %d choices, map %d", rows, H, top, kind);
+  if (rows == 0) return 0;
+  auto aligned = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+  const bool vec = H % 4 == 0 && aligned(y) && aligned(h) && aligned(base) && aligned(w) && aligned(b) && aligned(out);
+  const int per = vec ? 4 : 1;
+  const dim3 grid(rows, (H + 256 * per - 1) / (256 * per));
+#define LYP_COMBINE_STREAM(T, V)                                                                                    \
+  moe_combine_stream_kernel<T, V><<<grid, 256, 0, stream>>>(static_cast<const T*>(y), place_of, wgt, top, h, base,  \
+                                                            map, static_cast<T*>(out), H)
+  if (dtype == kF32) {
+    if (vec) LYP_COMBINE_STREAM(float, 4);
+    else LYP_COMBINE_STREAM(float, 1);
+  } else if (dtype == kBF16) {
+    if (vec) LYP_COMBINE_STREAM(bf16_t, 4);
+    else LYP_COMBINE_STREAM(bf16_t, 1);
+  } else {
+    LYP_REQUIRE(false, "moe_combine_stream: unknown dtype %d", dtype);
+  }
+#undef LYP_COMBINE_STREAM
+  LYP_LAUNCH_CHECK("moe_combine_stream");
   return 0;
 }
 

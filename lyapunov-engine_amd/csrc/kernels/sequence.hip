@@ -1,7 +1,7 @@
 // Row-wise and time-wise kernels for layers that norm a branch before it joins
 // the residual stream, filter a branch's input over time, or carry a
 // recurrence: the joining norm, a short causal convolution with its state, the
-// minGRU scan, the xIELU / tanh-GELU activations, and what a latent attention
+// minGRU scan, the xIELU / tanh-GELU / squared-relu activations, and what a latent attention
 // layer does around its products (norms of the latents, rotation of
 // neighbouring pairs, the write of a token's latent into its page slot).
 //
@@ -358,7 +358,7 @@ __global__ void short_conv_vec_kernel(const T* __restrict__ x, const float* __re
 // ------------------------------------------------------------- activations
 __device__ __forceinline__ float softplus_f(float v) { return v > 20.f ? v : log1pf(expf(v)); }
 
-enum Activation : int { kXielu = 0, kGeluTanh = 1 };
+enum Activation : int { kXielu = 0, kGeluTanh = 1, kRelu2 = 2 };
 
 // xIELU with two learned numbers p, q (params[0], params[1]):
 //   z > 0:  softplus(p) z^2 + z/2      z <= 0:  (1/2 + softplus(q)) (e^z - 1 - z) + z/2
@@ -367,6 +367,14 @@ __device__ __forceinline__ float xielu_f(float z, float ap, float aq) {
 }
 __device__ __forceinline__ float gelu_tanh_f(float z) {
   return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
+
+__device__ __forceinline__ float activate(int kind, float z, float ap, float aq) {
+  if (kind == kRelu2) {
+    const float y = fmaxf(z, 0.f);
+    return y * y;
+  }
+  return kind == kXielu ? xielu_f(z, ap, aq) : gelu_tanh_f(z);
 }
 
 // vec: 16 bytes a thread and turn; n is then a multiple of the vector's length and the operands are aligned
@@ -387,7 +395,7 @@ __global__ void activation_kernel(const T* __restrict__ in, T* __restrict__ out,
 #pragma unroll
       for (int e = 0; e < VEC; ++e) {
         const float z = to_f32(v[e]);
-        v[e] = from_f32<T>(kind == kXielu ? xielu_f(z, ap, aq) : gelu_tanh_f(z));
+        v[e] = from_f32<T>(activate(kind, z, ap, aq));
       }
       reinterpret_cast<VecT*>(out)[i] = v;
     }
@@ -395,7 +403,7 @@ __global__ void activation_kernel(const T* __restrict__ in, T* __restrict__ out,
   }
   for (size_t i = blockIdx.x * static_cast<size_t>(blockDim.x) + threadIdx.x; i < n; i += stride) {
     const float z = to_f32(in[i]);
-    out[i] = from_f32<T>(kind == kXielu ? xielu_f(z, ap, aq) : gelu_tanh_f(z));
+    out[i] = from_f32<T>(activate(kind, z, ap, aq));
   }
 }
 
@@ -592,11 +600,91 @@ __global__ void latent_query_rotate_kernel(const T* __restrict__ q, const int32_
   }
 }
 
+// For a layer whose queries come straight from its input: x [rows, ld] holds per token the queries of
+// all heads (H times dim plain values, then rot_dim to rotate), the key/value latent (kv_rank) and the
+// shared rotated key part (rot_dim), side by side as one product leaves them.  blockIdx.y == 0 norms
+// the latent, rotates the key part and writes both to the token's page slot; the other blocks rotate
+// the queries' parts into qa[row, head, kv_rank ..].  PAIR: rows in which every pair of values can be
+// read and written as one.
+template <typename T, bool PAIR>
+__global__ __launch_bounds__(256) void latent_direct_prep_kernel(
+    const T* __restrict__ x, int ld, const float* __restrict__ wkv, const int32_t* __restrict__ positions,
+    const float* __restrict__ table, int dims, const int32_t* __restrict__ slot_map, T* __restrict__ qa,
+    T* __restrict__ pages, int H, int dim, int kv_rank, int rot_dim, float eps) {
+  typedef T Two __attribute__((ext_vector_type(2)));
+  __shared__ float scratch[16];
+  const int t = blockIdx.x;
+  const T* row = x + static_cast<size_t>(t) * ld;
+  const int half = dims / 2, per = (rot_dim + 1) / 2;
+  const float* cs = table + static_cast<size_t>(positions[t]) * dims;
+  auto two = [&](const T* p, bool both, float& a, float& b) {
+    if constexpr (PAIR) {
+      const Two v = *reinterpret_cast<const Two*>(p);
+      a = to_f32(v[0]);
+      b = to_f32(v[1]);
+    } else {
+      a = to_f32(p[0]);
+      b = both ? to_f32(p[1]) : 0.f;
+    }
+  };
+  auto put = [&](T* p, bool both, float a, float b) {
+    if constexpr (PAIR) {
+      Two v;
+      v[0] = from_f32<T>(a);
+      v[1] = from_f32<T>(b);
+      *reinterpret_cast<Two*>(p) = v;
+    } else {
+      p[0] = from_f32<T>(a);
+      if (both) p[1] = from_f32<T>(b);
+    }
+  };
+  auto turned = [&](const T* src, T* dst, int i) {   // pair i of a part to rotate; pairs past the rotated ones pass
+    const bool both = 2 * i + 1 < rot_dim;
+    float a, b;
+    two(src + 2 * i, both, a, b);
+    if (i < half) {
+      float y1, y2;
+      rotate_pair(a, b, cs[i], cs[half + i], y1, y2);
+      a = y1;
+      b = y2;
+    }
+    put(dst + 2 * i, both, a, b);
+  };
+  const int wide = dim + rot_dim, DK = kv_rank + rot_dim;
+  if (blockIdx.y > 0) {
+    const int n = H * per, step = (gridDim.y - 1) * blockDim.x;
+    for (int idx = (blockIdx.y - 1) * blockDim.x + threadIdx.x; idx < n; idx += step) {
+      const int h = idx / per;
+      turned(row + h * wide + dim, qa + (static_cast<size_t>(t) * H + h) * DK + kv_rank, idx % per);
+    }
+    return;
+  }
+  const int slot = slot_map[t];
+  if (slot < 0) return;   // a padded row (the whole workgroup leaves)
+  const T* c = row + static_cast<size_t>(H) * wide;
+  T* prow = pages + static_cast<size_t>(slot) * DK;
+  for (int i = threadIdx.x; i < per; i += blockDim.x) turned(c + kv_rank, prow + kv_rank, i);
+  const int pairs = (kv_rank + 1) / 2;
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < pairs; i += blockDim.x) {
+    float a, b;
+    two(c + 2 * i, 2 * i + 1 < kv_rank, a, b);
+    ss += a * a + b * b;
+  }
+  const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / static_cast<float>(kv_rank) + eps);
+  for (int i = threadIdx.x; i < pairs; i += blockDim.x) {
+    const bool both = 2 * i + 1 < kv_rank;
+    float a, b;
+    two(c + 2 * i, both, a, b);
+    put(prow + 2 * i, both, (a * inv) * wkv[2 * i], both ? (b * inv) * wkv[2 * i + 1] : 0.f);
+  }
+}
+
 // Attention of every row of the step over its request's latents in the pages,
 // one shared key per token for all heads: key = the page row (Dk = kv_rank +
 // rot_dim values), value = its first kv_rank values.  One workgroup per (row,
 // head); blocks of keys: a thread a key for the scores, a thread a value column
-// for the sums.  The softmax's denominator also holds exp(sink[head]).
+// for the sums.  The softmax's denominator also holds exp(sink[head]) where there are sinks.
 // Sizes are run-time values; this is the kernel for sizes the matrix-core
 // kernel does not take.
 constexpr int kLatentBlock = 128;
@@ -629,7 +717,8 @@ __global__ __launch_bounds__(kLatentBlock) void latent_attn_rows_kernel(
   float acc[kCols];
 #pragma unroll
   for (int v = 0; v < kCols; ++v) acc[v] = 0.f;
-  float m = sink[h], l = 1.0f;      // the sink: a score without key or value
+  // the sink: a score without key or value (no sinks: nothing yet in the denominator)
+  float m = sink != nullptr ? sink[h] : LYP_NEG_INF, l = sink != nullptr ? 1.0f : 0.f;
   for (int k0 = 0; k0 < n_keys; k0 += kLatentBlock) {
     const int j = k0 + threadIdx.x;
     float s = LYP_NEG_INF;
@@ -644,7 +733,7 @@ __global__ __launch_bounds__(kLatentBlock) void latent_attn_rows_kernel(
     }
     const float m_new = fmaxf(m, block_max(s, scratch));
     const float p = s > LYP_NEG_INF ? expf(s - m_new) : 0.f;
-    const float rescale = expf(m - m_new);
+    const float rescale = m_new > LYP_NEG_INF ? expf(m - m_new) : 1.0f;
     const float psum = block_sum(p, scratch);
     l = l * rescale + psum;
     m = m_new;
@@ -667,7 +756,7 @@ __global__ __launch_bounds__(kLatentBlock) void latent_attn_rows_kernel(
       }
     }
   }
-  const float inv = 1.0f / l;
+  const float inv = l > 0.f ? 1.0f / l : 0.f;
 #pragma unroll
   for (int v = 0; v < kCols; ++v) {
     const int col = threadIdx.x + v * kLatentBlock;
@@ -795,7 +884,7 @@ int lyp_short_conv(const void* x, const float* w, void* state, const int32_t* q_
 
 int lyp_activation(const void* in, void* out, int dtype, long long n, int kind, const float* params,
                    hipStream_t stream) {
-  LYP_REQUIRE(n >= 0 && (kind == kXielu || kind == kGeluTanh), "activation: n=%lld kind=%d", n, kind);
+  LYP_REQUIRE(n >= 0 && (kind == kXielu || kind == kGeluTanh || kind == kRelu2), "activation: n=%lld kind=%d", n, kind);
   LYP_REQUIRE(kind != kXielu || params != nullptr, "activation: xIELU needs its two numbers");
   if (n == 0) return 0;
   const int per = dtype == kF32 ? 4 : 8;
@@ -879,6 +968,43 @@ int lyp_latent_prep(const void* d, int ld, const float* wq, const float* wkv, co
   else LYP_REQUIRE(false, "latent_prep: unknown dtype %d", dtype);
 #undef LYP_PREP
   LYP_LAUNCH_CHECK("latent_prep");
+  return 0;
+}
+
+// x [rows, ld] of dtype: H (dim + rot_dim) query values, kv_rank of the latent, rot_dim of the key part;
+// qa [rows, H, kv_rank + rot_dim], pages [slots, kv_rank + rot_dim] of dtype.
+int lyp_latent_direct_prep(const void* x, int ld, const float* wkv, const int32_t* positions, const float* table, int dims,
+                           const int32_t* slot_map, void* qa, void* pages, int dtype, int n_rows, int H, int dim,
+                           int kv_rank, int rot_dim, float eps, hipStream_t stream) {
+  LYP_REQUIRE(n_rows >= 0 && H > 0 && dim >= 0 && kv_rank > 0 && rot_dim >= 0 &&
+                  ld >= static_cast<long long>(H) * (dim + rot_dim) + kv_rank + rot_dim,
+              "latent_direct_prep: bad sizes rows=%d heads=%d dim=%d kv_rank=%d rot=%d ld=%d", n_rows, H, dim, kv_rank,
+              rot_dim, ld);
+  LYP_REQUIRE(dims >= 0 && dims % 2 == 0 && dims <= rot_dim && (dims == 0 || table != nullptr),
+              "latent_direct_prep: %d rotated dimensions of %d", dims, rot_dim);
+  if (n_rows == 0) return 0;
+  const size_t esz = dtype == kF32 ? 4 : 2;
+  const bool pair = ld % 2 == 0 && dim % 2 == 0 && kv_rank % 2 == 0 && rot_dim % 2 == 0 &&
+                    reinterpret_cast<uintptr_t>(x) % (2 * esz) == 0 && reinterpret_cast<uintptr_t>(qa) % (2 * esz) == 0 &&
+                    reinterpret_cast<uintptr_t>(pages) % (2 * esz) == 0;
+  const int work = H * ((rot_dim + 1) / 2);      // pairs of the queries; up to four a thread
+  const int threads = kv_rank >= 512 ? 256 : (kv_rank >= 256 ? 128 : 64);
+  const dim3 grid(n_rows, 1 + (work + 4 * threads - 1) / (4 * threads));
+#define LYP_DIRECT(T, P)                                                                                              \
+  latent_direct_prep_kernel<T, P><<<grid, threads, 0, stream>>>(static_cast<const T*>(x), ld, wkv, positions, table,  \
+                                                                dims, slot_map, static_cast<T*>(qa),                  \
+                                                                static_cast<T*>(pages), H, dim, kv_rank, rot_dim, eps)
+  if (dtype == kF32) {
+    if (pair) LYP_DIRECT(float, true);
+    else LYP_DIRECT(float, false);
+  } else if (dtype == kBF16) {
+    if (pair) LYP_DIRECT(bf16_t, true);
+    else LYP_DIRECT(bf16_t, false);
+  } else {
+    LYP_REQUIRE(false, "latent_direct_prep: unknown dtype %d", dtype);
+  }
+#undef LYP_DIRECT
+  LYP_LAUNCH_CHECK("latent_direct_prep");
   return 0;
 }
 

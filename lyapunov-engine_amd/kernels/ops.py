@@ -77,7 +77,7 @@ def core() -> ctypes.CDLL:
         lib.lyp_sample_cand.argtypes = [c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                         c_int, c_void_p, c_void_p, c_void_p]
         lib.lyp_lm_head.argtypes = [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
-                                    c_void_p, c_int, c_void_p]
+                                    c_void_p, c_int, c_float, c_float, c_void_p]
         lib.lyp_sample_workspace.argtypes = [c_int]
         lib.lyp_sample_workspace.restype = c_longlong
         lib.lyp_norm_threads_override.argtypes = [c_int]
@@ -126,7 +126,20 @@ def core() -> ctypes.CDLL:
                                      c_void_p, c_void_p]
         lib.lyp_moe_gemm.argtypes = [c_void_p, c_int, c_void_p, c_longlong, c_int, c_void_p, c_int, c_int, c_int,
                                      c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int,
-                                     c_float, c_float, c_int, c_void_p]
+                                     c_float, c_float, c_float, c_int, c_void_p]
+        lib.lyp_moe_sort_tables.argtypes = [c_void_p, c_longlong, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p,
+                                            c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_longlong, c_void_p]
+        lib.lyp_moe_combine_stream.argtypes = [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_float,
+                                               c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p]
+        lib.lyp_stream_map.argtypes = [c_void_p, c_void_p, c_void_p, c_int, c_int, c_longlong, c_int, c_float, c_void_p,
+                                       c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p]
+        lib.lyp_logit_cap.argtypes = [c_void_p, c_longlong, c_float, c_float, c_void_p]
+        lib.lyp_gemm_stream.argtypes = [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int,
+                                        c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p]
+        lib.lyp_gemm_relu2.argtypes = [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
+                                       c_void_p]
+        lib.lyp_latent_direct_prep.argtypes = [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
+                                               c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p]
         lib.lyp_glu_clamped.argtypes = [c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_float, c_void_p]
         lib.lyp_moe_combine.argtypes = [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int,
                                         c_int, c_void_p]
@@ -844,9 +857,21 @@ LM_HEAD_MAX_ROWS = 32     # what the output-head kernels may take (the library c
 LM_HEAD_BLOCKS = 1024     # most workgroups of the output-head kernels (the library says how many it used)
 
 
-def lm_head(x: torch.Tensor, w: torch.Tensor) -> tuple:
+def logit_cap(z: torch.Tensor, scale: float = 1.0, cap: float = 0.0) -> torch.Tensor:
+    """z <- cap * tanh(scale * z / cap) (cap 0: scale * z), float logits in place."""
+    _dev(z)
+    _f32(z)
+    if cap < 0:
+        raise KernelError(f"logit_cap: a cap of {cap}")
+    lib = core()
+    _check(lib.lyp_logit_cap(_p(z), z.numel(), float(scale), float(cap), _stream()), lib)
+    return z
+
+
+def lm_head(x: torch.Tensor, w: torch.Tensor, scale: float = 1.0, cap: float = 0.0) -> tuple:
     """-> (float logits x @ w.T for the output head [vocab, hidden], row maxima
-    or None).  Few rows (a decode step's) take a kernel of their own that reads
+    or None).  ``scale`` and ``cap`` shape every logit as ``logit_cap`` does, before the maxima are
+    taken.  Few rows (a decode step's) take a kernel of their own that reads
     the matrix with few long-lived waves and leaves, beside the logits, every
     workgroup's largest logit per row: an int32 tensor [rows, workgroups, 2] of
     (value bits, index) pairs, which ``sample`` takes as ``row_maxima`` instead
@@ -859,12 +884,13 @@ def lm_head(x: torch.Tensor, w: torch.Tensor) -> tuple:
         out = torch.empty((M, V), dtype=torch.float32, device=x.device)
         cand = torch.empty((M, LM_HEAD_BLOCKS, 2), dtype=torch.int32, device=x.device)
         rc = lib.lyp_lm_head(_p(x), _p(w), _p(out), _code(x.dtype), M, V, K, x.stride(0), w.stride(0), out.stride(0),
-                             _p(cand), LM_HEAD_BLOCKS, _stream())
+                             _p(cand), LM_HEAD_BLOCKS, float(scale), float(cap), _stream())
         if rc < 0:
             _check(rc, lib)
         if rc > 0:
             return out, (cand if rc == LM_HEAD_BLOCKS else cand.view(-1)[:M * rc * 2].view(M, rc, 2))
-    return linear(x, w, out_dtype=torch.float32), None
+    out = linear(x, w, out_dtype=torch.float32)
+    return out if scale == 1.0 and cap == 0.0 else logit_cap(out, scale, cap), None
 
 
 def sum_parts(parts: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
@@ -1001,13 +1027,13 @@ def short_conv(x: torch.Tensor, w: torch.Tensor, state: torch.Tensor | None, q_s
     return out
 
 
-ACTIVATIONS = {"xielu": 0, "gelu_tanh": 1}
+ACTIVATIONS = {"xielu": 0, "gelu_tanh": 1, "relu2": 2}
 
 
 def activation(x: torch.Tensor, kind: str, params: torch.Tensor | None = None,
                out: torch.Tensor | None = None) -> torch.Tensor:
-    """Elementwise activation in 32-bit: "xielu" (params: its two learned numbers, float) or
-    "gelu_tanh".  In place unless ``out`` is given."""
+    """Elementwise activation in 32-bit: "xielu" (params: its two learned numbers, float),
+    "gelu_tanh" or "relu2" (max(z, 0)^2).  In place unless ``out`` is given."""
     out = x if out is None else out
     _dev(x, params, out)
     _f32(params)
@@ -1017,6 +1043,22 @@ def activation(x: torch.Tensor, kind: str, params: torch.Tensor | None = None,
     lib = core()
     _check(lib.lyp_activation(_p(x), _p(out), _code(x.dtype), x.numel(), ACTIVATIONS[kind], _p(params), _stream()), lib)
     return out
+
+
+def linear_relu2(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """max(x @ w.T, 0)^2 in x's type.  With few rows the product's kernel does it on its way out."""
+    M, K = x.shape
+    if w.shape[1] == K and _few_rows_product(M, w, x.dtype):
+        _dev(x, w)
+        out = torch.empty((M, w.shape[0]), dtype=x.dtype, device=x.device)
+        lib = core()
+        rc = lib.lyp_gemm_relu2(_p(x), _p(w), _p(out), _code(x.dtype), M, w.shape[0], K, x.stride(0), w.stride(0),
+                                out.stride(0), _stream())
+        if rc < 0:
+            _check(rc, lib)
+        if rc == 0:
+            return out
+    return activation(linear(x, w, out_dtype=x.dtype), "relu2")
 
 
 def mingru_scan(pre: torch.Tensor, bz: torch.Tensor, bx: torch.Tensor, state: torch.Tensor, q_start: torch.Tensor,
@@ -1073,6 +1115,26 @@ def latent_prep(d: torch.Tensor, wq: torch.Tensor, wkv: torch.Tensor, positions:
                                _stream()), lib)
 
 
+def latent_direct_prep(x: torch.Tensor, wkv: torch.Tensor, positions: torch.Tensor, table: torch.Tensor | None,
+                       slot_map: torch.Tensor, qa: torch.Tensor, pages: torch.Tensor, *, num_heads: int, dim: int,
+                       kv_rank: int, rot_dim: int, eps: float) -> None:
+    """From one product's rows (x [T, H (dim + rot_dim) + kv_rank + rot_dim]: the queries of all heads, the
+    key/value latent, the shared key part): the queries' position-rotated parts into qa[:, head, kv_rank:]
+    (qa [T, H, kv_rank + rot_dim]), and the normed latent with the rotated key part into each token's page
+    slot (pages [pages, page size, kv_rank + rot_dim])."""
+    _dev(x, wkv, positions, table, slot_map, qa, pages)
+    _f32(wkv, table)
+    T, H = x.shape[0], num_heads
+    dims = 0 if table is None else table.shape[1]
+    if x.shape[1] != H * (dim + rot_dim) + kv_rank + rot_dim or tuple(qa.shape) != (T, H, kv_rank + rot_dim) or \
+            qa.dtype != x.dtype or pages.dtype != x.dtype or pages.dim() != 3 or pages.shape[2] != kv_rank + rot_dim or \
+            wkv.numel() != kv_rank or positions.numel() != T or slot_map.numel() != T or dims > rot_dim:
+        raise KernelError(f"latent_direct_prep: x {tuple(x.shape)}, qa {tuple(qa.shape)}, pages {tuple(pages.shape)}")
+    lib = core()
+    _check(lib.lyp_latent_direct_prep(_p(x), x.stride(0), _p(wkv), _p(positions), _p(table), dims, _p(slot_map), _p(qa),
+                                      _p(pages), _code(x.dtype), T, H, dim, kv_rank, rot_dim, float(eps), _stream()), lib)
+
+
 def latent_query_rotate(q: torch.Tensor, positions: torch.Tensor, table: torch.Tensor | None, qa: torch.Tensor, *,
                         num_heads: int, dim: int, rot_dim: int, kv_rank: int) -> None:
     """The rotated part of every query head (q [T, H (dim + rot_dim)], the last rot_dim of each head),
@@ -1090,17 +1152,17 @@ def latent_query_rotate(q: torch.Tensor, positions: torch.Tensor, table: torch.T
 
 
 def latent_attn_rows(qa: torch.Tensor, pages: torch.Tensor, block_tables: torch.Tensor, q_start: torch.Tensor,
-                     positions: torch.Tensor, ctx_len: torch.Tensor, sink: torch.Tensor, scale: float,
+                     positions: torch.Tensor, ctx_len: torch.Tensor, sink: torch.Tensor | None, scale: float,
                      out: torch.Tensor, *, kv_rank: int, rot_dim: int) -> torch.Tensor:
     """Causal attention of every row over its request's latents in the pages, all heads sharing one
     key per token (the page row) whose first kv_rank values are also the value; the softmax's
-    denominator holds exp(sink[head]) as well.  Any sizes; a workgroup per (row, head)."""
+    denominator holds exp(sink[head]) as well (``sink`` None: nothing more).  Any sizes; a workgroup per (row, head)."""
     _dev(qa, pages, block_tables, q_start, positions, ctx_len, sink, out)
     _f32(sink)
     T, H, Dk = qa.shape
     B = ctx_len.numel()
     if Dk != kv_rank + rot_dim or pages.dim() != 3 or pages.shape[2] != Dk or pages.dtype != qa.dtype or \
-            tuple(out.shape) != (T, H, kv_rank) or out.dtype != qa.dtype or sink.numel() != H or \
+            tuple(out.shape) != (T, H, kv_rank) or out.dtype != qa.dtype or (sink is not None and sink.numel() != H) or \
             block_tables.dtype != torch.int32 or block_tables.dim() != 2 or block_tables.shape[0] != B or \
             q_start.numel() != B + 1 or positions.numel() != T:
         raise KernelError(f"latent_attn_rows: qa {tuple(qa.shape)}, pages {tuple(pages.shape)}, out {tuple(out.shape)}")
@@ -1154,7 +1216,7 @@ def latent_attn_launch(T: int, B: int, H: int, max_ctx: int, dtype: torch.dtype,
 
 
 def latent_attn(qa: torch.Tensor, pages: torch.Tensor, block_tables: torch.Tensor, q_start: torch.Tensor,
-                positions: torch.Tensor, ctx_len: torch.Tensor, sink: torch.Tensor, scale: float, out: torch.Tensor,
+                positions: torch.Tensor, ctx_len: torch.Tensor, sink: torch.Tensor | None, scale: float, out: torch.Tensor,
                 launch: dict, part_o: torch.Tensor | None = None, part_ml: torch.Tensor | None = None, *,
                 kv_rank: int, rot_dim: int, merge: bool = True) -> torch.Tensor:
     """``latent_attn_rows`` on the matrix cores (sizes in multiples of 16), a prompt's rows and
@@ -1167,7 +1229,7 @@ def latent_attn(qa: torch.Tensor, pages: torch.Tensor, block_tables: torch.Tenso
     T, H, Dk = qa.shape
     B = ctx_len.numel()
     if Dk != kv_rank + rot_dim or pages.dim() != 3 or pages.shape[2] != Dk or pages.dtype != qa.dtype or \
-            tuple(out.shape) != (T, H, kv_rank) or out.dtype != qa.dtype or sink.numel() != H or \
+            tuple(out.shape) != (T, H, kv_rank) or out.dtype != qa.dtype or (sink is not None and sink.numel() != H) or \
             block_tables.dtype != torch.int32 or block_tables.dim() != 2 or block_tables.shape[0] != B or \
             q_start.numel() != B + 1 or positions.numel() != T or launch["row_groups"] < -(-T * H // 64) + B:
         raise KernelError(f"latent_attn: qa {tuple(qa.shape)}, pages {tuple(pages.shape)}, out {tuple(out.shape)}")
@@ -1196,8 +1258,9 @@ def latent_heads_out(w: torch.Tensor, out: torch.Tensor, *, kv_rank: int, rot_di
     T, H, vdim = out.shape
     if tuple(w.shape) != (H, vdim, kv_rank) or w.dtype != out.dtype or (mixed is None) == (part_o is None) or \
             (mixed is not None and (tuple(mixed.shape) != (T, H, kv_rank) or mixed.dtype != out.dtype)) or \
-            (part_o is not None and (part_ml is None or sink is None or part_o.numel() < T * H * n_parts * kv_rank
-                                     or part_ml.numel() < T * H * n_parts * 2 or sink.numel() != H)):
+            (part_o is not None and (part_ml is None or part_o.numel() < T * H * n_parts * kv_rank
+                                     or part_ml.numel() < T * H * n_parts * 2)) or \
+            (sink is not None and sink.numel() != H):
         raise KernelError(f"latent_heads_out: w {tuple(w.shape)}, out {tuple(out.shape)}")
     lib = latent_lib(kv_rank, rot_dim)
     _check(lib.lyp_latent_heads_out(_p(part_o), _p(part_ml), _p(sink), _p(mixed), _p(w), _p(out), _code(out.dtype),
@@ -1457,22 +1520,51 @@ def moe_route_from(x: torch.Tensor, router: torch.Tensor, bias: torch.Tensor | N
 class MoePlan:
     """Where the (token, choice) pairs of a step stand once sorted by expert, on the device."""
 
-    def __init__(self, idx: torch.Tensor, E: int, route=None):
-        """``route`` (partial sums [parts, T, experts], bias, top, always, weights): the choices are not
-        made yet; the sort's kernel adds the router's partial sums up, chooses into ``idx`` and the
-        weights, and sorts."""
+    def _place(self, pairs: int, top: int, E: int) -> tuple:
+        """Sizes of the plan's pieces: expert offsets, pair at each place, place of each pair, tiles
+        (expert, first row), their count."""
         lib = core()
-        self.pairs, self.top, self.E = idx.numel(), idx.shape[1], E
-        self.tile_rows = lib.lyp_moe_tile_rows(self.pairs, E)
-        self.most_tiles = lib.lyp_moe_most_tiles(self.pairs, E, self.tile_rows)
-        # one allocation: expert offsets, pair at each place, place of each pair, tiles, their count
-        sizes = (E + 1, self.pairs, self.pairs, self.most_tiles, self.most_tiles, 1)
-        buf = torch.empty(sum(sizes), dtype=torch.int32, device=idx.device)
+        self.pairs, self.top, self.E = pairs, top, E
+        self.tile_rows = lib.lyp_moe_tile_rows(pairs, E)
+        self.most_tiles = lib.lyp_moe_most_tiles(pairs, E, self.tile_rows)
+        return (E + 1, pairs, pairs, self.most_tiles, self.most_tiles, 1)
+
+    def _take(self, buf: torch.Tensor, sizes: tuple) -> None:
         views, at = [], 0
         for n in sizes:
             views.append(buf[at:at + n])
             at += n
         self.expert_off, self.sorted_pair, self.place_of, self.tile_expert, self.tile_row0, self.n_tiles = views
+
+    @classmethod
+    def from_tables(cls, tables: torch.Tensor, tokens: torch.Tensor, E: int) -> list:
+        """A plan per layer, all made in one launch, for layers in which a table names every token
+        id's experts: tables int32 [layers, vocab, top] (entries below E), tokens int32 [T] (below
+        vocab)."""
+        _dev(tables, tokens)
+        if tables.dtype != torch.int32 or tables.dim() != 3 or tokens.dtype != torch.int32 or tokens.dim() != 1:
+            raise KernelError(f"moe tables: {tuple(tables.shape)} {tables.dtype}, tokens {tuple(tokens.shape)} {tokens.dtype}")
+        L, V, top = tables.shape
+        plans = [cls.__new__(cls) for _ in range(L)]
+        for p in plans:
+            sizes = p._place(tokens.numel() * top, top, E)
+        buf = torch.empty((L, sum(sizes)), dtype=torch.int32, device=tokens.device)
+        for p, row in zip(plans, buf):
+            p._take(row, sizes)
+        p = plans[0]
+        lib = core()
+        _check(lib.lyp_moe_sort_tables(_p(tables), V * top, _p(tokens), L, tokens.numel(), top, E, p.tile_rows,
+                                       _p(p.expert_off), _p(p.sorted_pair), _p(p.place_of), _p(p.tile_expert),
+                                       _p(p.tile_row0), _p(p.n_tiles), buf.shape[1], _stream()), lib)
+        return plans
+
+    def __init__(self, idx: torch.Tensor, E: int, route=None):
+        """``route`` (partial sums [parts, T, experts], bias, top, always, weights): the choices are not
+        made yet; the sort's kernel adds the router's partial sums up, chooses into ``idx`` and the
+        weights, and sorts."""
+        lib = core()
+        sizes = self._place(idx.numel(), idx.shape[1], E)      # one allocation
+        self._take(torch.empty(sum(sizes), dtype=torch.int32, device=idx.device), sizes)
         if route is not None:
             part, bias, top, always, wgt = route
             _check(lib.lyp_moe_route_sort(_p(part), part.shape[0], _p(bias), part.shape[1], part.shape[2], top, always,
@@ -1493,10 +1585,11 @@ def moe_sort(idx: torch.Tensor, num_experts: int) -> MoePlan:
 
 
 def moe_gemm(a: torch.Tensor, w: torch.Tensor, plan: MoePlan, *, gated: bool, limit: float = 0.0,
-             alpha: float = 0.0, gather: bool = False, relu2: bool = False) -> torch.Tensor:
+             alpha: float = 0.0, plus: float = 1.0, gather: bool = False, relu2: bool = False) -> torch.Tensor:
     """One product per expert over the rows sorted to it.  gated: a [T, K] (rows gathered by token),
-    w [E, 2 N, K] (an expert's gate rows, then its up rows) -> [pairs, N], the gated activation of
-    ``glu_clamped`` applied.  Otherwise a [pairs, K] in sorted order, w [E, N, K] -> [pairs, N]; with
+    w [E, 2 N, K] (an expert's gate rows, then its up rows) -> [pairs, N], the gated activation
+    g * sigmoid(alpha * g) * (u + plus) applied, g = min(gate, limit) and u = clamp(up, -limit, limit) (no
+    limit: infinity).  Otherwise a [pairs, K] in sorted order, w [E, N, K] -> [pairs, N]; with
     ``gather`` a is [T, K] and gathered by token as for a gated product, with ``relu2`` the result
     is max(y, 0)^2."""
     _dev(a, w)
@@ -1510,11 +1603,11 @@ def moe_gemm(a: torch.Tensor, w: torch.Tensor, plan: MoePlan, *, gated: bool, li
     _check(lib.lyp_moe_gemm(_p(a), a.stride(0), _p(w), w.stride(0), w.stride(1), _p(out), out.stride(0), _code(a.dtype),
                             int(gated), _p(plan.tile_expert), _p(plan.tile_row0), _p(plan.n_tiles), plan.most_tiles,
                             plan.tile_rows, _p(plan.expert_off), _p(plan.sorted_pair), plan.top, N, K, float(limit),
-                            float(alpha), int(gather) | 2 * int(relu2), _stream()), lib)
+                            float(alpha), float(plus), int(gather) | 2 * int(relu2), _stream()), lib)
     return out
 
 
-def moe_combine(y: torch.Tensor, plan: MoePlan, weights: torch.Tensor, rows: int, addend: torch.Tensor | None = None,
+def moe_combine(y: torch.Tensor, plan: MoePlan, weights: torch.Tensor | None, rows: int, addend: torch.Tensor | None = None,
                 shared: torch.Tensor | None = None) -> torch.Tensor:
     """float [1, rows, H]: addend + shared + sum over a token's choices of weight * y[place of the
     pair], added up in 32-bit in the order of the choices (one slice of partial sums, which a norm
@@ -1524,12 +1617,119 @@ def moe_combine(y: torch.Tensor, plan: MoePlan, weights: torch.Tensor, rows: int
     for t in (addend, shared):
         if t is not None and (tuple(t.shape) != (rows, H) or t.dtype != y.dtype):
             raise KernelError(f"moe_combine: {tuple(t.shape)} {t.dtype} beside [{rows}, {H}] {y.dtype}")
-    if weights.dtype != torch.float32 or weights.numel() != plan.pairs or rows * plan.top != plan.pairs:
+    if rows * plan.top != plan.pairs or (weights is not None and (weights.dtype != torch.float32 or
+                                                                  weights.numel() != plan.pairs)):
         raise KernelError("moe_combine: weights do not fit the pairs")
     out = torch.empty((1, rows, H), dtype=torch.float32, device=y.device)
     lib = core()
     _check(lib.lyp_moe_combine(_p(y), _p(plan.place_of), _p(weights), plan.top, _p(addend), _p(shared), _p(out),
                                _code(y.dtype), rows, H, _stream()), lib)
+    return out
+
+
+class PendingExperts:
+    """The weighted sum over a token's experts, not carried out yet: ``stream_next`` puts it straight
+    onto the residual stream; ``run()`` gives it as ``moe_combine`` does."""
+
+    def __init__(self, y: torch.Tensor, plan: MoePlan, weights: torch.Tensor | None, rows: int):
+        self.y, self.plan, self.weights, self.rows = y, plan, weights, rows
+
+    def run(self) -> torch.Tensor:
+        return moe_combine(self.y, self.plan, self.weights, self.rows)
+
+
+# ------------------------------------ a residual stream read feature by feature
+class StreamMap:
+    """What a branch reads of the residual stream when every feature is worked out by itself: the value
+    as it is (``weight`` None), or tanh(alpha v) * weight + bias (float vectors)."""
+
+    def __init__(self, weight: torch.Tensor | None = None, bias: torch.Tensor | None = None, alpha: float = 1.0):
+        _f32(weight, bias)
+        if (weight is None) != (bias is None):
+            raise KernelError("a bent stream has weights and biases")
+        self.kind = 0 if weight is None else 1
+        self.weight, self.bias, self.alpha = weight, bias, float(alpha)
+
+
+class Restart:
+    """The residual stream begins again as base + delta, whatever it held: ``base`` float [T, H], ``delta`` as
+    anything that may be added to a stream."""
+
+    def __init__(self, base: torch.Tensor, delta):
+        self.base, self.delta = base, delta
+
+    def join(self, h: torch.Tensor) -> None:
+        """Carry it out on h; nothing is left to add (returns None)."""
+        _map_rows(h, self.base, plain_delta(self.delta), StreamMap(), None, None)
+        return None
+
+
+def plain_delta(delta):
+    """A product or an experts' sum that is still pending, carried out: a tensor (or float partial sums)."""
+    return delta.run() if isinstance(delta, (PendingLinear, PendingExperts)) else delta
+
+
+def _map_rows(h, base, delta, smap: StreamMap, out, rows) -> None:
+    """h (None: not kept) = base + delta; out (None: not wanted) = smap of it, of ``rows`` alone if given."""
+    _dev(h, base, delta, smap.weight, smap.bias, out, rows)
+    T, H = base.shape
+    n = T if rows is None else rows.numel()
+    parts, stride = 0, 0
+    if delta is not None:
+        parts, stride = (delta.shape[0], T * H) if delta.dim() == 3 else (1, 0)
+        if tuple(delta.shape[-2:]) != (T, H) or (delta.dim() == 3 and delta.dtype != torch.float32):
+            raise KernelError(f"stream_map: {tuple(delta.shape)} {delta.dtype} onto {(T, H)}")
+    if base.dtype != torch.float32 or (h is not None and (h.dtype != torch.float32 or tuple(h.shape) != (T, H))) or \
+            (out is not None and tuple(out.shape) != (n, H)) or (smap.kind and smap.weight.numel() != H) or \
+            (smap.kind and smap.bias.numel() != H):
+        raise KernelError(f"stream_map: base {tuple(base.shape)} {base.dtype}, out {None if out is None else tuple(out.shape)}")
+    if rows is not None and rows.dtype != torch.int32:
+        raise KernelError("stream_map: rows are int32")
+    lib = core()
+    _check(lib.lyp_stream_map(_p(h), _p(base), _p(delta), _code(delta.dtype) if delta is not None else F32, parts, stride,
+                              smap.kind, smap.alpha, _p(smap.weight), _p(smap.bias), _p(out),
+                              _code(out.dtype) if out is not None else F32, _p(rows), n, H, _stream()), lib)
+
+
+def stream_next(h: torch.Tensor, delta, smap: StreamMap, dtype: torch.dtype, rows: torch.Tensor | None = None,
+                keep: bool = True) -> torch.Tensor:
+    """Carry out what is still to be added to the float residual stream ``h`` (None, a tensor, float partial
+    sums, a PendingLinear, a PendingExperts, or a Restart around one of them) and return what ``smap``
+    makes of the rows, in ``dtype``.  A pending product or sum does both in its own kernel.  ``rows`` picks
+    the rows to map and leaves h alone; ``keep`` False: h need not receive the sum."""
+    base = h
+    if isinstance(delta, Restart):
+        base, delta = delta.base, delta.delta
+    T, H = h.shape
+    if rows is None and isinstance(delta, (PendingLinear, PendingExperts)):
+        out = torch.empty((T, H), dtype=dtype, device=h.device)
+        keeps = h if keep else None
+        _dev(h, base, smap.weight, smap.bias)
+        _f32(h, base)
+        if tuple(base.shape) != (T, H) or (smap.kind and (smap.weight.numel() != H or smap.bias.numel() != H)):
+            raise KernelError(f"stream_next: base {tuple(base.shape)} for a stream of {(T, H)}")
+        lib = core()
+        if isinstance(delta, PendingLinear):
+            x, w = delta.x, delta.w
+            if x.dtype == dtype and tuple(w.shape) == (H, x.shape[1]) and x.shape[0] == T and _few_rows_product(T, w, dtype):
+                _dev(x, w)
+                rc = lib.lyp_gemm_stream(_p(x), _p(w), _p(base), H, _p(keeps), H, _code(dtype), T, H, x.shape[1], x.stride(0),
+                                         w.stride(0), smap.kind, smap.alpha, _p(smap.weight), _p(smap.bias), _p(out), H,
+                                         _stream())
+                if rc < 0:
+                    _check(rc, lib)
+                if rc == 0:
+                    return out
+        elif delta.y.dtype == dtype and delta.y.shape[1] == H and delta.rows == T:
+            _dev(delta.y, delta.weights)
+            _check(lib.lyp_moe_combine_stream(_p(delta.y), _p(delta.plan.place_of), _p(delta.weights), delta.plan.top,
+                                              _p(keeps), _p(base), smap.kind, smap.alpha, _p(smap.weight), _p(smap.bias),
+                                              _p(out), _code(dtype), T, H, _stream()), lib)
+            return out
+    delta = plain_delta(delta)
+    out = torch.empty((T if rows is None else rows.numel(), H), dtype=dtype, device=h.device)
+    writes = keep and rows is None and (delta is not None or base is not h)
+    _map_rows(h if writes else None, base, delta, smap, out, rows)
     return out
 
 

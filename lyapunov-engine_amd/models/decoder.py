@@ -17,11 +17,12 @@ from typing import Iterator, Optional
 
 import torch
 
-from ..config.registry import BLOCKS, EMBEDDINGS, HEADS, NORMS, STREAM_SHIFTS
+from ..config.registry import BLOCKS, EMBEDDINGS, HEADS, NORMS, STREAM_ENTRIES, STREAM_SHIFTS
 from ..config.specs import LayerCall, ModelSpec
 from ..kernels import ops
 from ..parts.base import (LayerCache, Logits, PagedSpec, Part, PositionEncoding, StateSpec, StepContext, WeightSource,
                           WeightSpec)
+from ..parts.block import settled
 
 
 @dataclass(frozen=True)
@@ -54,16 +55,26 @@ class DecoderModel(Part):
             self.head.tie(self.embedding)
         self.stream_shift = STREAM_SHIFTS.build(spec.stream_shift, hidden_size=spec.hidden_size) \
             if spec.stream_shift is not None else None
+        self.stream_entry = STREAM_ENTRIES.build(spec.stream_entry, hidden_size=spec.hidden_size) \
+            if spec.stream_entry is not None else None
         self.schedule: tuple = tuple(spec.schedule)
         for call in self.schedule:
             if not 0 <= call.layer < len(self.layers):
                 raise ValueError(f"the running order names layer {call.layer}; there are {len(self.layers)}")
             if call.shift is not None and self.stream_shift is None:
                 raise ValueError("a call of the running order adds a stream shift, and the model has none")
+            if call.enter and (self.stream_entry is None or call.reinject or call.shift is not None):
+                raise ValueError("a call of the running order enters the stream anew, and the model has no entry for it "
+                                 "(or the call adds something else as well)")
         self.device: Optional[torch.device] = None
         self.dtype: Optional[torch.dtype] = None
         self.max_positions = spec.max_position      # positions a step may reach; ``materialize`` may lower it
         self._layout = self._plan_cache()
+        groups: dict = {}
+        for _, part in self.named_parts():
+            if part.step_group() is not None:
+                groups.setdefault((type(part), part.step_group()), []).append(part)
+        self._step_groups = list(groups.values())
 
     @property
     def embed(self) -> Optional[torch.Tensor]:
@@ -86,6 +97,8 @@ class DecoderModel(Part):
         yield from walk(self.spec.embed_prefix, self.embedding)
         if self.stream_shift is not None:
             yield from walk(self.spec.stream_shift_prefix, self.stream_shift)
+        if self.stream_entry is not None:
+            yield from walk(self.spec.stream_entry_prefix, self.stream_entry)
         for i, layer in enumerate(self.layers):
             yield from walk(self.spec.layer_prefix.format(i=i), layer)
         yield from walk(self.spec.final_norm_prefix, self.final_norm)
@@ -173,6 +186,8 @@ class DecoderModel(Part):
         self.embedding.materialize(self.device, dtype)
         if self.stream_shift is not None:
             self.stream_shift.materialize(self.device, dtype)
+        if self.stream_entry is not None:
+            self.stream_entry.materialize(self.device, dtype)
         for layer in self.layers:
             layer.materialize(self.device, dtype)
         self.final_norm.materialize(self.device, dtype)
@@ -186,11 +201,23 @@ class DecoderModel(Part):
         ``caches[i]`` is the LayerCache of ``schedule[i]``."""
         h = self.embedding.forward(ctx, ctx.token_ids)
         # calls that add the embedding's output again read it from a second copy (h itself moves on)
-        first = self.embedding.forward(ctx, ctx.token_ids) if any(c.reinject for c in self.schedule) else None
+        again = any(c.reinject or (c.enter and i) for i, c in enumerate(self.schedule))
+        first = self.embedding.forward(ctx, ctx.token_ids) if again else h
+        ctx.prepared = {}
+        for parts in self._step_groups:
+            type(parts[0]).begin_step(ctx, parts)
+        entry = self.stream_entry.prepare(ctx, first) if self.stream_entry is not None else None
         delta = None
         for call, cache in zip(self.schedule, caches):
-            if isinstance(delta, ops.ScaledBranch) and (call.reinject or call.shift is not None):
-                delta = delta.join(h)
+            if call.reinject or call.shift is not None:
+                if isinstance(delta, (ops.ScaledBranch, ops.Restart)):
+                    delta = delta.join(h)
+                if isinstance(delta, ops.PendingExperts):
+                    delta = delta.run()
+            if call.enter:
+                if isinstance(delta, (ops.ScaledBranch, ops.JoiningBranch)):
+                    delta = delta.join(h)
+                delta = self.stream_entry.forward(ctx, h, delta, entry)
             if call.reinject:
                 if isinstance(delta, ops.JoiningBranch):
                     delta = delta.join(h)
@@ -201,13 +228,11 @@ class DecoderModel(Part):
             h, delta = self.layers[call.layer].forward(ctx, h, delta, cache)
         if ctx.R == 0:
             return None
-        if isinstance(delta, ops.PendingLinear) and not getattr(self.final_norm, "can_defer", False):
-            delta = delta.run()
-        if isinstance(delta, ops.JoiningBranch) and not getattr(self.final_norm, "joins_branches", False):
-            delta = delta.join(h)
-        if isinstance(delta, ops.ScaledBranch) and not getattr(self.final_norm, "takes_scaled", False):
-            delta = delta.join(h)
-        x = self.final_norm.forward(ctx, h, delta, rows=ctx.logit_rows)
+        delta = settled(self.final_norm, h, delta)
+        rows = ctx.logit_rows
+        if getattr(self.final_norm, "takes_any_delta", False) and ctx.fixed is not None and not ctx.fixed.tokens:
+            rows = None          # a recorded step of one token a request wants every row, in order
+        x = self.final_norm.forward(ctx, h, delta, rows=rows)
         out = self.head.forward(ctx, x)
         return out if isinstance(out, Logits) else Logits(out)
 

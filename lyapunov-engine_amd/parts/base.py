@@ -65,7 +65,7 @@ class WeightSpec:
 
     attr: str
     sources: tuple         # of WeightSource
-    init: str = "normal"   # random-weights mode: "normal" (0, std) or "ones" (1 + noise)
+    init: str = "normal"   # random-weights mode: "normal" (0, std), "ones" (1 + noise) or "choices:<n>" (a row: different integers below n)
     interleave: int = 0    # n > 0: rows alternate between the sources in runs of n (n of the first, n of the second, ...)
 
     @property
@@ -96,6 +96,17 @@ class Part:
         """Build device tables that are computed rather than loaded."""
         for c in self.children().values():
             c.materialize(device, dtype)
+
+    def step_group(self):
+        """A hashable key for parts that have work to do on the device once per step, whatever runs
+        how often in it, and can do it together: before the first layer, the decoder hands all parts
+        of one key to the ``begin_step`` of their class.  None: nothing to do."""
+        return None
+
+    @classmethod
+    def begin_step(cls, ctx: "StepContext", parts: list) -> None:
+        """Do that work; what the parts' ``forward`` is to find goes into ``ctx.prepared``."""
+        raise NotImplementedError
 
     def step_planner(self) -> Optional["StepPlanner"]:
         """What this part wants worked out once per step, on the host, from the
@@ -271,6 +282,7 @@ class StepContext:
     state_slots_host: list = field(default_factory=list)
     workspace: dict = field(default_factory=dict)   # scratch tensors shared by the layers of a step
     fixed: Optional[FixedStep] = None     # set while a fixed step is recorded or replayed
+    prepared: dict = field(default_factory=dict)    # what parts worked out once for this run of the step (Part.begin_step)
 
     def scratch(self, key: str, numel: int, dtype: torch.dtype = torch.float32) -> torch.Tensor:
         t = self.workspace.get(key)
@@ -402,6 +414,20 @@ class StreamShift(Part):
         raise NotImplementedError
 
 
+class StreamEntry(Part):
+    """What makes the residual stream anew before a call of the running order that asks for it, from
+    the stream so far and the embedding's output."""
+
+    def prepare(self, ctx: StepContext, first: torch.Tensor):
+        """What every entry of this step shares; ``first`` is the embedding's output, float [T, hidden]."""
+        return first
+
+    def forward(self, ctx: StepContext, h: torch.Tensor, delta, prepared):
+        """-> what is to be added to h from here on (as a rule a kernels.ops.Restart): ``delta`` is what
+        still had to be added to h before."""
+        raise NotImplementedError
+
+
 class FeedForward(Part):
     takes_pending_norm = False   # as for Mixer
 
@@ -431,5 +457,5 @@ class Block(Part):
 __all__ = [
     "WeightSource", "WeightSpec", "free_size", "shape_fits", "made_up_shape", "Part", "PagedSpec", "PageTensor", "SLOT", "StateSpec", "GroupView", "LayerCache", "StepContext",
     "StepBatch", "StepPlan", "StepPlanner", "FixedStep",
-    "Norm", "PositionEncoding", "Mixer", "FeedForward", "InputFilter", "StreamShift", "Block", "Logits", "Any",
+    "Norm", "PositionEncoding", "Mixer", "FeedForward", "InputFilter", "StreamShift", "StreamEntry", "Block", "Logits", "Any",
 ]

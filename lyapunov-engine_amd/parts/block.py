@@ -18,21 +18,29 @@ from .base import Block, LayerCache, StepContext, WeightSource, WeightSpec
 
 @BLOCKS.register("prenorm")
 class PreNormBlock(Block):
+    """The feed-forward branch may be absent (``LayerSpec.ffn`` None).  ``names["separator"]`` is what
+    stands between a part's piece of the tensor names and what follows (default: a dot)."""
+
     def __init__(self, spec: LayerSpec):
         self.names = dict(spec.names)
         self.norm1 = NORMS.build(spec.norm1)
         self.mixer = MIXERS.build(spec.mixer)
-        self.norm2 = NORMS.build(spec.norm2)
-        self.ffn = FEED_FORWARDS.build(spec.ffn)
+        self.ffn = FEED_FORWARDS.build(spec.ffn) if spec.ffn is not None else None
+        self.norm2 = NORMS.build(spec.norm2) if self.ffn is not None else None
 
     def children(self):
         n = self.names
-        return {n["norm1"] + ".": self.norm1, n["mixer"] + ".": self.mixer, n["norm2"] + ".": self.norm2,
-                n["ffn"] + ".": self.ffn}
+        sep = n.get("separator", ".")
+        out = {n["norm1"] + sep: self.norm1, n["mixer"] + sep: self.mixer}
+        if self.ffn is not None:
+            out.update({n["norm2"] + sep: self.norm2, n["ffn"] + sep: self.ffn})
+        return out
 
     def forward(self, ctx: StepContext, h, delta, cache: LayerCache):
         x = normed(self.norm1, self.mixer, ctx, h, delta)
         a = self.mixer.forward(ctx, x, cache)
+        if self.ffn is None:
+            return h, a
         x = normed(self.norm2, self.ffn, ctx, h, a)
         return h, self.ffn.forward(ctx, x)
 
@@ -207,15 +215,25 @@ def normed(norm, consumer, ctx: StepContext, h, delta):
     consumer that takes it may pass the rows on unevaluated (ops.PendingNorm);
     a norm that does not know of pending products gets the product itself, and
     one that does not know of joining branches finds the branch joined."""
+    delta = settled(norm, h, delta)
+    if getattr(norm, "can_defer", False):
+        return norm.forward(ctx, h, delta, lazy=getattr(consumer, "takes_pending_norm", False))
+    return norm.forward(ctx, h, delta)
+
+
+def settled(norm, h, delta):
+    """``delta`` in a form that ``norm`` takes: what it does not know of is carried out first."""
     if isinstance(delta, ops.JoiningBranch) and not getattr(norm, "joins_branches", False):
         delta = delta.join(h)
     if isinstance(delta, ops.ScaledBranch) and not getattr(norm, "takes_scaled", False):
         delta = delta.join(h)
-    if getattr(norm, "can_defer", False):
-        return norm.forward(ctx, h, delta, lazy=getattr(consumer, "takes_pending_norm", False))
-    if isinstance(delta, ops.PendingLinear):
+    if isinstance(delta, ops.Restart) and not getattr(norm, "takes_any_delta", False):
+        delta = delta.join(h)
+    if isinstance(delta, ops.PendingExperts) and not getattr(norm, "takes_any_delta", False):
         delta = delta.run()
-    return norm.forward(ctx, h, delta)
+    if isinstance(delta, ops.PendingLinear) and not getattr(norm, "can_defer", False):
+        delta = delta.run()
+    return delta
 
 
 def stream_rows(ctx: StepContext, h, delta):
@@ -228,10 +246,10 @@ def stream_rows(ctx: StepContext, h, delta):
             return h
         out = torch.empty(h.shape, dtype=ctx.dtype, device=h.device)
         return ops.branch_join(h, delta.y, delta.weight, delta.mult, delta.eps, shift=delta.shift, out=out)
-    if isinstance(delta, ops.ScaledBranch):
+    if isinstance(delta, (ops.ScaledBranch, ops.Restart)):
         delta = delta.join(h)
     if delta is not None:
-        ops.stream_add(h, delta)
+        ops.stream_add(h, ops.plain_delta(delta))
     return ops.cast(h, ctx.dtype)
 
 

@@ -14,9 +14,9 @@ from typing import Optional
 
 import torch
 
-from ..config.registry import EMBEDDINGS, HEADS, NORMS, STREAM_SHIFTS
+from ..config.registry import EMBEDDINGS, HEADS, NORMS, STREAM_ENTRIES, STREAM_SHIFTS
 from ..kernels import ops
-from .base import Embedding, Head, Logits, StepContext, StreamShift, WeightSource, WeightSpec
+from .base import Embedding, Head, Logits, StepContext, StreamEntry, StreamShift, WeightSource, WeightSpec
 
 
 @EMBEDDINGS.register("lookup")
@@ -65,8 +65,12 @@ class SinusoidEmbedding(TokenEmbedding):
 
 @HEADS.register("linear")
 class LinearHead(Head):
-    def __init__(self, vocab_size: int, hidden_size: int, tensor: str = "weight"):
+    def __init__(self, vocab_size: int, hidden_size: int, tensor: str = "weight", scale: float = 1.0, cap: float = 0.0):
+        """``scale`` multiplies every logit; with ``cap`` > 0 it then becomes cap * tanh(logit / cap)."""
+        if cap < 0:
+            raise ValueError(f"logits are capped at a positive number, not {cap}")
         self.vocab_size, self.hidden_size, self.tensor = vocab_size, hidden_size, tensor
+        self.scale, self.cap = float(scale), float(cap)
         self.weight: Optional[torch.Tensor] = None
         self._tied_to: Optional[Embedding] = None
 
@@ -83,7 +87,7 @@ class LinearHead(Head):
             self.weight = self._tied_to.weight      # one matrix, two uses
 
     def forward(self, ctx: StepContext, x: torch.Tensor) -> Logits:
-        return Logits(*ops.lm_head(x, self.weight))
+        return Logits(*ops.lm_head(x, self.weight, self.scale, self.cap))
 
 
 @STREAM_SHIFTS.register("table")
@@ -106,3 +110,32 @@ class ShiftTable(StreamShift):
         if not 0 <= i < self.count:
             raise IndexError(f"stream shift {i} of {self.count}")
         return self.weight_f[i]
+
+
+@STREAM_ENTRIES.register("projected_pair")
+class ProjectedPair(StreamEntry):
+    """x <- W [x; x0], x0 the embedding's output: one matrix [hidden, 2 hidden] whose first half of the
+    columns reads the stream and whose second half reads x0.  The two halves are kept apart: W0 x0 is
+    the same for every entry of a step and worked out once, and an entry is a product with the
+    stream's half that begins from it.  The new stream is in 32-bit."""
+
+    def __init__(self, hidden_size: int, tensor: str = "weight"):
+        self.hidden_size, self.tensor = int(hidden_size), tensor
+        self.stream_half: Optional[torch.Tensor] = None
+        self.first_half: Optional[torch.Tensor] = None
+        self._as_it_is: Optional[ops.StreamMap] = None
+
+    def weight_specs(self):
+        H = self.hidden_size
+        return [WeightSpec("stream_half", (WeightSource(self.tensor, (H, 2 * H), columns=(0, H)),)),
+                WeightSpec("first_half", (WeightSource(self.tensor, (H, 2 * H), columns=(H, 2 * H)),))]
+
+    def materialize(self, device, dtype):
+        self._as_it_is = ops.StreamMap()
+
+    def prepare(self, ctx: StepContext, first: torch.Tensor):
+        return ops.linear(ops.cast(first, ctx.dtype), self.first_half, out_dtype=torch.float32)
+
+    def forward(self, ctx: StepContext, h, delta, prepared):
+        x = ops.stream_next(h, delta, self._as_it_is, ctx.dtype, keep=False)
+        return ops.Restart(prepared, ops.linear(x, self.stream_half, out_dtype=torch.float32, may_split=True, pending=True))

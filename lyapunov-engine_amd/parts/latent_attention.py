@@ -7,6 +7,9 @@ Per token x:
     weights = softmax over {scale * q_h . key_h (causal), sink_h}, the sink without a value
     y = W_o concat_h(sum weights * value_h)
 
+Without a query latent (``q_rank`` 0) the queries come straight from x, q = W_q x, in one product with
+W_dkv x; without ``use_sink`` the softmax is over the keys alone.
+
 Only (c, r) is kept per token: kv_rank + rot_dim numbers, whatever the number of
 heads.  The scores and sums are taken on the latents themselves:
 q_h . W_uk,h c = (W_uk,h^T q_h) . c, so every head's query is carried into the
@@ -49,8 +52,10 @@ _BOUND = ContextBound()
 class LatentAttention(Mixer):
     def __init__(self, hidden_size: int, num_heads: int, dim: int, rot_dim: int, vdim: int, q_rank: int,
                  kv_rank: int, scale: float, eps: float, position: Optional[PartSpec] = None,
-                 names: Optional[dict] = None):
-        for what, v in (("heads", num_heads), ("vdim", vdim), ("q_rank", q_rank), ("kv_rank", kv_rank)):
+                 names: Optional[dict] = None, use_sink: bool = True, pending: bool = False):
+        """``q_rank`` 0: no query latent.  ``pending``: few rows' output product is left to the norm that
+        follows (ops.PendingLinear) and other steps' may come as partial sums, for a norm that takes them."""
+        for what, v in (("heads", num_heads), ("vdim", vdim), ("q_rank", q_rank if q_rank else 1), ("kv_rank", kv_rank)):
             if v <= 0:
                 raise ValueError(f"latent attention: {what} must be positive, got {v}")
         if dim < 0 or rot_dim < 0 or dim + rot_dim == 0:
@@ -62,7 +67,8 @@ class LatentAttention(Mixer):
         self.position = POSITION_ENCODINGS.build(position) if position is not None and rot_dim else None
         if self.position is not None and self.position.rotary_dim > rot_dim:
             raise ValueError("more rotated dimensions than the rotated part has")
-        n = dict(dq="dq", q_norm="dq.norm", uq="uq", dkv="dkv", kv_norm="dkv.norm", uk="uk", uv="uv", sink="sink", o="o")
+        self.use_sink, self.pending = bool(use_sink), bool(pending)
+        n = dict(q="q", dq="dq", q_norm="dq.norm", uq="uq", dkv="dkv", kv_norm="dkv.norm", uk="uk", uv="uv", sink="sink", o="o")
         n.update(names or {})
         self.names = n
         # sizes in multiples of 16 take the matrix-core kernel, any others the row-by-row one
@@ -72,17 +78,22 @@ class LatentAttention(Mixer):
 
     def weight_specs(self):
         n, H = self.names, self.num_heads
-        return [
-            WeightSpec("down_proj", (WeightSource(n["dq"], (self.q_rank, self.hidden_size)),
-                                     WeightSource(n["dkv"], (self.kv_rank + self.rot_dim, self.hidden_size)))),
-            WeightSpec("q_norm", (WeightSource(n["q_norm"], (self.q_rank,)),), init="ones"),
+        dkv = WeightSource(n["dkv"], (self.kv_rank + self.rot_dim, self.hidden_size))
+        if self.q_rank:
+            specs = [WeightSpec("down_proj", (WeightSource(n["dq"], (self.q_rank, self.hidden_size)), dkv)),
+                     WeightSpec("q_norm", (WeightSource(n["q_norm"], (self.q_rank,)),), init="ones"),
+                     WeightSpec("uq", (WeightSource(n["uq"], (H * (self.dim + self.rot_dim), self.q_rank)),))]
+        else:
+            specs = [WeightSpec("down_proj", (WeightSource(n["q"], (H * (self.dim + self.rot_dim), self.hidden_size)), dkv))]
+        specs += [
             WeightSpec("kv_norm", (WeightSource(n["kv_norm"], (self.kv_rank,)),), init="ones"),
-            WeightSpec("uq", (WeightSource(n["uq"], (H * (self.dim + self.rot_dim), self.q_rank)),)),
             WeightSpec("uk", (WeightSource(n["uk"], (H * self.dim, self.kv_rank)),)),
             WeightSpec("uv", (WeightSource(n["uv"], (H * self.vdim, self.kv_rank)),)),
-            WeightSpec("sink", (WeightSource(n["sink"], (H,)),)),
             WeightSpec("o_proj", (WeightSource(n["o"], (self.hidden_size, H * self.vdim)),)),
         ]
+        if self.use_sink:
+            specs.append(WeightSpec("sink", (WeightSource(n["sink"], (H,)),)))
+        return specs
 
     def children(self):
         return {"rotary.": self.position} if self.position is not None else {}
@@ -90,9 +101,9 @@ class LatentAttention(Mixer):
     def materialize(self, device, dtype):
         super().materialize(device, dtype)
         H = self.num_heads
-        self.q_norm_f = self.q_norm.float().contiguous()
+        self.q_norm_f = self.q_norm.float().contiguous() if self.q_rank else None
         self.kv_norm_f = self.kv_norm.float().contiguous()
-        self.sink_f = self.sink.float().contiguous()
+        self.sink_f = self.sink.float().contiguous() if self.use_sink else None
         # every head's W_uk as [kv_rank, dim]: the matrix that carries the head's plain query part
         # into the latent space, stored as a projection weight [out, in]
         self.uk_t = self.uk.view(H, self.dim, self.kv_rank).transpose(1, 2).contiguous() if self.dim else None
@@ -113,17 +124,24 @@ class LatentAttention(Mixer):
         table = self.position.table if self.position is not None else None
         dev = pages.device
         down = ops.linear(x, self.down_proj, out_dtype=ctx.dtype)
-        cq = torch.empty((T, self.q_rank), dtype=ctx.dtype, device=dev)
-        ops.latent_prep(down, self.q_norm_f, self.kv_norm_f, ctx.positions, table, g.slot_mapping, cq, pages,
-                        q_rank=self.q_rank, kv_rank=self.kv_rank, rot_dim=self.rot_dim, eps=self.eps)
-        q = ops.linear(cq, self.uq, out_dtype=ctx.dtype)
         qa = torch.empty((T, H, self.kv_rank + self.rot_dim), dtype=ctx.dtype, device=dev)
+        if self.q_rank:
+            cq = torch.empty((T, self.q_rank), dtype=ctx.dtype, device=dev)
+            ops.latent_prep(down, self.q_norm_f, self.kv_norm_f, ctx.positions, table, g.slot_mapping, cq, pages,
+                            q_rank=self.q_rank, kv_rank=self.kv_rank, rot_dim=self.rot_dim, eps=self.eps)
+            q = ops.linear(cq, self.uq, out_dtype=ctx.dtype)
+        else:
+            ops.latent_direct_prep(down, self.kv_norm_f, ctx.positions, table, g.slot_mapping, qa, pages, num_heads=H,
+                                   dim=self.dim, kv_rank=self.kv_rank, rot_dim=self.rot_dim, eps=self.eps)
+            q = down[:, :H * (self.dim + self.rot_dim)]
         if self.dim:
-            ops.gemm_nt_heads(q.view(T, H, self.dim + self.rot_dim)[:, :, :self.dim], self.uk_t, qa[:, :, :self.kv_rank])
+            heads_in = q.unflatten(1, (H, self.dim + self.rot_dim))[:, :, :self.dim]
+            ops.gemm_nt_heads(heads_in, self.uk_t, qa[:, :, :self.kv_rank])
         else:
             qa[:, :, :self.kv_rank].zero_()
-        ops.latent_query_rotate(q, ctx.positions, table, qa, num_heads=H, dim=self.dim, rot_dim=self.rot_dim,
-                                kv_rank=self.kv_rank)
+        if self.q_rank:
+            ops.latent_query_rotate(q, ctx.positions, table, qa, num_heads=H, dim=self.dim, rot_dim=self.rot_dim,
+                                    kv_rank=self.kv_rank)
         # a recorded step may hold rows that belong to no request: nothing writes them
         padded_rows = ctx.fixed is not None and ctx.fixed.tokens > 0
         mixed = (torch.zeros if padded_rows else torch.empty)((T, H, self.kv_rank), dtype=ctx.dtype, device=dev)
@@ -145,9 +163,13 @@ class LatentAttention(Mixer):
                                          part_ml=part_ml, sink=self.sink_f, n_parts=launch["n_parts"])
                 else:
                     ops.latent_heads_out(self.uv_heads, heads, kv_rank=self.kv_rank, rot_dim=self.rot_dim, mixed=mixed)
-                return ops.linear(heads.view(T, H * self.vdim), self.o_proj, out_dtype=ctx.dtype)
+                return self._out(ctx, heads)
         else:
             ops.latent_attn_rows(qa, pages, g.block_tables, ctx.q_start, ctx.positions, ctx.ctx_len, self.sink_f,
                                  self.scale, mixed, kv_rank=self.kv_rank, rot_dim=self.rot_dim)
         ops.gemm_nt_heads(mixed, self.uv_heads, heads)
-        return ops.linear(heads.view(T, H * self.vdim), self.o_proj, out_dtype=ctx.dtype)
+        return self._out(ctx, heads)
+
+    def _out(self, ctx: StepContext, heads):
+        return ops.linear(heads.view(ctx.T, self.num_heads * self.vdim), self.o_proj, out_dtype=ctx.dtype,
+                          may_split=self.pending, pending=self.pending)

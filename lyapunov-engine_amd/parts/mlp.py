@@ -20,16 +20,19 @@ from .base import FeedForward, StepContext, WeightSource, WeightSpec
 class DenseFeedForward(FeedForward):
     """down(act(up(x))), no gate and no biases.  ``activation``: "xielu", with its two learned
     numbers p, q in one tensor (z > 0: softplus(p) z^2 + z/2; z <= 0: (1/2 + softplus(q)) (e^z - 1 - z)
-    + z/2), or "gelu_tanh"."""
+    + z/2), "gelu_tanh", or "relu2" (max(z, 0)^2, in the up product's kernel where the rows are few).
+    ``pending``: few rows' down product is left to the norm that follows (ops.PendingLinear) and other
+    steps' may come as partial sums, for a norm that takes them."""
 
     def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "xielu",
-                 names: Optional[dict] = None):
+                 names: Optional[dict] = None, pending: bool = False):
         if activation not in ops.ACTIVATIONS:
             raise ValueError(f"unknown activation {activation!r}; known: {sorted(ops.ACTIVATIONS)}")
         self.hidden_size, self.intermediate_size, self.activation = int(hidden_size), int(intermediate_size), activation
         n = dict(up="up", down="down", act="act")
         n.update(names or {})
         self.names = n
+        self.pending = bool(pending)
         self.up_proj: Optional[torch.Tensor] = None
         self.down_proj: Optional[torch.Tensor] = None
         self.act_params: Optional[torch.Tensor] = None
@@ -48,9 +51,12 @@ class DenseFeedForward(FeedForward):
             self.act_params_f = self.act_params.float().contiguous()
 
     def forward(self, ctx: StepContext, x):
-        up = ops.linear(x, self.up_proj, out_dtype=ctx.dtype)
-        ops.activation(up, self.activation, self.act_params_f)
-        return ops.linear(up, self.down_proj, out_dtype=ctx.dtype)
+        if self.activation == "relu2":
+            up = ops.linear_relu2(x, self.up_proj)
+        else:
+            up = ops.linear(x, self.up_proj, out_dtype=ctx.dtype)
+            ops.activation(up, self.activation, self.act_params_f)
+        return ops.linear(up, self.down_proj, out_dtype=ctx.dtype, may_split=self.pending, pending=self.pending)
 
 
 @FEED_FORWARDS.register("gated_dense")

@@ -1,4 +1,4 @@
-"""RMSNorm over the hidden dimension, fused with the residual add.
+"""Norms, fused with the residual add.  RMSNorm over the hidden dimension:
 
 x * rsqrt(mean(x^2) + eps) * weight, all in 32-bit, as the reference's eager
 path (python/lyapunov_engine/ops.py:49-50) and kernel
@@ -113,3 +113,47 @@ class GroupRMSNorm(Norm):
         n = h.shape[0] if rows is None else rows.numel()
         out = torch.empty((n, self.size), dtype=out_dtype or ctx.dtype, device=h.device)
         return ops.group_rmsnorm(h, self.weight_f, self.groups, self.eps, out, delta=delta, scale=scale, rows=rows)
+
+
+@NORMS.register("dynamic_tanh")
+class DynamicTanh(Norm):
+    """tanh(alpha * x) * weight + bias, feature by feature and in 32-bit: no mean, no variance, no sum
+    over the row.  ``alpha`` is one learned number, stored with the bias beside the weight under
+    ``names`` after the part's prefix.
+
+    As a feature's result needs nothing but that feature, the norm is the last step of the kernel
+    that forms the stream's new value (``ops.stream_next``): a product of few rows, an experts'
+    weighted sum, or the row kernel that adds anything else."""
+
+    can_defer = True         # takes products still to be run
+    takes_any_delta = True   # and everything else that may still have to be added
+
+    def __init__(self, size: int, tensor: str = "weight", names: Optional[dict] = None):
+        self.size = int(size)
+        n = dict(weight=tensor, bias=(tensor + "." if tensor else "") + "b", alpha=(tensor + "." if tensor else "") + "alpha")
+        n.update(names or {})
+        self.names = n
+        self.weight: Optional[torch.Tensor] = None
+        self.bias: Optional[torch.Tensor] = None
+        self.alpha: Optional[torch.Tensor] = None
+        self._map: Optional[ops.StreamMap] = None
+
+    def weight_specs(self):
+        n = self.names
+        return [WeightSpec("weight", (WeightSource(n["weight"], (self.size,)),), init="ones"),
+                WeightSpec("bias", (WeightSource(n["bias"], (self.size,)),)),
+                WeightSpec("alpha", (WeightSource(n["alpha"], ()),), init="ones")]
+
+    @property
+    def map(self) -> "ops.StreamMap":
+        """The norm as a map of features (made on first use; a norm's weights do not change)."""
+        if self._map is None:
+            self._map = ops.StreamMap(self.weight.float().contiguous(), self.bias.float().contiguous(), float(self.alpha))
+        return self._map
+
+    def materialize(self, device, dtype):
+        self._map = None
+        self.map
+
+    def forward(self, ctx: StepContext, h, delta=None, rows=None, lazy=False):
+        return ops.stream_next(h, delta, self.map, ctx.dtype, rows=rows)

@@ -13,6 +13,12 @@ The "llama3" frequency scaling is not in the reference.  By wavelength
 2*pi/inv_freq against the original context length L: shorter than L/high stays;
 longer than L/low is divided by ``factor``; in between the two are blended with
 s = (L/wavelength - low) / (high - low): (1 - s) * inv_freq/factor + s * inv_freq.
+
+The "yarn" scaling (64-bit tables only) stretches the slow frequencies by ``factor``.  The pair that turns
+t times within ``original`` positions is number n(t) = dim * ln(original / (2 pi t)) / (2 ln theta); up to
+floor(n(fast)) a frequency stays, from ceil(n(slow)) on it is divided, and in between the two are blended
+in a straight line over the pairs' numbers.  Cosines and sines are multiplied by ``gain``
+(0.1 ln(factor) + 1 unless given).
 """
 from __future__ import annotations
 
@@ -46,6 +52,17 @@ def rotary_inv_freq(dim: int, theta: float, scaling: Optional[dict] = None) -> t
     return torch.where(medium, blended, scaled)
 
 
+def yarn_share(dim: int, theta: float, scaling: dict) -> torch.Tensor:
+    """For every pair, the share (0 to 1, 64-bit) of the divided frequency in its own."""
+    def number(turns: float) -> float:
+        return dim * math.log(float(scaling["original"]) / (2.0 * math.pi * turns)) / (2.0 * math.log(theta))
+
+    first = max(math.floor(number(float(scaling["fast"]))), 0)
+    last = min(math.ceil(number(float(scaling["slow"]))), dim - 1)
+    i = torch.arange(dim // 2, dtype=torch.float64)
+    return ((i - first) / max(last - first, 1e-3)).clamp(0.0, 1.0)
+
+
 # Tables in use, by what fixes their contents: parts with equal parameters (the
 # layers of a model, as a rule) share one tensor.  A table goes when the last
 # part that uses it does.
@@ -73,13 +90,21 @@ class RotaryEncoding(PositionEncoding):
 
     def build_table(self) -> torch.Tensor:
         if self.precise:
-            if self.scaling and self.scaling.get("rope_type", "default") not in ("default", "linear"):
-                raise ValueError("the 64-bit table knows plain and linearly scaled frequencies")
-            factor = float(self.scaling["factor"]) if self.scaling and self.scaling.get("rope_type") == "linear" else 1.0
+            kind = self.scaling.get("rope_type", "default") if self.scaling else "default"
+            if kind not in ("default", "linear", "yarn"):
+                raise ValueError("the 64-bit table knows plain, linearly scaled and stretched (yarn) frequencies")
             idx = torch.arange(0, self.rotary_dim, 2, dtype=torch.float64)
-            freq = torch.pow(torch.tensor(self.theta, dtype=torch.float64), -idx / self.rotary_dim) / factor
+            freq = torch.pow(torch.tensor(self.theta, dtype=torch.float64), -idx / self.rotary_dim)
+            gain = 1.0
+            if kind == "linear":
+                freq = freq / float(self.scaling["factor"])
+            elif kind == "yarn":
+                factor = float(self.scaling["factor"])
+                share = yarn_share(self.rotary_dim, self.theta, self.scaling)
+                freq = freq / factor * share + freq * (1.0 - share)
+                gain = float(self.scaling.get("gain", 0.1 * math.log(factor) + 1.0))
             angles = torch.outer(torch.arange(self.positions, dtype=torch.float64), freq)
-            return torch.cat((angles.cos(), angles.sin()), dim=-1).float().contiguous()
+            return (gain * torch.cat((angles.cos(), angles.sin()), dim=-1)).float().contiguous()
         inv_freq = rotary_inv_freq(self.rotary_dim, self.theta, self.scaling)
         angles = torch.outer(torch.arange(self.positions, dtype=torch.float32), inv_freq)
         return torch.cat((angles.cos(), angles.sin()), dim=-1).contiguous()

@@ -159,3 +159,68 @@ class GroupRoutedExperts(FeedForward):
         act = ops.moe_gemm(x, self.up, plan, gated=False, gather=True, relu2=True)
         y = ops.moe_gemm(act, self.down, plan, gated=False)
         return ops.moe_combine(y, plan, wgt, x.shape[0])
+
+
+@FEED_FORWARDS.register("table_experts")
+class TableExperts(FeedForward):
+    """Experts without a router: a table [vocab, top] of integers names every token id's experts (a
+    row's entries differ), each with weight 1 / top.
+
+        expert e:  y_e = W_down,e (silu(W_gate,e x) * (W_up,e x))      no biases
+        out = the mean of the token's experts' outputs
+
+    The choice rests on the step's token ids alone, so the (token, choice) pairs of all such layers
+    are sorted by expert in one launch before the first layer runs (``begin_step``), once for all
+    passes of a layer that runs several times.  Both products walk the sorted tiles; the weighted sum
+    is left to the norm that follows (ops.PendingExperts)."""
+
+    def __init__(self, hidden_size: int, num_experts: int, top: int, intermediate_size: int, vocab_size: int,
+                 names: Optional[dict] = None):
+        if not 1 <= top <= num_experts or intermediate_size <= 0 or vocab_size <= 0:
+            raise ValueError(f"table experts: {top} of {num_experts} experts of {intermediate_size}, {vocab_size} token ids")
+        self.hidden_size, self.num_experts, self.top = int(hidden_size), int(num_experts), int(top)
+        self.intermediate_size, self.vocab_size = int(intermediate_size), int(vocab_size)
+        n = dict(table="table", expert="e{j}.", gate="gate", up="up", down="down")
+        n.update(names or {})
+        self.names = n
+        self.table = self.gate_up = self.down = None
+        self._stacked = None         # of a group's first part: all the group's tables, and their owners
+
+    def weight_specs(self):
+        n, E, I, H = self.names, self.num_experts, self.intermediate_size, self.hidden_size
+        gate_up, down = [], []
+        for j in range(E):
+            e = n["expert"].format(j=j)
+            gate_up += [WeightSource(e + n["gate"], (I, H)), WeightSource(e + n["up"], (I, H))]
+            down.append(WeightSource(e + n["down"], (H, I)))
+        return [WeightSpec("table", (WeightSource(n["table"], (self.vocab_size, self.top)),), init=f"choices:{E}"),
+                WeightSpec("gate_up", tuple(gate_up)), WeightSpec("down", tuple(down))]
+
+    def materialize(self, device, dtype):
+        E, I, H = self.num_experts, self.intermediate_size, self.hidden_size
+        self.gate_up = self.gate_up.view(E, 2 * I, H)      # per expert: gate rows, then up rows
+        self.down = self.down.view(E, H, I)
+        if self.table.dtype != torch.int32:
+            raise ValueError(f"a table of experts holds integers, not {self.table.dtype}")
+        if int(self.table.min()) < 0 or int(self.table.max()) >= E:
+            raise ValueError(f"a table of experts names {int(self.table.min())} to {int(self.table.max())}; there are {E}")
+        self._stacked = None
+
+    def step_group(self):
+        return (self.vocab_size, self.top, self.num_experts)
+
+    @classmethod
+    def begin_step(cls, ctx: StepContext, parts: list) -> None:
+        lead = parts[0]
+        if lead._stacked is None:
+            lead._stacked = torch.stack([p.table for p in parts])
+            for p, t in zip(parts, lead._stacked):
+                p.table = t                                # one copy of every table
+        for p, plan in zip(parts, ops.MoePlan.from_tables(lead._stacked, ctx.token_ids, lead.num_experts)):
+            ctx.prepared[p] = plan
+
+    def forward(self, ctx: StepContext, x):
+        plan = ctx.prepared[self]
+        act = ops.moe_gemm(x, self.gate_up, plan, gated=True, limit=float("inf"), alpha=1.0, plus=0.0)
+        y = ops.moe_gemm(act, self.down, plan, gated=False)
+        return ops.PendingExperts(y, plan, None, x.shape[0])

@@ -40,6 +40,10 @@ def random_tensors(model, seed: int, dtype: torch.dtype, init_std: Optional[floa
     for name, (shape, init) in model.expected_tensors().items():
         gen = torch.Generator(device=device)
         gen.manual_seed(_tensor_seed(seed, name))
+        if init.startswith("choices:"):      # integers: every row some of the n numbers below n, none twice
+            rows, top = made_up_shape(shape)
+            yield name, torch.rand((rows, int(init[8:])), generator=gen, device=device).argsort(dim=1)[:, :top].to(torch.int32).contiguous()
+            continue
         t = torch.randn(made_up_shape(shape), generator=gen, dtype=torch.float32, device=device)
         if init == "ones":
             t = 1.0 + t * nstd
