@@ -210,8 +210,39 @@ VOBOTAR_SIZES = {
     "1b": (vobotar_shape(2048, 32, 8, 64, 16, 128256, 8192), TONILIX_SIZES["1b"][0]),
     "wide": (vobotar_shape(4096, 32, 8, 128, 8, 128256, 14336), TONILIX_SIZES["wide"][0]),
 }
+
+
+# Panodra models with layers of a real model's sizes: latent attention with a sink and a stretched
+# rotation before a dense squared-relu feed-forward, in turn with latent attention without either before
+# experts that a table picks (the experts a token uses have together the dense layer's weights, and as
+# much again for their gates); the first four layers run twice.  Beside each stands the Faledra model of
+# equal width, depth, heads, latent and dense feed-forward: the closest design (attention over latents,
+# looped layers).
+def panodra_shape(width, heads, ff, layers, vocab, kv_rank, experts, top):
+    def mixer(scaling):
+        rot = dict(base=500000.0, dims=32)
+        if scaling:
+            rot["scaling"] = dict(factor=8.0, original=4096, fast=32.0, slow=1.0)
+        return dict(heads=heads, dim=64, rot_dim=32, vdim=64, kv_rank=kv_rank, scale=96 ** -0.5, rot=rot)
+
+    def dense():
+        return dict(type="latent_attention", mixer=mixer(True), mlp=dict(kind="dense", ff=ff * 3 // 2))
+
+    def routed():
+        return dict(type="latent_attention_2", mixer=mixer(False),
+                    mlp=dict(kind="moe", expert=dict(ff=ff * 3 // (2 * top)), router=dict(experts=experts, top=top)))
+
+    return dict(architecture="Panodra", vocab=vocab, width=width, norm=dict(eps=1e-5), logit_scale=0.5, logit_softcap=30.0,
+                loop=dict(start=0, stop=4, times=2), layers=[routed() if i % 2 else dense() for i in range(layers)])
+
+
+PANODRA_SIZES = {
+    "small": (panodra_shape(1024, 16, 4096, 4, 32000, 128, 16, 4), DESIGN_SIZES["small"][0]),
+    "1b": (panodra_shape(2048, 32, 8192, 12, 128256, 256, 32, 4), DESIGN_SIZES["1b"][0]),
+    "wide": (panodra_shape(4096, 32, 14336, 4, 128256, 512, 32, 4), DESIGN_SIZES["wide"][0]),
+}
 # what stands beside a design's sizes
-BESIDE = {"faledra": "llama", "ronupel": "llama", "tonilix": "faledra", "vobotar": "tonilix"}
+BESIDE = {"faledra": "llama", "ronupel": "llama", "tonilix": "faledra", "vobotar": "tonilix", "panodra": "faledra"}
 
 
 class _Vocab:
@@ -223,12 +254,13 @@ class _Vocab:
 
 def run_design(args):
     """Prefill and decode speed of another design's sizes, each beside a model of equal size: the Llama
-    shape, or for Tonilix the Faledra model."""
+    shape, or another design's model (``BESIDE``)."""
     import torch
 
     context, block_size, out = 2304, 16, {}
     design = args.design
-    sizes = {"faledra": DESIGN_SIZES, "ronupel": RONUPEL_SIZES, "tonilix": TONILIX_SIZES, "vobotar": VOBOTAR_SIZES}[design]
+    sizes = {"faledra": DESIGN_SIZES, "ronupel": RONUPEL_SIZES, "tonilix": TONILIX_SIZES, "vobotar": VOBOTAR_SIZES,
+             "panodra": PANODRA_SIZES}[design]
     beside = BESIDE[design]
     for size in (args.size.split(",") if args.size else sorted(sizes)):
         other, second = sizes[size]
@@ -472,10 +504,10 @@ def main():
                     help="mixed: the continuous batch of BASELINE.json configs[3] instead of the headline")
     ap.add_argument("--skip-points", action="store_true", help="only the headline decode and the prefill")
     ap.add_argument("--skip-check", action="store_true", help="no comparison of bfloat16 logits with a 32-bit run")
-    ap.add_argument("--design", default="llama", choices=["llama", "faledra", "ronupel", "tonilix", "vobotar"],
-                    help="faledra, ronupel, tonilix, vobotar: that design's prefill and decode speed at a few sizes, each "
-                         "beside the Llama shape (Tonilix: the Faledra model; Vobotar: the Tonilix model) of equal size, "
-                         "instead of the headline")
+    ap.add_argument("--design", default="llama", choices=["llama", "faledra", "ronupel", "tonilix", "vobotar", "panodra"],
+                    help="faledra, ronupel, tonilix, vobotar, panodra: that design's prefill and decode speed at a few "
+                         "sizes, each beside the Llama shape (Tonilix and Panodra: the Faledra model; Vobotar: the Tonilix "
+                         "model) of equal size, instead of the headline")
     ap.add_argument("--size", default="", help="with another --design: which sizes, with commas (default: all)")
     args = ap.parse_args()
     if args.gpus != 1:

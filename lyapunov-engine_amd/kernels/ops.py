@@ -1195,7 +1195,9 @@ def latent_lib(kv_rank: int, rot_dim: int) -> ctypes.CDLL:
 
 
 def latent_attn_fits_matrix_cores(kv_rank: int, rot_dim: int) -> bool:
-    return kv_rank % 16 == 0 and rot_dim % 16 == 0 and 16 <= kv_rank <= 512 and rot_dim <= 256
+    # (the last condition: a tile of 32 keys in float fits the LDS, row by row and transposed)
+    return (kv_rank % 16 == 0 and rot_dim % 16 == 0 and 16 <= kv_rank <= 512 and 0 <= rot_dim <= 256
+            and 32 * (2 * kv_rank + rot_dim + 4) * 4 <= 160 * 1024)
 
 
 def latent_attn_launch(T: int, B: int, H: int, max_ctx: int, dtype: torch.dtype, kv_rank: int, rot_dim: int,

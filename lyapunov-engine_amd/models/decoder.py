@@ -201,12 +201,11 @@ class DecoderModel(Part):
         ``caches[i]`` is the LayerCache of ``schedule[i]``."""
         h = self.embedding.forward(ctx, ctx.token_ids)
         # calls that add the embedding's output again read it from a second copy (h itself moves on)
-        again = any(c.reinject or (c.enter and i) for i, c in enumerate(self.schedule))
-        first = self.embedding.forward(ctx, ctx.token_ids) if again else h
+        first = self.embedding.forward(ctx, ctx.token_ids) if any(c.reinject for c in self.schedule) else None
         ctx.prepared = {}
         for parts in self._step_groups:
             type(parts[0]).begin_step(ctx, parts)
-        entry = self.stream_entry.prepare(ctx, first) if self.stream_entry is not None else None
+        entry = self.stream_entry.prepare(ctx, h) if self.stream_entry is not None else None
         delta = None
         for call, cache in zip(self.schedule, caches):
             if call.reinject or call.shift is not None:

@@ -419,8 +419,9 @@ class StreamEntry(Part):
     the stream so far and the embedding's output."""
 
     def prepare(self, ctx: StepContext, first: torch.Tensor):
-        """What every entry of this step shares; ``first`` is the embedding's output, float [T, hidden]."""
-        return first
+        """What every entry of this step shares.  ``first`` is the embedding's output, float [T, hidden]:
+        the stream itself, which the layers then write to."""
+        raise NotImplementedError
 
     def forward(self, ctx: StepContext, h: torch.Tensor, delta, prepared):
         """-> what is to be added to h from here on (as a rule a kernels.ops.Restart): ``delta`` is what

@@ -155,9 +155,9 @@ def enter_pass(x: torch.Tensor, x0: torch.Tensor, w: torch.Tensor) -> torch.Tens
     return torch.cat((x, x0), dim=-1) @ w.T
 
 
-def capped_logits(x: torch.Tensor, table: torch.Tensor, scale: float, cap: float) -> torch.Tensor:
+def capped_logits(x: torch.Tensor, table: torch.Tensor, scale: float, cap: float | None) -> torch.Tensor:
     z = x @ table.T * scale
-    return cap * torch.tanh(z / cap)
+    return z if cap is None else cap * torch.tanh(z / cap)
 
 
 # ------------------------------------------------------------------------- model
@@ -196,7 +196,8 @@ def forward(tokens, tensors: dict, config: dict, trace: list | None = None) -> t
             x = x + (dense_ff(h, w) if lc["mlp"]["kind"] == "dense" else table_experts(h, tokens, w))
         if trace is not None:
             trace.append(x.clone())
-    return capped_logits(norm_of(x, tensors, "final.norm"), tensors["embed"], config["logit_scale"], config["logit_softcap"])
+    return capped_logits(norm_of(x, tensors, "final.norm"), tensors["embed"], config.get("logit_scale", 1.0),
+                         config.get("logit_softcap"))
 
 
 def load_folder(folder: str, dtype=torch.float64):
