@@ -11,6 +11,7 @@
 //   * glu_act: [rows, 2 I] (gates, then ups) -> act(gate) * up, act = silu or the tanh form of gelu.
 //   * gate_mul: x *= sigmoid(gate) or silu(gate), the gate a column range of a wider tensor.
 //   * weighted_sum: out = sa * (a + bias) + sb * b as float partial sums for the residual stream.
+//   * head_difference: two sums a head, the second times a number taken off the first, normed over the head, gated.
 //   * qkv_bias_temper_kv: from a float projection [q | k | v | ...]: biases added, every query
 //     multiplied by 1 + coef * ln(floor((p + 1) / every) + 1), queries out in the activations'
 //     type, keys and values into the token's page slot (keys [page][kv head][slot][dim], values
@@ -195,6 +196,30 @@ __global__ __launch_bounds__(256) void qkv_bias_temper_kv_kernel(
   }
 }
 
+// a float [rows, H, 2, V] -> out [rows, H, V]: o = a[0] - lambda * a[1], o / sqrt(mean(o^2) + eps) * post, times
+// sigmoid of gate [rows, >= H V] (ld_gate apart; null: not gated).  A wave a (row, head).
+template <typename T>
+__global__ __launch_bounds__(256) void head_difference_kernel(const float* __restrict__ a, const float* __restrict__ gate,
+                                                              int ld_gate, T* __restrict__ out, size_t heads, int H, int V,
+                                                              float lambda, float eps, float post) {
+  const int lane = threadIdx.x % kWave;
+  const size_t at = blockIdx.x * static_cast<size_t>(blockDim.x / kWave) + threadIdx.x / kWave;
+  if (at >= heads) return;
+  const float* first = a + at * 2 * V;
+  float ss = 0.f;
+  for (int d = lane; d < V; d += kWave) {
+    const float v = first[d] - lambda * first[V + d];
+    ss += v * v;
+  }
+  const float unit = post / sqrtf(wave_sum(ss) / static_cast<float>(V) + eps);
+  const float* g = gate != nullptr ? gate + at / H * ld_gate + at % H * V : nullptr;
+  for (int d = lane; d < V; d += kWave) {
+    float v = (first[d] - lambda * first[V + d]) * unit;
+    if (g != nullptr) v /= 1.0f + expf(-g[d]);
+    out[at * V + d] = from_f32<T>(v);
+  }
+}
+
 }  // namespace lyp
 
 using namespace lyp;
@@ -334,6 +359,26 @@ int lyp_qkv_bias_temper_kv(const float* pre, int ld, const float* bias, const in
   else
     LYP_REQUIRE(false, "qkv_bias_temper_kv: unknown dtype %d", dtype);
   LYP_LAUNCH_CHECK("qkv_bias_temper_kv");
+  return 0;
+}
+
+// a float [rows, H, 2, V], gate float [rows, >= H * V] (ld_gate apart) or null, out [rows, H, V] of dtype.
+int lyp_head_difference(const float* a, const float* gate, int ld_gate, void* out, int dtype, int n_rows, int H, int V,
+                        float lambda, float eps, float post, hipStream_t stream) {
+  LYP_REQUIRE(n_rows >= 0 && H > 0 && V > 0 && (gate == nullptr || ld_gate >= H * V), "head_difference: %d rows, %d heads of %d",
+              n_rows, H, V);
+  const size_t heads = static_cast<size_t>(n_rows) * H;
+  if (heads == 0) return 0;
+  const int blocks = static_cast<int>((heads + 3) / 4);
+  if (dtype == kF32)
+    head_difference_kernel<float><<<blocks, 256, 0, stream>>>(a, gate, ld_gate, static_cast<float*>(out), heads, H, V, lambda,
+                                                              eps, post);
+  else if (dtype == kBF16)
+    head_difference_kernel<bf16_t><<<blocks, 256, 0, stream>>>(a, gate, ld_gate, static_cast<bf16_t*>(out), heads, H, V, lambda,
+                                                               eps, post);
+  else
+    LYP_REQUIRE(false, "head_difference: unknown dtype %d", dtype);
+  LYP_LAUNCH_CHECK("head_difference");
   return 0;
 }
 

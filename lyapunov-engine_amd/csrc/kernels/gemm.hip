@@ -329,6 +329,13 @@ enum SkinnyEpilogue : int {
   kEpiResidual = 5,  // C is the float residual stream: C += A . W^T
   kEpiStream = 6,    // C = base + A . W^T (float), and the next branch's input map(C) with it (StreamTail)
   kEpiRelu2 = 7,     // stored in the operands' type as max(y, 0)^2
+  kEpiGlu = 8,       // as kEpiSwiglu, gated as GluTail says
+};
+
+// kEpiGlu: with g = min(gate, limit) and u = clamp(up, -limit, limit), the output is
+// g * sigmoid(slope * g) * (u + plus).
+struct GluTail {
+  float limit, slope, plus;
 };
 
 // The residual epilogue's by-products for the RMS norm that follows: with
@@ -398,7 +405,7 @@ template <typename T, int MB, int EPI, bool NORMED = false, int ROWS = 16, bool 
 __global__ __launch_bounds__(1024) void gemm_skinny_kernel(const T* __restrict__ A, const T* __restrict__ W,
                                                            void* __restrict__ Cv, int M, int N, int K, int lda,
                                                            int ldw, int ldc, RopeTail tail, NormHead head,
-                                                           ResidualTail res, StreamTail stm) {
+                                                           ResidualTail res, StreamTail stm, GluTail glu) {
   constexpr bool JOINS = EPI == kEpiResidual || EPI == kEpiStream;   // the sum goes onto the residual stream
   using MM = Mma16Wide<T>;
   using Frag = typename MM::Frag;
@@ -684,6 +691,11 @@ __global__ __launch_bounds__(1024) void gemm_skinny_kernel(const T* __restrict__
       const float gate = total(e), up = total(e + 128);  // the same token, row + 8
       static_cast<T*>(Cv)[static_cast<size_t>(m) * ldc + (n0 / 2 + row)] =
           from_f32<T>((gate / (1.0f + expf(-gate))) * up);
+    } else if constexpr (EPI == kEpiGlu) {
+      if (row >= 8) continue;
+      const float gate = fminf(total(e), glu.limit), up = fminf(fmaxf(total(e + 128), -glu.limit), glu.limit);
+      static_cast<T*>(Cv)[static_cast<size_t>(m) * ldc + (n0 / 2 + row)] =
+          from_f32<T>((gate / (1.0f + expf(-glu.slope * gate))) * (up + glu.plus));
     } else if constexpr (EPI == kEpiResidual) {
       float* hp = static_cast<float*>(Cv) + static_cast<size_t>(m) * ldc + n;
       const bool first = e == static_cast<int>(threadIdx.x);
@@ -999,7 +1011,7 @@ template <typename T, int EPI, bool NORMED = false, int ROWS = 16, bool PAIRED =
 static void launch_skinny(const T* A, const T* W, void* C, int M, int N, int K, int lda, int ldw, int ldc,
                           int slices, hipStream_t stream, const RopeTail& tail = RopeTail{},
                           const NormHead& head = NormHead{}, const ResidualTail& res = ResidualTail{},
-                          const StreamTail& stm = StreamTail{}) {
+                          const StreamTail& stm = StreamTail{}, const GluTail& glu = GluTail{}) {
   // tiles a wave keeps: paired, 8 rows of W each for 8 tokens each; else 16 rows of W for 16 tokens each
   const int MB = PAIRED ? (ROWS / 8) * ((M + 7) / 8) : (M + 15) / 16;
   const int waves = skinny_waves(N, K, MB * RT, slices, ROWS * RT, PAIRED ? 128 : 64);
@@ -1017,7 +1029,7 @@ static void launch_skinny(const T* A, const T* W, void* C, int M, int N, int K, 
         asked = true;                                                                                                  \
       }                                                                                                                \
     }                                                                                                                  \
-    kernel<<<grid, block, lds, stream>>>(A, W, C, M, N, K, lda, ldw, ldc, tail, head, res, stm);                       \
+    kernel<<<grid, block, lds, stream>>>(A, W, C, M, N, K, lda, ldw, ldc, tail, head, res, stm, glu);                  \
   } while (0)
 #define LYP_SKINNY(MBV) LYP_SKINNY_TB(MBV, 1)
   if constexpr (PAIRED && ROWS == 16) {
@@ -1044,11 +1056,14 @@ static void launch_skinny(const T* A, const T* W, void* C, int M, int N, int K, 
 // The plain tile with one or two row tiles per workgroup, as skinny_row_tiles says.
 template <typename T, int EPI>
 static void launch_skinny_rows(const T* A, const T* W, void* C, int M, int N, int K, int lda, int ldw, int ldc,
-                               int slices, hipStream_t stream, const RopeTail& tail = RopeTail{}) {
+                               int slices, hipStream_t stream, const RopeTail& tail = RopeTail{},
+                               const GluTail& glu = GluTail{}) {
   if (skinny_row_tiles(M, N, slices) >= 2)
-    launch_skinny<T, EPI, false, 16, false, 2>(A, W, C, M, N, K, lda, ldw, ldc, slices, stream, tail);
+    launch_skinny<T, EPI, false, 16, false, 2>(A, W, C, M, N, K, lda, ldw, ldc, slices, stream, tail, NormHead{},
+                                               ResidualTail{}, StreamTail{}, glu);
   else
-    launch_skinny<T, EPI>(A, W, C, M, N, K, lda, ldw, ldc, slices, stream, tail);
+    launch_skinny<T, EPI>(A, W, C, M, N, K, lda, ldw, ldc, slices, stream, tail, NormHead{}, ResidualTail{}, StreamTail{},
+                          glu);
 }
 
 static int g_wide_gemm = 1;   // many bfloat16 rows: 1 the wide kernel, tile by rule; for tests and measurements 0 the general kernel, 2 / 3 tiles of 128 / 256 features
@@ -1421,6 +1436,57 @@ extern "C" int lyp_gemm_relu2(const void* A, const void* W, void* out, int dtype
   else
     LYP_REQUIRE(false, "gemm_relu2: unknown dtype %d", dtype);
   LYP_LAUNCH_CHECK("gemm_relu2");
+  return 0;
+}
+
+// out[M, N/2] = g * sigmoid(slope * g) * (u + plus), g = min(gate, limit) and u = clamp(up, -limit, limit), W's rows
+// in tiles of 16 as for lyp_gemm_swiglu.  ssq_part != null: the activations are xs that still lack their
+// rows' 1 / rms (see lyp_gemm_residual).  Returns 1 (and does nothing) when the few-rows kernel does not
+// apply: then run lyp_gemm_nt and lyp_glu_clamped with runs of 8.
+extern "C" int lyp_gemm_glu(const void* A, const float* ssq_part, int n_parts, int width, float eps, const void* W,
+                            void* out, int dtype, int M, int N, int K, int lda, int ldw, int ldo, float limit,
+                            float slope, float plus, hipStream_t stream) {
+  LYP_REQUIRE(N % 16 == 0 && ldo >= N / 2, "gemm_glu: %d rows of weights, output stride %d", N, ldo);
+  LYP_REQUIRE(ssq_part == nullptr || (n_parts > 0 && width > 0), "gemm_glu: no sums of squares");
+  LYP_REQUIRE(dtype == kF32 || dtype == kBF16, "gemm_glu: unknown dtype %d", dtype);
+  if ((ssq_part != nullptr && M > 16) || !skinny_ok(M, K, lda, ldw, A, W, dtype)) return 1;
+  const NormHead head{ssq_part, n_parts, width, eps};
+  const GluTail glu{limit, slope, plus};
+#define LYP_GLU(T)                                                                                                       \
+  do {                                                                                                                   \
+    if (ssq_part != nullptr)                                                                                             \
+      launch_skinny<T, kEpiGlu, true>(static_cast<const T*>(A), static_cast<const T*>(W), out, M, N, K, lda, ldw, ldo, 1, \
+                                      stream, RopeTail{}, head, ResidualTail{}, StreamTail{}, glu);                      \
+    else                                                                                                                 \
+      launch_skinny_rows<T, kEpiGlu>(static_cast<const T*>(A), static_cast<const T*>(W), out, M, N, K, lda, ldw, ldo, 1, \
+                                     stream, RopeTail{}, glu);                                                           \
+  } while (0)
+  if (dtype == kF32) LYP_GLU(float);
+  else LYP_GLU(bf16_t);
+#undef LYP_GLU
+  LYP_LAUNCH_CHECK("gemm_glu");
+  return 0;
+}
+
+// out[M, N] = (xs / rms) . W^T, in the operands' type or float (out_f32), for at most 16 rows xs that still
+// lack their rows' 1 / rms (see lyp_gemm_residual).  Returns 1 (and does nothing) when the few-rows kernel
+// does not apply.
+extern "C" int lyp_gemm_normed(const void* xs, int ldx, const float* ssq_part, int n_parts, int width, float eps,
+                               const void* W, void* out, int dtype, int out_f32, int M, int N, int K, int ldw, int ldo,
+                               hipStream_t stream) {
+  LYP_REQUIRE(N > 0 && ldo >= N, "gemm_normed: N=%d, output stride %d", N, ldo);
+  LYP_REQUIRE(ssq_part && n_parts > 0 && width > 0, "gemm_normed: no sums of squares");
+  LYP_REQUIRE(dtype == kF32 || dtype == kBF16, "gemm_normed: unknown dtype %d", dtype);
+  if (M > 16 || !skinny_ok(M, K, ldx, ldw, xs, W, dtype)) return 1;
+  const NormHead head{ssq_part, n_parts, width, eps};
+#define LYP_NORMED(T, EPI)                                                                                               \
+  launch_skinny<T, EPI, true>(static_cast<const T*>(xs), static_cast<const T*>(W), out, M, N, K, ldx, ldw, ldo, 1, stream, \
+                              RopeTail{}, head)
+  if (dtype == kF32) LYP_NORMED(float, kEpiF32);
+  else if (out_f32) LYP_NORMED(bf16_t, kEpiF32);
+  else LYP_NORMED(bf16_t, kEpiAct);
+#undef LYP_NORMED
+  LYP_LAUNCH_CHECK("gemm_normed");
   return 0;
 }
 

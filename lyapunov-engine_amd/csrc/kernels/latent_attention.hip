@@ -25,6 +25,11 @@
 // with several it leaves (maximum, sum, unnormalised sums) per partition for
 // latent_combine_kernel.  The order of additions for a row depends on the
 // partition size and on the row's place in its tile only through rounding.
+//
+// With a window a row sees its own key and the window - 1 before it: a workgroup's walk begins at the
+// tile that holds the first key its first row sees (partitions are counted from there, so a launch
+// needs no more of them than the window and a group's tokens take), and keys that no row of the
+// workgroup sees are staged as zeros, whatever their slots hold.
 #include <algorithm>
 
 #include "common.h"
@@ -69,7 +74,7 @@ __global__ __launch_bounds__(256, KV <= 256 ? 2 : 1) void latent_attn_kernel(
     const T* __restrict__ qa, const T* __restrict__ pages, const int32_t* __restrict__ block_tables, int table_width,
     int page_size, const int32_t* __restrict__ q_start, const int32_t* __restrict__ positions,
     const int32_t* __restrict__ ctx_len, int B, const float* __restrict__ sink, float scale, T* __restrict__ out,
-    float* __restrict__ part_o, float* __restrict__ part_ml, int H, int n_parts, int part_keys, int page_shift) {
+    float* __restrict__ part_o, float* __restrict__ part_ml, int H, int n_parts, int part_keys, int page_shift, int window) {
   using MW = Mma16Wide<T>;                 // 16 x 16 tile over KCH values of the inner dimension
   using WFrag = typename MW::Frag;
   using M4 = Mma16<T>;                     // the same over 16 values (four a lane)
@@ -109,16 +114,19 @@ __global__ __launch_bounds__(256, KV <= 256 ? 2 : 1) void latent_attn_kernel(
   const bool exists = r < rows_b;
   const bool valid = live && exists;
   const int tok = q0 + (exists ? r / H : 0), head = exists ? r % H : 0;
-  const int limit = valid ? positions[tok] + 1 : 0;   // keys [0, limit) are seen
+  const int limit = valid ? positions[tok] + 1 : 0;   // keys [lo, limit) are seen
+  const int lo = window > 0 ? max(0, limit - window) : 0;
   const size_t grow = static_cast<size_t>(tok) * H + head;
 
   // keys this workgroup walks: its partition, up to what its last row sees
   const int last_row = min(row0 + kRowsPerGroup, rows_b) - 1;
   const int group_end = live ? positions[q0 + last_row / H] + 1 : 0;
-  const int k_begin = part * part_keys;
+  const int group_lo = (live && window > 0) ? max(0, positions[q0 + row0 / H] + 1 - window) : 0;
+  const int k_begin = group_lo / KT * KT + part * part_keys;
   const int k_end = min(group_end, k_begin + part_keys);
   const int wave_last = min(row0 + wave * 16 + 16, rows_b) - 1;
   const int wave_end = (live && wave_last >= row0 + wave * 16) ? positions[q0 + wave_last / H] + 1 : 0;
+  const int wave_lo = (window > 0 && wave_end > 0) ? max(0, positions[q0 + (row0 + wave * 16) / H] + 1 - window) : 0;
 
   WFrag qf[NCW > 0 ? NCW : 1];
   Frag qtail;
@@ -151,7 +159,7 @@ __global__ __launch_bounds__(256, KV <= 256 ? 2 : 1) void latent_attn_kernel(
     if (tid < KT) {
       const int key = k0 + tid;
       int row = -1;
-      if (key < k_end) {
+      if (key < k_end && key >= group_lo) {
         const int page = page_shift >= 0 ? table[key >> page_shift] : table[key / page_size];
         const int slot = page_shift >= 0 ? key & (page_size - 1) : key % page_size;
         if (page >= 0) row = page * page_size + slot;
@@ -210,6 +218,7 @@ __global__ __launch_bounds__(256, KV <= 256 ? 2 : 1) void latent_attn_kernel(
     const int tile_end = min(KT, k_end - k0);
     for (int kk = 0; kk < tile_end; kk += 16 * NS) {
       if (k0 + kk >= wave_end) break;   // nothing further is seen by this wave's rows
+      if (k0 + kk + 16 * NS <= wave_lo) continue;   // nor anything this far back
       f32x4 s[NS];
       float tmax = LYP_NEG_INF;
 #pragma unroll
@@ -235,7 +244,7 @@ __global__ __launch_bounds__(256, KV <= 256 ? 2 : 1) void latent_attn_kernel(
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           const int key = k0 + kk + 16 * u + 4 * grp + e;
-          s[u][e] = key < limit ? s[u][e] * scale : LYP_NEG_INF;
+          s[u][e] = key < limit && key >= lo ? s[u][e] * scale : LYP_NEG_INF;
           tmax = fmaxf(tmax, s[u][e]);
         }
       }
@@ -467,15 +476,18 @@ int lyp_latent_heads_out(const float* part_o, const float* part_ml, const float*
 // qa [rows, H, DK], pages [pages, page_size, DK], out [rows, H, KV] of dtype; tables as in a step.
 // merge == 0: with several partitions the merge pass is left to the caller (lyp_latent_heads_out).
 // row_groups: an upper bound on the 64-row groups of all requests (rows * H / 64 rounded up, plus one
-// per request).  n_parts > 1 needs part_o [rows * H * n_parts * KV] and part_ml [rows * H * n_parts * 2].
+// per request).  window > 0: a row sees its own key and the window - 1 before it; partitions are then counted from
+// the tile of the first key a row group sees.  n_parts > 1 needs part_o [rows * H * n_parts * KV] and part_ml [rows * H * n_parts * 2].
 int lyp_latent_attn(const void* qa, const void* pages, const int32_t* block_tables, int table_width, int page_size,
                     const int32_t* q_start, const int32_t* positions, const int32_t* ctx_len, int B,
                     const float* sink, float scale, void* out, int dtype, int n_rows, int H, int row_groups,
-                    int n_parts, int part_keys, float* part_o, float* part_ml, int merge, hipStream_t stream) {
+                    int n_parts, int part_keys, float* part_o, float* part_ml, int merge, int window,
+                    hipStream_t stream) {
   LYP_REQUIRE(n_rows >= 0 && B > 0 && H > 0 && page_size > 0 && table_width > 0 && row_groups > 0,
               "latent_attn: bad sizes rows=%d B=%d H=%d page=%d", n_rows, B, H, page_size);
   LYP_REQUIRE(n_parts >= 1 && n_parts <= 256 && part_keys > 0, "latent_attn: %d partitions of %d keys", n_parts,
               part_keys);
+  LYP_REQUIRE(window >= 0, "latent_attn: a window of %d", window);
   LYP_REQUIRE(part_keys % lyp_latent_tile_keys(dtype) == 0 || n_parts == 1,
               "latent_attn: partitions of %d keys are no multiple of the tile", part_keys);
   LYP_REQUIRE(n_parts == 1 || (part_o != nullptr && part_ml != nullptr), "latent_attn: partitions need a workspace");
@@ -497,7 +509,7 @@ int lyp_latent_attn(const void* qa, const void* pages, const int32_t* block_tabl
     latent_attn_kernel<T><<<grid, 256, Tile<T>::kBytes, stream>>>(                                                  \
         static_cast<const T*>(qa), static_cast<const T*>(pages), block_tables, table_width, page_size, q_start,     \
         positions, ctx_len, B, sink, scale, static_cast<T*>(out), part_o, part_ml, H, n_parts, part_keys,           \
-        page_shift);                                                                                                \
+        page_shift, window);                                                                                        \
     if (n_parts > 1 && merge)                                                                                       \
       latent_combine_kernel<T><<<n_rows * H, KV >= 256 ? 256 : (KV >= 128 ? 128 : 64), 0, stream>>>(                \
           part_o, part_ml, sink, static_cast<T*>(out), H, n_parts);                                                 \

@@ -1,7 +1,8 @@
 // A feed-forward that sends every token to a few of many small experts.
 //
 //   route      per token: router logits (float, computed by a 32-bit product) plus
-//              a bias, the `top` largest, and the softmax over those alone.
+//              a bias, the `top` largest, and the softmax over those alone or the chosen
+//              experts' shares of the softmax over all (RouteRule).
 //   sort       the (token, choice) pairs in order of their expert: where each
 //              expert's run starts, which pair stands at each place, the place
 //              of each pair, and the list of row tiles (expert, first place) the
@@ -17,8 +18,8 @@
 //              Otherwise rows are read by place and the product is stored.
 //   table      instead of route: a table [vocab, top] names every token id's experts, so that all layers'
 //              pairs can be sorted before the first of them runs (one launch, a workgroup a layer).
-//   combine    out[t] = addend[t] + shared[t] + sum_k weight[t, k] * y[place(t, k)],
-//              in 32-bit, in the order of k.
+//   combine    out[t] = addend[t] + share[t] * shared[t] + sum_k weight[t, k] * y[place(t, k)],
+//              in 32-bit, in the order of k (no shares given: 1).
 //
 // Every row's sums run over the inner dimension in the same order wherever the
 // row stands in its tile, so a token's result does not depend on what else is in
@@ -33,31 +34,57 @@ constexpr int kRouteRegs = 8;            // experts per lane: up to 64 * 8 exper
 constexpr int kMostExperts = 64 * kRouteRegs;
 constexpr int kMostTop = 32;
 
+// How the chosen experts' logits become weights, and what else the router's product says of a row.
+//   all      0: the softmax over the chosen logits alone; 1: the chosen experts' shares of the softmax
+//            over all E logits; either times `scale`
+//   gated    1: a logit stands behind the row's E (no bias): sigmoid of it is the row's share of what
+//            every token uses, as the weight of the `always` pair, and in share[row] where that is wanted
+struct RouteRule {
+  int all = 0;
+  float scale = 1.0f;
+  int gated = 0;
+  float* share = nullptr;
+};
+
 // One wave chooses for one row: z points at the row's E logits (bias not yet added).
 // `always` >= 0: one more pair is written after the chosen ones, expert `always` with weight 1 (an
 // expert every token uses, kept as one more matrix behind the routed ones).
 // `parts` > 1: the logits are the sum of that many partial sums, `part_stride` floats apart.
 __device__ __forceinline__ void route_row(const float* z, const float* __restrict__ bias, int E, int top,
                                           int32_t* __restrict__ idx, float* __restrict__ wgt, int lane, int always,
-                                          int parts = 1, size_t part_stride = 0) {
+                                          const RouteRule& rule, int row, int parts = 1, size_t part_stride = 0) {
   float v[kRouteRegs];
+  // logit e of the row: four partial sums asked for at a time, added in their order
+  auto logit = [&](int e) {
+    float sum = 0.f;
+    for (int p0 = 0; p0 < parts; p0 += 4) {
+      float t[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) t[i] = p0 + i < parts ? z[(p0 + i) * part_stride + e] : 0.f;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) sum += t[i];
+    }
+    return sum;
+  };
 #pragma unroll
   for (int r = 0; r < kRouteRegs; ++r) {
     const int e = lane + kWave * r;
-    if (e < E) {
-      // four partial sums asked for at a time, added in their order
-      float sum = 0.f;
-      for (int p0 = 0; p0 < parts; p0 += 4) {
-        float t[4];
+    v[r] = e < E ? logit(e) + (bias != nullptr ? bias[e] : 0.f) : LYP_NEG_INF;
+  }
+  float share = 1.0f;
+  if (rule.gated) {
+    share = 1.0f / (1.0f + expf(-logit(E)));     // the same in every lane
+    if (rule.share != nullptr && lane == 0) rule.share[row] = share;
+  }
+  float total_all = 0.f, m_all = 0.f;
+  if (rule.all) {
+    m_all = LYP_NEG_INF;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) t[i] = p0 + i < parts ? z[(p0 + i) * part_stride + e] : 0.f;
+    for (int r = 0; r < kRouteRegs; ++r) m_all = fmaxf(m_all, v[r]);
+    m_all = wave_max(m_all);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) sum += t[i];
-      }
-      v[r] = sum + (bias != nullptr ? bias[e] : 0.f);
-    } else {
-      v[r] = LYP_NEG_INF;
-    }
+    for (int r = 0; r < kRouteRegs; ++r) total_all += lane + kWave * r < E ? expf(v[r] - m_all) : 0.f;
+    total_all = wave_sum(total_all);
   }
   float chosen_v = 0.f;      // lane k keeps the k-th choice
   int chosen_e = 0;
@@ -80,31 +107,31 @@ __device__ __forceinline__ void route_row(const float* z, const float* __restric
   }
   const float m = __shfl(chosen_v, 0, kWave);      // the first choice is the largest
   const float p = lane < top ? expf(chosen_v - m) : 0.f;
-  const float total = wave_sum(p);
+  const float total = rule.all ? total_all : wave_sum(p);      // (the first choice has the largest logit of all)
   if (lane < top) {
     idx[lane] = chosen_e;
-    wgt[lane] = p / total;
+    wgt[lane] = p / total * rule.scale;
   }
   if (always >= 0 && lane == top) {
     idx[top] = always;
-    wgt[top] = 1.0f;
+    wgt[top] = share;
   }
 }
 
-// z [rows, E] float logits without bias.  One wave per row.
+// z [rows, E (+ 1 with rule.gated)] float logits without bias.  One wave per row.
 __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ z, const float* __restrict__ bias,
                                                         int rows, int E, int top, int32_t* __restrict__ idx,
-                                                        float* __restrict__ wgt, int always, int parts) {
+                                                        float* __restrict__ wgt, int always, int parts, RouteRule rule) {
   const int lane = threadIdx.x % kWave;
   const int row = blockIdx.x * (blockDim.x / kWave) + threadIdx.x / kWave;
   if (row >= rows) return;
-  const int per = top + (always >= 0 ? 1 : 0);
-  route_row(z + static_cast<size_t>(row) * E, bias, E, top, idx + static_cast<size_t>(row) * per,
-            wgt + static_cast<size_t>(row) * per, lane, always, parts, static_cast<size_t>(rows) * E);
+  const int per = top + (always >= 0 ? 1 : 0), stride = E + rule.gated;
+  route_row(z + static_cast<size_t>(row) * stride, bias, E, top, idx + static_cast<size_t>(row) * per,
+            wgt + static_cast<size_t>(row) * per, lane, always, rule, row, parts, static_cast<size_t>(rows) * stride);
 }
 
 // The router's product and the choice in one kernel: x [rows, K] in T, the router's matrix
-// w [E, K] in float; logits in 32-bit on the float matrix instruction.  A workgroup takes 16 rows;
+// w [E, K] in float (E rows here: one more than there are experts with rule.gated); logits in 32-bit on the float matrix instruction.  A workgroup takes 16 rows;
 // its eight waves share the inner dimension (an eighth each, added up in the order of the waves),
 // walk the experts in blocks of 16, four blocks a pass, and then choose for two rows each.  A wave
 // asks for four steps' operands at once: the kernel is as long as its chain of loads.
@@ -116,7 +143,7 @@ template <typename T>
 __global__ __launch_bounds__(kRouteWaves* kWave) void moe_route_fused_kernel(
     const T* __restrict__ x, int ldx, const float* __restrict__ w, const float* __restrict__ bias, int rows, int E,
     int K, int top, int32_t* __restrict__ idx, float* __restrict__ wgt, int always, int vec_ok,
-    float* __restrict__ part) {
+    float* __restrict__ part, RouteRule rule) {
   extern __shared__ float s_route[];                 // [waves][kRouteBlocks][64 lanes][4], then z [16][E]
   float* s_part = s_route;
   float* s_z = s_route + kRouteWaves * kRouteBlocks * kWave * 4;
@@ -221,8 +248,8 @@ __global__ __launch_bounds__(kRouteWaves* kWave) void moe_route_fused_kernel(
   for (int q = wave; q < 16; q += kRouteWaves) {
     const int rr = t0 + q;
     if (rr >= rows) break;
-    route_row(s_z + q * E, bias, E, top, idx + static_cast<size_t>(rr) * per, wgt + static_cast<size_t>(rr) * per, lane,
-              always);
+    route_row(s_z + q * E, bias, E - rule.gated, top, idx + static_cast<size_t>(rr) * per,
+              wgt + static_cast<size_t>(rr) * per, lane, always, rule, rr);
   }
 }
 
@@ -247,6 +274,7 @@ struct RouteFirst {
   const float* bias;
   float* wgt;
   int parts, rows, experts, top, always;
+  RouteRule rule;
 };
 
 // TABLE: pair p is the (p % top)-th expert that a table names for token id tokens[p / top]; a workgroup
@@ -286,11 +314,11 @@ __global__ __launch_bounds__(kSortThreads) void moe_sort_kernel(
   int bits = 1;                       // bits that tell the experts (and -1) apart
   while ((1 << bits) <= E) ++bits;
   if (!TABLE && first.part != nullptr) {
-    const int per = first.top + (first.always >= 0 ? 1 : 0);
+    const int per = first.top + (first.always >= 0 ? 1 : 0), stride = first.experts + first.rule.gated;
     for (int row = wave; row < first.rows; row += kSortWaves)
-      route_row(first.part + static_cast<size_t>(row) * first.experts, first.bias, first.experts, first.top,
+      route_row(first.part + static_cast<size_t>(row) * stride, first.bias, first.experts, first.top,
                 idx + static_cast<size_t>(row) * per, first.wgt + static_cast<size_t>(row) * per, lane, first.always,
-                first.parts, static_cast<size_t>(first.rows) * first.experts);
+                first.rule, row, first.parts, static_cast<size_t>(first.rows) * stride);
     __syncthreads();   // the choices are read back below by other threads of this workgroup
   }
   for (int e = tid; e < E; e += kSortThreads) cnt[e] = 0;
@@ -829,33 +857,60 @@ __global__ __launch_bounds__(NW * 64) void moe_gemm_wide_kernel(
   }
 }
 
-// gate_up [rows, 2 I] (gates first) -> out [rows, I], the experts' activation
+// gate_up [rows, 2 I] -> out [rows, I], the experts' activation; interleave 0: gates first, n > 0: runs of n
+// gates and their n ups in turn
 template <typename T>
 __global__ void glu_clamped_kernel(const T* __restrict__ gate_up, T* __restrict__ out, int rows, int I, float limit,
-                                   float alpha) {
+                                   float alpha, float plus, int interleave) {
   const size_t total = static_cast<size_t>(rows) * I;
   for (size_t i = blockIdx.x * static_cast<size_t>(blockDim.x) + threadIdx.x; i < total;
        i += static_cast<size_t>(gridDim.x) * blockDim.x) {
     const size_t r = i / I, c = i % I;
-    const float g = fminf(to_f32(gate_up[r * 2 * I + c]), limit);
-    const float u = fminf(fmaxf(to_f32(gate_up[r * 2 * I + I + c]), -limit), limit);
-    out[i] = from_f32<T>(g / (1.0f + expf(-alpha * g)) * (u + 1.0f));
+    const size_t at = interleave > 0 ? c / interleave * 2 * interleave + c % interleave : c;
+    const float g = fminf(to_f32(gate_up[r * 2 * I + at]), limit);
+    const float u = fminf(fmaxf(to_f32(gate_up[r * 2 * I + at + (interleave > 0 ? interleave : I)]), -limit), limit);
+    out[i] = from_f32<T>(g / (1.0f + expf(-alpha * g)) * (u + plus));
   }
 }
 
-// out [rows, H] float = addend + shared + sum_k wgt[row, k] * y[place_of[row * top + k]]
-// (no weights given: 1 / top each)
+// The same for I and the runs in multiples of 8 (or no runs) and 16-byte aligned rows: eight neighbouring values a thread.
+template <typename T>
+__global__ __launch_bounds__(256) void glu_clamped_vec_kernel(const T* __restrict__ gate_up, T* __restrict__ out, size_t total8,
+                                                              int I, float limit, float alpha, float plus, int interleave) {
+  typedef T Vec __attribute__((ext_vector_type(8)));
+  for (size_t i8 = blockIdx.x * static_cast<size_t>(blockDim.x) + threadIdx.x; i8 < total8;
+       i8 += static_cast<size_t>(gridDim.x) * blockDim.x) {
+    const size_t r = i8 / (I / 8), c = (i8 % (I / 8)) * 8;
+    const size_t at = interleave > 0 ? c / interleave * 2 * interleave + c % interleave : c;
+    const T* row = gate_up + r * 2 * I + at;
+    const Vec gv = *reinterpret_cast<const Vec*>(row);
+    const Vec uv = *reinterpret_cast<const Vec*>(row + (interleave > 0 ? interleave : I));
+    Vec o;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const float g = fminf(to_f32(gv[e]), limit);
+      const float u = fminf(fmaxf(to_f32(uv[e]), -limit), limit);
+      o[e] = from_f32<T>(g / (1.0f + expf(-alpha * g)) * (u + plus));
+    }
+    *reinterpret_cast<Vec*>(out + i8 * 8) = o;
+  }
+}
+
+// out [rows, H] float = addend + share[row] * shared + sum_k wgt[row, k] * y[place_of[row * top + k]]
+// (no weights given: 1 / top each; no shares given: 1)
 // One workgroup a row; the row's places and weights are read once; a thread takes V neighbouring
 // columns at a time (V = 4 where rows are whole multiples of that, else 1), two such groups in flight.
 template <typename T, int V>
 __global__ void moe_combine_kernel(const T* __restrict__ y, const int32_t* __restrict__ place_of,
                                    const float* __restrict__ wgt, int top, const T* __restrict__ addend,
-                                   const T* __restrict__ shared, float* __restrict__ out, int rows, int H) {
+                                   const T* __restrict__ shared, const float* __restrict__ share,
+                                   float* __restrict__ out, int rows, int H) {
   __shared__ int32_t s_at[kMostTop];
   __shared__ float s_w[kMostTop];
   typedef T VecT __attribute__((ext_vector_type(V)));
   typedef float VecF __attribute__((ext_vector_type(V)));
   const int row = blockIdx.x;
+  const float part = share != nullptr ? share[row] : 1.0f;
   if (threadIdx.x < top) {
     s_at[threadIdx.x] = place_of[static_cast<size_t>(row) * top + threadIdx.x];
     s_w[threadIdx.x] = wgt != nullptr ? wgt[static_cast<size_t>(row) * top + threadIdx.x] : 1.0f / static_cast<float>(top);
@@ -883,7 +938,7 @@ __global__ void moe_combine_kernel(const T* __restrict__ y, const int32_t* __res
       for (int i = 0; i < V; ++i) v[u][i] = 0.f;
       if (c >= H) continue;
       if (addend != nullptr) v[u] += get(addend + static_cast<size_t>(row) * H + c);
-      if (shared != nullptr) v[u] += get(shared + static_cast<size_t>(row) * H + c);
+      if (shared != nullptr) v[u] += part * get(shared + static_cast<size_t>(row) * H + c);
     }
     for (int k = 0; k < top; ++k) {
       const size_t base = static_cast<size_t>(s_at[k]) * H;
@@ -968,7 +1023,7 @@ int lyp_moe_route(const float* z, const float* bias, int rows, int E, int top, i
               kMostTop);
   if (rows == 0) return 0;
   LYP_REQUIRE(top < kMostTop || always < 0, "moe_route: %d chosen and one more", top);
-  moe_route_kernel<<<(rows + 3) / 4, 256, 0, stream>>>(z, bias, rows, E, top, idx, wgt, always, 1);
+  moe_route_kernel<<<(rows + 3) / 4, 256, 0, stream>>>(z, bias, rows, E, top, idx, wgt, always, 1, RouteRule{});
   LYP_LAUNCH_CHECK("moe_route");
   return 0;
 }
@@ -1030,30 +1085,32 @@ int lyp_moe_route_splits(int rows, int K) {
 }
 
 int lyp_moe_route_fused(const void* x, int ldx, int dtype, const float* w, const float* bias, int rows, int E, int K,
-                        int top, int32_t* idx, float* wgt, int always, float* part, int splits, int choose,
-                        hipStream_t stream) {
+                        int top, int32_t* idx, float* wgt, int always, float* part, int splits, int choose, int all,
+                        float scale, int gated, float* share, hipStream_t stream) {
+  const RouteRule rule{all, scale, gated, share};
+  LYP_REQUIRE((gated == 0 || gated == 1) && (share == nullptr || gated), "moe_route: %d logits behind the experts'", gated);
   LYP_REQUIRE(splits >= 1 && (splits == 1 || part != nullptr), "moe_route: %d shares of the inner dimension", splits);
   LYP_REQUIRE(rows >= 0 && E > 0 && E <= kMostExperts && top > 0 && top <= E && top <= kMostTop && K > 0 && ldx >= K,
               "moe_route: %d rows, %d experts (at most %d), %d chosen (at most %d), inner size %d", rows, E,
               kMostExperts, top, kMostTop, K);
   LYP_REQUIRE(top < kMostTop || always < 0, "moe_route: %d chosen and one more", top);
   if (rows == 0) return 0;
-  const size_t lds = sizeof(float) * (kRouteWaves * kRouteBlocks * kWave * 4 + 16 * E);
+  const size_t lds = sizeof(float) * (kRouteWaves * kRouteBlocks * kWave * 4 + 16 * (E + gated));
   const dim3 blocks((rows + 15) / 16, splits);
   const int esz = dtype == kF32 ? 4 : 2;
   const int vec_ok = K % 4 == 0 && ldx % 4 == 0 && reinterpret_cast<uintptr_t>(x) % (4 * esz) == 0 &&
                      reinterpret_cast<uintptr_t>(w) % 16 == 0;
   if (dtype == kF32)
     moe_route_fused_kernel<float><<<blocks, kRouteWaves * kWave, lds, stream>>>(
-        static_cast<const float*>(x), ldx, w, bias, rows, E, K, top, idx, wgt, always, vec_ok, part);
+        static_cast<const float*>(x), ldx, w, bias, rows, E + gated, K, top, idx, wgt, always, vec_ok, part, rule);
   else if (dtype == kBF16)
     moe_route_fused_kernel<bf16_t><<<blocks, kRouteWaves * kWave, lds, stream>>>(
-        static_cast<const bf16_t*>(x), ldx, w, bias, rows, E, K, top, idx, wgt, always, vec_ok, part);
+        static_cast<const bf16_t*>(x), ldx, w, bias, rows, E + gated, K, top, idx, wgt, always, vec_ok, part, rule);
   else
     LYP_REQUIRE(false, "moe_route: unknown dtype %d", dtype);
   // (choose == 0 with splits > 1: the caller adds the partial sums up and chooses, lyp_moe_route_sort)
   if (splits > 1 && choose)
-    moe_route_kernel<<<(rows + 3) / 4, 256, 0, stream>>>(part, bias, rows, E, top, idx, wgt, always, splits);
+    moe_route_kernel<<<(rows + 3) / 4, 256, 0, stream>>>(part, bias, rows, E, top, idx, wgt, always, splits, rule);
   LYP_LAUNCH_CHECK("moe_route");
   return 0;
 }
@@ -1074,7 +1131,7 @@ int lyp_moe_sort(const int32_t* idx, int pairs, int E, int tile_rows, int32_t* e
   const size_t lds = sizeof(int32_t) * (3 * E + 1 + kSortWaves * E);
   moe_sort_kernel<false><<<1, kSortThreads, lds, stream>>>(const_cast<int32_t*>(idx), pairs, E, tile_rows, expert_off,
                                                            sorted_pair, place_of, tile_expert, tile_row0, n_tiles,
-                                                           RouteFirst{nullptr, nullptr, nullptr, 0, 0, 0, 0, -1},
+                                                           RouteFirst{nullptr, nullptr, nullptr, 0, 0, 0, 0, -1, RouteRule{}},
                                                            TableChoice{});
   LYP_LAUNCH_CHECK("moe_sort");
   return 0;
@@ -1084,8 +1141,8 @@ int lyp_moe_sort(const int32_t* idx, int pairs, int E, int tile_rows, int32_t* e
 // sums (lyp_moe_route_fused with choose == 0 left them); idx and wgt [rows][top (+ 1)] are written here.
 int lyp_moe_route_sort(const float* part, int parts, const float* bias, int rows, int experts, int top, int always,
                        int32_t* idx, float* wgt, int E, int tile_rows, int32_t* expert_off, int32_t* sorted_pair,
-                       int32_t* place_of, int32_t* tile_expert, int32_t* tile_row0, int32_t* n_tiles,
-                       hipStream_t stream) {
+                       int32_t* place_of, int32_t* tile_expert, int32_t* tile_row0, int32_t* n_tiles, int all,
+                       float scale, int gated, float* share, hipStream_t stream) {
   const int pairs = rows * (top + (always >= 0 ? 1 : 0));
   LYP_REQUIRE(part != nullptr && parts >= 1 && rows > 0 && experts > 0 && experts <= kMostExperts && top > 0 &&
                   top <= experts && top <= kMostTop && (top < kMostTop || always < 0),
@@ -1095,7 +1152,8 @@ int lyp_moe_route_sort(const float* part, int parts, const float* bias, int rows
   const size_t lds = sizeof(int32_t) * (3 * E + 1 + kSortWaves * E);
   moe_sort_kernel<false><<<1, kSortThreads, lds, stream>>>(idx, pairs, E, tile_rows, expert_off, sorted_pair, place_of,
                                                            tile_expert, tile_row0, n_tiles,
-                                                           RouteFirst{part, bias, wgt, parts, rows, experts, top, always},
+                                                           RouteFirst{part, bias, wgt, parts, rows, experts, top, always,
+                                                                      RouteRule{all, scale, gated, share}},
                                                            TableChoice{});
   LYP_LAUNCH_CHECK("moe_route_sort");
   return 0;
@@ -1117,7 +1175,7 @@ int lyp_moe_sort_tables(const int32_t* tables, long long table_stride, const int
   const size_t lds = sizeof(int32_t) * (3 * E + 1 + kSortWaves * E);
   moe_sort_kernel<true><<<layers, kSortThreads, lds, stream>>>(
       nullptr, static_cast<int>(pairs), E, tile_rows, expert_off, sorted_pair, place_of, tile_expert, tile_row0, n_tiles,
-      RouteFirst{nullptr, nullptr, nullptr, 0, 0, 0, 0, -1}, TableChoice{tables, tokens, table_stride, out_stride, top});
+      RouteFirst{nullptr, nullptr, nullptr, 0, 0, 0, 0, -1, RouteRule{}}, TableChoice{tables, tokens, table_stride, out_stride, top});
   LYP_LAUNCH_CHECK("moe_sort_tables");
   return 0;
 }
@@ -1184,18 +1242,33 @@ int lyp_moe_gemm(const void* a, int lda, const void* w, long long w_expert_strid
   return 0;
 }
 
-int lyp_glu_clamped(const void* gate_up, void* out, int dtype, int rows, int I, float limit, float alpha,
-                    hipStream_t stream) {
-  LYP_REQUIRE(rows >= 0 && I > 0, "glu_clamped: bad sizes");
+int lyp_glu_clamped(const void* gate_up, void* out, int dtype, int rows, int I, float limit, float alpha, float plus,
+                    int interleave, hipStream_t stream) {
+  LYP_REQUIRE(rows >= 0 && I > 0 && interleave >= 0 && (interleave == 0 || I % interleave == 0),
+              "glu_clamped: bad sizes %d x %d in runs of %d", rows, I, interleave);
   if (rows == 0) return 0;
   const long long total = static_cast<long long>(rows) * I;
+  if (I % 8 == 0 && interleave % 8 == 0 && reinterpret_cast<uintptr_t>(gate_up) % 16 == 0 &&
+      reinterpret_cast<uintptr_t>(out) % 16 == 0 && (dtype == kF32 || dtype == kBF16)) {
+    const size_t total8 = static_cast<size_t>(total) / 8;
+    const int blocks8 = static_cast<int>(std::min<size_t>((total8 + 255) / 256, 8192));
+    if (dtype == kF32)
+      glu_clamped_vec_kernel<float><<<blocks8, 256, 0, stream>>>(static_cast<const float*>(gate_up), static_cast<float*>(out),
+                                                                 total8, I, limit, alpha, plus, interleave);
+    else
+      glu_clamped_vec_kernel<bf16_t><<<blocks8, 256, 0, stream>>>(static_cast<const bf16_t*>(gate_up),
+                                                                  static_cast<bf16_t*>(out), total8, I, limit, alpha, plus,
+                                                                  interleave);
+    LYP_LAUNCH_CHECK("glu_clamped");
+    return 0;
+  }
   const int blocks = static_cast<int>(std::min<long long>((total + 255) / 256, 8192));
   if (dtype == kF32)
     glu_clamped_kernel<float><<<blocks, 256, 0, stream>>>(static_cast<const float*>(gate_up),
-                                                          static_cast<float*>(out), rows, I, limit, alpha);
+                                                          static_cast<float*>(out), rows, I, limit, alpha, plus, interleave);
   else if (dtype == kBF16)
     glu_clamped_kernel<bf16_t><<<blocks, 256, 0, stream>>>(static_cast<const bf16_t*>(gate_up),
-                                                           static_cast<bf16_t*>(out), rows, I, limit, alpha);
+                                                           static_cast<bf16_t*>(out), rows, I, limit, alpha, plus, interleave);
   else
     LYP_REQUIRE(false, "glu_clamped: unknown dtype %d", dtype);
   LYP_LAUNCH_CHECK("glu_clamped");
@@ -1203,8 +1276,8 @@ int lyp_glu_clamped(const void* gate_up, void* out, int dtype, int rows, int I, 
 }
 
 int lyp_moe_combine(const void* y, const int32_t* place_of, const float* wgt, int top, const void* addend,
-                    const void* shared, float* out, int dtype, int rows, int H, hipStream_t stream) {
-  LYP_REQUIRE(rows >= 0 && H > 0 && top > 0, "moe_combine: bad sizes");
+                    const void* shared, const float* share, float* out, int dtype, int rows, int H, hipStream_t stream) {
+  LYP_REQUIRE(rows >= 0 && H > 0 && top > 0 && (share == nullptr || shared != nullptr), "moe_combine: bad sizes");
   if (rows == 0) return 0;
   LYP_REQUIRE(top <= kMostTop, "moe_combine: %d choices a token (at most %d)", top, kMostTop);
   const bool vec = H % 4 == 0 && reinterpret_cast<uintptr_t>(y) % 16 == 0 && reinterpret_cast<uintptr_t>(addend) % 16 == 0 &&
@@ -1214,7 +1287,7 @@ int lyp_moe_combine(const void* y, const int32_t* place_of, const float* wgt, in
 #define LYP_COMBINE(T, V)                                                                                      \
   moe_combine_kernel<T, V><<<rows, threads, 0, stream>>>(static_cast<const T*>(y), place_of, wgt, top,        \
                                                         static_cast<const T*>(addend),                       \
-                                                        static_cast<const T*>(shared), out, rows, H)
+                                                        static_cast<const T*>(shared), share, out, rows, H)
   if (dtype == kF32) {
     if (vec) LYP_COMBINE(float, 4);
     else LYP_COMBINE(float, 1);

@@ -4,7 +4,8 @@
 // with another layer's:
 //
 //   pre [rows, ld] float: H*D query values, G*D key values and (unless the values are the keys)
-//   G*V value values side by side, as the product's accumulators left them.
+//   GV*V value values side by side, as the product's accumulators left them (GV value heads: G, or a
+//   divisor of it where several key heads share a value head).
 //     x <- pre + bias
 //     values: the key projection itself (values_from_keys: taken before any norm) or the value
 //       projection; blended, v <- (1 - lambda) v + lambda v_other, when another layer's values
@@ -32,14 +33,14 @@ __global__ __launch_bounds__(512) void qkv_prepare_kernel(
     const float* __restrict__ wk, float eps, const int32_t* __restrict__ positions, const float* __restrict__ table,
     int rot, int pairing, int values_from_keys, const float* __restrict__ blend, const float* __restrict__ v_other,
     int ld_other, float* __restrict__ v_keep, const int32_t* __restrict__ slot_map, T* __restrict__ q_out,
-    T* __restrict__ kpool, T* __restrict__ vpool, int H, int G, int D, int V, int bs, int staged) {
+    T* __restrict__ kpool, T* __restrict__ vpool, int H, int G, int D, int V, int bs, int staged, int GV) {
   extern __shared__ __attribute__((aligned(16))) float s_prep[];
   float* s_ss = s_prep;             // H + G sums of squares, then the two whole-projection factors
   float* xs = s_prep + ((H + G + 2 + 3) & ~3);   // the biased row (when staged)
   const int t = blockIdx.x;
   const float* row = pre + static_cast<size_t>(t) * ld;
   const int nq = H * D, nk = G * D;
-  const int n_used = nq + nk + (values_from_keys ? 0 : G * V);
+  const int n_used = nq + nk + (values_from_keys ? 0 : GV * V);
   const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave, nwaves = blockDim.x / kWave;
   if (staged) {
     const bool by4 = (ld & 3) == 0 && (n_used & 3) == 0 && (reinterpret_cast<uintptr_t>(pre) & 15) == 0 &&
@@ -128,14 +129,16 @@ __global__ __launch_bounds__(512) void qkv_prepare_kernel(
   // values: the key/value heads of this workgroup's share
   const int voff = values_from_keys ? nq : nq + nk;
   const float lam = blend != nullptr ? blend[0] : 0.f;
+  const int key_heads = G / GV;      // that share a value head: the first of them brings it
   for (int hh = max(first, H) + wave; hh < last; hh += nwaves) {
-    const int g = hh - H;
+    if ((hh - H) % key_heads != 0) continue;
+    const int g = (hh - H) / key_heads;
     for (int d = lane; d < V; d += kWave) {
       const int idx = g * V + d;
       float v = at(voff + idx);
-      if (v_keep != nullptr) v_keep[static_cast<size_t>(t) * G * V + idx] = v;
+      if (v_keep != nullptr) v_keep[static_cast<size_t>(t) * GV * V + idx] = v;
       if (blend != nullptr) v = (1.0f - lam) * v + lam * v_other[static_cast<size_t>(t) * ld_other + idx];
-      if (slot >= 0) vpool[((static_cast<size_t>(page) * G + g) * V + d) * bs + off] = from_f32<T>(v);
+      if (slot >= 0) vpool[((static_cast<size_t>(page) * GV + g) * V + d) * bs + off] = from_f32<T>(v);
     }
   }
 }
@@ -148,21 +151,22 @@ extern "C" {
 
 // pre float [rows, ld]; bias float over pre's used columns or null; wq / wk float or null (norm_mode 1: [D];
 // 2: [H*D] / [G*D]); table float [positions, rot] or null; blend: a float on the device, or null; v_other float
-// [rows, >= G*V] (ld_other apart); v_keep float [rows, G*V] or null; q_out [rows, H*D] and the pools of dtype.
+// [rows, >= GV*V] (ld_other apart); v_keep float [rows, GV*V] or null; q_out [rows, H*D] and the pools of dtype.
 int lyp_qkv_prepare(const float* pre, int ld, const float* bias, int norm_mode, const float* wq, const float* wk,
                     float eps, const int32_t* positions, const float* table, int rot, int pairing, int values_from_keys,
                     const float* blend, const float* v_other, int ld_other, float* v_keep, const int32_t* slot_map,
                     void* q_out, void* kpool, void* vpool, int dtype, int n_rows, int H, int G, int D, int V, int bs,
-                    hipStream_t stream) {
+                    int GV, hipStream_t stream) {
   LYP_REQUIRE(n_rows >= 0 && H > 0 && G > 0 && D > 0 && V > 0 && bs > 0, "qkv_prepare: bad sizes rows=%d H=%d G=%d D=%d V=%d",
               n_rows, H, G, D, V);
-  LYP_REQUIRE(ld >= (H + G) * D + (values_from_keys ? 0 : G * V) && (!values_from_keys || V == D),
+  LYP_REQUIRE(GV > 0 && G % GV == 0 && (!values_from_keys || GV == G), "qkv_prepare: %d key heads over %d value heads", G, GV);
+  LYP_REQUIRE(ld >= (H + G) * D + (values_from_keys ? 0 : GV * V) && (!values_from_keys || V == D),
               "qkv_prepare: rows of %d values for %d+%d heads of %d/%d", ld, H, G, D, V);
   LYP_REQUIRE(norm_mode >= 0 && norm_mode <= 2 && (pairing == 0 || pairing == 1), "qkv_prepare: norm %d, pairing %d",
               norm_mode, pairing);
   LYP_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= D && (rot == 0 || (table != nullptr && positions != nullptr)),
               "qkv_prepare: %d rotated values of %d", rot, D);
-  LYP_REQUIRE(blend == nullptr || (v_other != nullptr && ld_other >= G * V), "qkv_prepare: a blend without the other values");
+  LYP_REQUIRE(blend == nullptr || (v_other != nullptr && ld_other >= GV * V), "qkv_prepare: a blend without the other values");
   LYP_REQUIRE(q_out != nullptr && (slot_map == nullptr || (kpool != nullptr && vpool != nullptr)), "qkv_prepare: no output");
   if (n_rows == 0) return 0;
   const int work = (H + G) * D;
@@ -173,7 +177,7 @@ int lyp_qkv_prepare(const float* pre, int ld, const float* bias, int norm_mode, 
   const int shares = n_rows <= 64 ? std::min(H + G, 16) : 1;
   const int heads_each = (H + G + shares - 1) / shares;
   const int threads = std::min(512, std::max(64, 64 * std::min(heads_each, 8)));
-  const int n_used = work + (values_from_keys ? 0 : G * V);
+  const int n_used = work + (values_from_keys ? 0 : GV * V);
   const int head_words = (H + G + 2 + 3) & ~3;
   const int staged = sizeof(float) * (head_words + n_used) <= 64 * 1024 ? 1 : 0;
   const size_t lds = sizeof(float) * (head_words + (staged ? n_used : 0));
@@ -181,7 +185,7 @@ int lyp_qkv_prepare(const float* pre, int ld, const float* bias, int norm_mode, 
   qkv_prepare_kernel<T><<<dim3(n_rows, shares), threads, lds, stream>>>(pre, ld, bias, norm_mode, wq, wk, eps, positions, table, rot, \
                                                           pairing, values_from_keys, blend, v_other, ld_other, v_keep, \
                                                           slot_map, static_cast<T*>(q_out), static_cast<T*>(kpool),    \
-                                                          static_cast<T*>(vpool), H, G, D, V, bs, staged)
+                                                          static_cast<T*>(vpool), H, G, D, V, bs, staged, GV)
   if (dtype == kF32) LYP_PREP(float);
   else if (dtype == kBF16) LYP_PREP(bf16_t);
   else LYP_REQUIRE(false, "qkv_prepare: unknown dtype %d", dtype);

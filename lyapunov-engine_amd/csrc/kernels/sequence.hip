@@ -2,8 +2,7 @@
 // the residual stream, filter a branch's input over time, or carry a
 // recurrence: the joining norm, a short causal convolution with its state, the
 // minGRU scan, the xIELU / tanh-GELU / squared-relu activations, and what a latent attention
-// layer does around its products (norms of the latents, rotation of
-// neighbouring pairs, the write of a token's latent into its page slot).
+// layer does around its products (norms of the latents, rotation, the write of a token's latent into its page slot).
 //
 // All arithmetic is 32-bit; only loads and stores see the storage type.  Small
 // parameter vectors (norm weights, filter taps, biases, sinks) arrive as float.
@@ -525,15 +524,24 @@ __global__ void mingru_chunk_output_kernel(const float* __restrict__ pre, const 
 // (kv_rank) and the shared rotated key part (rot_dim), side by side.  Writes the
 // RMS-normed query latent to cq [rows, q_rank], and the normed key/value latent
 // followed by the key part, rotated by the token's position, into the token's
-// page slot: pages [slot][kv_rank + rot_dim].  Pairs (2i, 2i+1) of the first
-// `dims` values of the key part turn by the angle of table row `position`
-// (dims/2 cosines, then dims/2 sines).
+// page slot: pages [slot][kv_rank + rot_dim].  The first `dims` values of the
+// key part turn in pairs by the angles of table row `position` (dims/2 cosines,
+// then dims/2 sines): values 2i and 2i+1 (pairing 0) or i and i + dims/2
+// (pairing 1).
+struct RotaryPair {
+  int a, b;
+};
+// Where pair i of a part of `rot_dim` values stands; from pair dims/2 on they are the neighbours that do not turn.
+__device__ __forceinline__ RotaryPair rotary_pair(int i, int half, int pairing) {
+  return pairing == 1 && i < half ? RotaryPair{i, i + half} : RotaryPair{2 * i, 2 * i + 1};
+}
+
 template <typename T>
 __global__ void latent_prep_kernel(const T* __restrict__ d, int ld, const float* __restrict__ wq,
                                    const float* __restrict__ wkv, const int32_t* __restrict__ positions,
                                    const float* __restrict__ table, int dims, const int32_t* __restrict__ slot_map,
                                    T* __restrict__ cq, T* __restrict__ pages, int q_rank, int kv_rank, int rot_dim,
-                                   float eps) {
+                                   float eps, int pairing) {
   __shared__ float scratch[16];
   const int t = blockIdx.x;
   const T* row = d + static_cast<size_t>(t) * ld;
@@ -562,10 +570,11 @@ __global__ void latent_prep_kernel(const T* __restrict__ d, int ld, const float*
   const int half = dims / 2;
   for (int i = threadIdx.x; i < rot_dim / 2 + (rot_dim & 1); i += blockDim.x) {
     if (i < half) {
+      const RotaryPair p = rotary_pair(i, half, pairing);
       float y1, y2;
-      rotate_pair(to_f32(kr[2 * i]), to_f32(kr[2 * i + 1]), cs[i], cs[half + i], y1, y2);
-      prow[kv_rank + 2 * i] = from_f32<T>(y1);
-      prow[kv_rank + 2 * i + 1] = from_f32<T>(y2);
+      rotate_pair(to_f32(kr[p.a]), to_f32(kr[p.b]), cs[i], cs[half + i], y1, y2);
+      prow[kv_rank + p.a] = from_f32<T>(y1);
+      prow[kv_rank + p.b] = from_f32<T>(y2);
     } else {
       prow[kv_rank + 2 * i] = kr[2 * i];
       if (2 * i + 1 < rot_dim) prow[kv_rank + 2 * i + 1] = kr[2 * i + 1];
@@ -579,7 +588,7 @@ __global__ void latent_prep_kernel(const T* __restrict__ d, int ld, const float*
 template <typename T>
 __global__ void latent_query_rotate_kernel(const T* __restrict__ q, const int32_t* __restrict__ positions,
                                            const float* __restrict__ table, int dims, T* __restrict__ qa, int H,
-                                           int dim, int rot_dim, int kv_rank) {
+                                           int dim, int rot_dim, int kv_rank, int pairing) {
   const int t = blockIdx.x;
   const float* cs = table + static_cast<size_t>(positions[t]) * dims;
   const int half = dims / 2;
@@ -589,10 +598,11 @@ __global__ void latent_query_rotate_kernel(const T* __restrict__ q, const int32_
     const T* src = q + (static_cast<size_t>(t) * H + h) * (dim + rot_dim) + dim;
     T* dst = qa + (static_cast<size_t>(t) * H + h) * (kv_rank + rot_dim) + kv_rank;
     if (i < half) {
+      const RotaryPair p = rotary_pair(i, half, pairing);
       float y1, y2;
-      rotate_pair(to_f32(src[2 * i]), to_f32(src[2 * i + 1]), cs[i], cs[half + i], y1, y2);
-      dst[2 * i] = from_f32<T>(y1);
-      dst[2 * i + 1] = from_f32<T>(y2);
+      rotate_pair(to_f32(src[p.a]), to_f32(src[p.b]), cs[i], cs[half + i], y1, y2);
+      dst[p.a] = from_f32<T>(y1);
+      dst[p.b] = from_f32<T>(y2);
     } else {
       dst[2 * i] = src[2 * i];
       if (2 * i + 1 < rot_dim) dst[2 * i + 1] = src[2 * i + 1];
@@ -694,7 +704,7 @@ __global__ __launch_bounds__(kLatentBlock) void latent_attn_rows_kernel(
     const T* __restrict__ qa, const T* __restrict__ pages, const int32_t* __restrict__ block_tables, int table_width,
     int page_size, const int32_t* __restrict__ q_start, const int32_t* __restrict__ positions,
     const int32_t* __restrict__ ctx_len, int B, const float* __restrict__ sink, float scale, T* __restrict__ out, int H,
-    int kv_rank, int rot_dim) {
+    int kv_rank, int rot_dim, int window) {
   extern __shared__ float smem[];
   const int Dk = kv_rank + rot_dim;
   float* qs = smem;                 // Dk
@@ -719,7 +729,8 @@ __global__ __launch_bounds__(kLatentBlock) void latent_attn_rows_kernel(
   for (int v = 0; v < kCols; ++v) acc[v] = 0.f;
   // the sink: a score without key or value (no sinks: nothing yet in the denominator)
   float m = sink != nullptr ? sink[h] : LYP_NEG_INF, l = sink != nullptr ? 1.0f : 0.f;
-  for (int k0 = 0; k0 < n_keys; k0 += kLatentBlock) {
+  const int lo = window > 0 ? max(0, n_keys - window) : 0;   // with a window: the first key that is seen
+  for (int k0 = lo; k0 < n_keys; k0 += kLatentBlock) {
     const int j = k0 + threadIdx.x;
     float s = LYP_NEG_INF;
     if (j < n_keys) {
@@ -952,17 +963,19 @@ int lyp_mingru_scan_chunks(const float* pre, const float* bz, const float* bx, f
 
 int lyp_latent_prep(const void* d, int ld, const float* wq, const float* wkv, const int32_t* positions,
                     const float* table, int dims, const int32_t* slot_map, void* cq, void* pages, int dtype,
-                    int n_rows, int q_rank, int kv_rank, int rot_dim, float eps, hipStream_t stream) {
+                    int n_rows, int q_rank, int kv_rank, int rot_dim, float eps, int pairing, hipStream_t stream) {
   LYP_REQUIRE(n_rows >= 0 && q_rank > 0 && kv_rank > 0 && rot_dim >= 0 && ld >= q_rank + kv_rank + rot_dim,
               "latent_prep: bad sizes rows=%d q_rank=%d kv_rank=%d rot=%d ld=%d", n_rows, q_rank, kv_rank, rot_dim, ld);
   LYP_REQUIRE(dims >= 0 && dims % 2 == 0 && dims <= rot_dim && (dims == 0 || table != nullptr),
               "latent_prep: %d rotated dimensions of %d", dims, rot_dim);
+  LYP_REQUIRE(pairing == 0 || pairing == 1, "latent_prep: pairing %d", pairing);
   if (n_rows == 0) return 0;
   const int threads = row_threads(std::max(q_rank, kv_rank));
 #define LYP_PREP(T)                                                                                           \
   latent_prep_kernel<T><<<n_rows, threads, 0, stream>>>(static_cast<const T*>(d), ld, wq, wkv, positions,     \
                                                         table, dims, slot_map, static_cast<T*>(cq),           \
-                                                        static_cast<T*>(pages), q_rank, kv_rank, rot_dim, eps)
+                                                        static_cast<T*>(pages), q_rank, kv_rank, rot_dim, eps, \
+                                                        pairing)
   if (dtype == kF32) LYP_PREP(float);
   else if (dtype == kBF16) LYP_PREP(bf16_t);
   else LYP_REQUIRE(false, "latent_prep: unknown dtype %d", dtype);
@@ -1009,20 +1022,22 @@ int lyp_latent_direct_prep(const void* x, int ld, const float* wkv, const int32_
 }
 
 int lyp_latent_query_rotate(const void* q, const int32_t* positions, const float* table, int dims, void* qa,
-                            int dtype, int n_rows, int H, int dim, int rot_dim, int kv_rank, hipStream_t stream) {
+                            int dtype, int n_rows, int H, int dim, int rot_dim, int kv_rank, int pairing,
+                            hipStream_t stream) {
   LYP_REQUIRE(n_rows >= 0 && H > 0 && dim >= 0 && rot_dim >= 0 && kv_rank > 0, "latent_query_rotate: bad sizes");
   LYP_REQUIRE(dims >= 0 && dims % 2 == 0 && dims <= rot_dim && (dims == 0 || table != nullptr),
               "latent_query_rotate: %d rotated dimensions of %d", dims, rot_dim);
+  LYP_REQUIRE(pairing == 0 || pairing == 1, "latent_query_rotate: pairing %d", pairing);
   if (n_rows == 0 || rot_dim == 0) return 0;
   const int threads = 128;
   if (dtype == kF32)
     latent_query_rotate_kernel<float><<<n_rows, threads, 0, stream>>>(static_cast<const float*>(q), positions, table,
                                                                       dims, static_cast<float*>(qa), H, dim, rot_dim,
-                                                                      kv_rank);
+                                                                      kv_rank, pairing);
   else if (dtype == kBF16)
     latent_query_rotate_kernel<bf16_t><<<n_rows, threads, 0, stream>>>(static_cast<const bf16_t*>(q), positions, table,
                                                                        dims, static_cast<bf16_t*>(qa), H, dim, rot_dim,
-                                                                       kv_rank);
+                                                                       kv_rank, pairing);
   else
     LYP_REQUIRE(false, "latent_query_rotate: unknown dtype %d", dtype);
   LYP_LAUNCH_CHECK("latent_query_rotate");
@@ -1032,8 +1047,8 @@ int lyp_latent_query_rotate(const void* q, const int32_t* positions, const float
 int lyp_latent_attn_rows(const void* qa, const void* pages, const int32_t* block_tables, int table_width,
                          int page_size, const int32_t* q_start, const int32_t* positions, const int32_t* ctx_len,
                          int B, const float* sink, float scale, void* out, int dtype, int n_rows, int H, int kv_rank,
-                         int rot_dim, hipStream_t stream) {
-  LYP_REQUIRE(n_rows >= 0 && B > 0 && H > 0 && kv_rank > 0 && rot_dim >= 0 && page_size > 0 && table_width > 0,
+                         int rot_dim, int window, hipStream_t stream) {
+  LYP_REQUIRE(n_rows >= 0 && B > 0 && H > 0 && kv_rank > 0 && rot_dim >= 0 && page_size > 0 && table_width > 0 && window >= 0,
               "latent_attn_rows: bad sizes");
   LYP_REQUIRE(kv_rank <= 8 * kLatentBlock, "latent_attn_rows: latents of up to %d values, not %d", 8 * kLatentBlock,
               kv_rank);
@@ -1043,11 +1058,11 @@ int lyp_latent_attn_rows(const void* qa, const void* pages, const int32_t* block
   if (dtype == kF32)
     latent_attn_rows_kernel<float><<<grid, kLatentBlock, lds, stream>>>(
         static_cast<const float*>(qa), static_cast<const float*>(pages), block_tables, table_width, page_size, q_start,
-        positions, ctx_len, B, sink, scale, static_cast<float*>(out), H, kv_rank, rot_dim);
+        positions, ctx_len, B, sink, scale, static_cast<float*>(out), H, kv_rank, rot_dim, window);
   else if (dtype == kBF16)
     latent_attn_rows_kernel<bf16_t><<<grid, kLatentBlock, lds, stream>>>(
         static_cast<const bf16_t*>(qa), static_cast<const bf16_t*>(pages), block_tables, table_width, page_size,
-        q_start, positions, ctx_len, B, sink, scale, static_cast<bf16_t*>(out), H, kv_rank, rot_dim);
+        q_start, positions, ctx_len, B, sink, scale, static_cast<bf16_t*>(out), H, kv_rank, rot_dim, window);
   else
     LYP_REQUIRE(false, "latent_attn_rows: unknown dtype %d", dtype);
   LYP_LAUNCH_CHECK("latent_attn_rows");

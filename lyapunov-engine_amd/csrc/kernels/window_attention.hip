@@ -198,28 +198,34 @@ constexpr int kRowsBlock = 128;
 constexpr int kRowsCols = 8;   // value columns a thread may own
 
 // One workgroup per (row, head).  The visible keys of a row are walked as one
-// run: the kept first tokens that the window no longer covers, then the window.
-template <typename T>
+// run: the kept first tokens that the window no longer covers, then the window
+// (or the row's chunk: the positions from the last multiple of `chunk` on).
+// `maps` > 1: that many neighbouring query heads read neighbouring key heads of
+// their own and one value head together (H and G count query and key heads; there are
+// G / maps value heads, and query head h reads key head (h / maps / (H / G)) * maps + h % maps).
+// The sums leave in TO, which may be float where they are worked on further.
+template <typename T, typename TO>
 __global__ __launch_bounds__(kRowsBlock) void attn_rows_kernel(
     const T* __restrict__ q, int q_stride, const T* __restrict__ kpool, const T* __restrict__ vpool,
     const int32_t* __restrict__ block_tables, int table_width, int bs, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ positions, const int32_t* __restrict__ ctx_len, int B,
-    const float* __restrict__ sink, float scale, int window, int keep_first, T* __restrict__ out, int out_stride,
-    int H, int G, int D, int V, float cap, const float* __restrict__ slopes) {
+    const float* __restrict__ sink, float scale, int window, int keep_first, TO* __restrict__ out, int out_stride,
+    int H, int G, int D, int V, float cap, const float* __restrict__ slopes, int chunk, int maps) {
   extern __shared__ float smem[];
   float* qs = smem;              // D
   float* ps = smem + D;          // kRowsBlock
   __shared__ float scratch[16];
   const int t = blockIdx.x, h = blockIdx.y;
-  const int g = h / (H / G);
-  T* orow = out + static_cast<size_t>(t) * out_stride + static_cast<size_t>(h) * V;
+  const int gv = h / maps / (H / G), GV = G / maps;       // the value head
+  const int g = gv * maps + h % maps;                     // the key head
+  TO* orow = out + static_cast<size_t>(t) * out_stride + static_cast<size_t>(h) * V;
   const int b = row_owner(q_start, B, t);
   if (t >= q_start[B] || ctx_len[b] <= 0) {   // a row that belongs to no request, or to a padded one
-    for (int i = threadIdx.x; i < V; i += blockDim.x) orow[i] = from_f32<T>(0.f);
+    for (int i = threadIdx.x; i < V; i += blockDim.x) orow[i] = from_f32<TO>(0.f);
     return;
   }
   const int pos = positions[t];
-  const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+  const int lo = window > 0 ? max(0, pos - window + 1) : (chunk > 0 ? pos - pos % chunk : 0);
   const int n_kept = window > 0 ? min(keep_first, lo) : 0;
   const int n_vis = n_kept + (pos - lo + 1);
   const int32_t* table = block_tables + static_cast<size_t>(b) * table_width;
@@ -266,7 +272,7 @@ __global__ __launch_bounds__(kRowsBlock) void attn_rows_kernel(
           const int key = vj < n_kept ? vj : lo + (vj - n_kept);
           const int page = table[key / bs];
           if (page >= 0)
-            a += ps[jj] * to_f32(vpool[((static_cast<size_t>(page) * G + g) * V + col) * bs + key % bs]);
+            a += ps[jj] * to_f32(vpool[((static_cast<size_t>(page) * GV + gv) * V + col) * bs + key % bs]);
         }
         acc[v] = a;
       }
@@ -276,7 +282,7 @@ __global__ __launch_bounds__(kRowsBlock) void attn_rows_kernel(
 #pragma unroll
   for (int v = 0; v < kRowsCols; ++v) {
     const int col = threadIdx.x + v * kRowsBlock;
-    if (col < V) orow[col] = from_f32<T>(acc[v] * inv);
+    if (col < V) orow[col] = from_f32<TO>(acc[v] * inv);
   }
 }
 
@@ -333,24 +339,27 @@ int lyp_qk_norm_rope_kv(void* qkv, int ld, int dtype, const float* wq, const flo
 int lyp_attn_rows(const void* q, int q_stride, const void* kpool, const void* vpool, const int32_t* block_tables,
                   int table_width, int bs, const int32_t* q_start, const int32_t* positions, const int32_t* ctx_len,
                   int B, const float* sink, float scale, int window, int keep_first, void* out, int out_stride,
-                  int dtype, int n_rows, int H, int G, int D, int V, float cap, const float* slopes,
-                  hipStream_t stream) {
+                  int dtype, int n_rows, int H, int G, int D, int V, float cap, const float* slopes, int chunk,
+                  int maps, int out_f32, hipStream_t stream) {
   LYP_REQUIRE(n_rows >= 0 && B > 0 && H > 0 && G > 0 && H % G == 0 && D > 0 && V > 0 && bs > 0 && table_width > 0,
               "attn_rows: bad sizes");
   LYP_REQUIRE(V <= kRowsCols * kRowsBlock, "attn_rows: values of up to %d, not %d", kRowsCols * kRowsBlock, V);
   LYP_REQUIRE(window >= 0 && keep_first >= 0 && q_stride >= H * D && out_stride >= H * V,
               "attn_rows: window %d, kept %d, strides %d %d", window, keep_first, q_stride, out_stride);
   LYP_REQUIRE(H <= 65535, "attn_rows: too many heads for one launch");
+  LYP_REQUIRE(chunk >= 0 && (chunk == 0 || window == 0), "attn_rows: a window of %d and a chunk of %d", window, chunk);
+  LYP_REQUIRE(maps >= 1 && H % maps == 0 && G % maps == 0, "attn_rows: %d/%d heads in groups of %d", H, G, maps);
   if (n_rows == 0) return 0;
   const size_t lds = sizeof(float) * (D + kRowsBlock);
   dim3 grid(n_rows, H);
-#define LYP_ROWS(T)                                                                                             \
-  attn_rows_kernel<T><<<grid, kRowsBlock, lds, stream>>>(                                                       \
+#define LYP_ROWS(T, TO)                                                                                         \
+  attn_rows_kernel<T, TO><<<grid, kRowsBlock, lds, stream>>>(                                                   \
       static_cast<const T*>(q), q_stride, static_cast<const T*>(kpool), static_cast<const T*>(vpool),           \
       block_tables, table_width, bs, q_start, positions, ctx_len, B, sink, scale, window, keep_first,           \
-      static_cast<T*>(out), out_stride, H, G, D, V, cap, slopes)
-  if (dtype == kF32) LYP_ROWS(float);
-  else if (dtype == kBF16) LYP_ROWS(bf16_t);
+      static_cast<TO*>(out), out_stride, H, G, D, V, cap, slopes, chunk, maps)
+  if (dtype == kF32) LYP_ROWS(float, float);
+  else if (dtype == kBF16 && out_f32) LYP_ROWS(bf16_t, float);
+  else if (dtype == kBF16) LYP_ROWS(bf16_t, bf16_t);
   else LYP_REQUIRE(false, "attn_rows: unknown dtype %d", dtype);
 #undef LYP_ROWS
   LYP_LAUNCH_CHECK("attn_rows");

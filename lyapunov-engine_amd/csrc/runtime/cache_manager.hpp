@@ -6,8 +6,8 @@
 // when a request ends.  Added here:
 //   * groups: layers with different needs (all keys, or a window of them) keep
 //     pages of their own, with a pool, a page size and a block table per group;
-//   * a window group gives a page back as soon as every later token is out of
-//     its reach, and takes it again for another request;
+//   * a group of windowed or chunked layers gives a page back as soon as every
+//     later token is out of its reach, and takes it again for another request;
 //   * growth by any number of tokens (the reference grows by one token and only
 //     when total % block_size == 1, block_manager.cpp:56-79);
 //   * a slot of fixed-size state per live request, for mixers that carry state
@@ -28,6 +28,11 @@ struct GroupSpec {
   int page_size = 16;
   int window = 0;  // 0: every key is kept; W > 0: a token sees keys (pos - W, pos]
   int keep_first = 0;  // with a window: a request's first keep_first keys stay visible, so their pages are never given back
+  int chunk = 0;  // C > 0 (and no window): a token sees the keys of its own run of C positions, counted from 0
+
+  bool keeps_all() const { return window <= 0 && chunk <= 0; }
+  // The first key a token at position `pos` sees, kept first keys apart.
+  int first_seen(int pos) const { return window > 0 ? pos - window + 1 : (chunk > 0 ? pos - pos % chunk : 0); }
 };
 
 class CacheManager {
@@ -65,15 +70,15 @@ class CacheManager {
   // Takes the pages for positions < new_len.  Throws, and changes nothing, if a
   // group runs out.
   void extend(int64_t id, int new_len);
-  // The step that computed positions < new_len is done: window groups give
-  // back the pages no later token can see.
+  // The step that computed positions < new_len is done: groups that do not keep
+  // every key give back the pages no later token can see.
   void commit(int64_t id, int new_len);
   // Gives everything back.  Unknown ids are ignored
   // (csrc/engine/block_manager.cpp:83-86).
   void free(int64_t id);
   void reset();
 
-  // Logical page -> physical page, -1 where a window group gave the page back.
+  // Logical page -> physical page, -1 where a window or chunk group gave the page back.
   const std::vector<int32_t>& table(int64_t id, int g) const;
   int state_slot(int64_t id) const;
   int ref_count(int g, int page) const { return ref_.at(g).at(page); }

@@ -36,6 +36,7 @@ static int one_round(std::mt19937& rng) {
   const int window = pick(0, 2) == 0 ? pick(2, 3 * page) : 0;
   std::vector<GroupSpec> groups{{pages, page, 0}};
   if (window) groups.push_back({pages, page, window, pick(0, 1) ? pick(1, 2 * page) : 0});   // some windows keep first tokens
+  if (pick(0, 2) == 0) groups.push_back({pages, page, 0, 0, pick(1, 3 * page)});                                          // a group of chunked layers
   CacheManager cache(groups, pick(2, 6));
   SchedulerConfig cfg;
   cfg.max_num_seqs = pick(1, 6);

@@ -18,7 +18,7 @@ class EngineCore:
                  block_size: int = 16, num_state_slots: int = 64, cache_groups: Optional[list] = None):
         """``cache_groups``: (pages, page size) for each of the model's cache
         groups in turn (``model.cache_layout().groups``: layers whose keys and
-        values have one shape and one window share a group), where they are to
+        values have one shape and one reach share a group), where they are to
         differ from ``num_blocks`` and ``block_size``; None in place of a pair
         keeps those.  A group of windowed layers needs far fewer pages than one
         that keeps every key."""
@@ -30,7 +30,7 @@ class EngineCore:
         self.block_size = block_size
         layout = model.cache_layout()
         sizes = self.group_sizes(layout, num_blocks, block_size, cache_groups)
-        groups = [GroupConfig(pages, size, gl.spec.window, gl.spec.keep_first)
+        groups = [GroupConfig(pages, size, gl.spec.window, gl.spec.keep_first, gl.spec.chunk)
                   for (pages, size), gl in zip(sizes, layout.groups)]
         # A model without keys and values (state only) still gets a group, so
         # that requests have a length and the manager one code path.
@@ -52,13 +52,13 @@ class EngineCore:
               max_model_len: Optional[int]) -> int:
         """The positions a request of this engine can ever reach: its model
         length, and the pool of every cache group that keeps all of a request's
-        tokens (a group of windowed layers gives pages back as the window
-        passes, so its pool bounds the window and the step's portion, not the
-        request; a model that keeps everything in windows or in state is bound
+        tokens (a group of windowed or chunked layers gives pages back as the
+        window or chunk passes, so its pool bounds that and the step's portion,
+        not the request; a model that keeps everything so or in state is bound
         by the model length alone)."""
         layout = model.cache_layout()
         sizes = EngineCore.group_sizes(layout, num_blocks, block_size, cache_groups)
-        bounds = [pages * size for (pages, size), gl in zip(sizes, layout.groups) if gl.spec.window == 0]
+        bounds = [pages * size for (pages, size), gl in zip(sizes, layout.groups) if gl.spec.keeps_all]
         reach = min(bounds) if bounds else model.spec.max_position
         return min(reach, int(max_model_len)) if max_model_len else reach
 

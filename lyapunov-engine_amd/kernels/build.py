@@ -2,7 +2,7 @@
 
 There is one library of kernels whose sizes are run-time values (``core``), one
 attention library per head size (``attn_hd<N>``; the head size is a compile-time
-constant there), one of host code around the vendor's GEMM library (``blas``),
+constant there) and others likewise per pair of sizes (``latent_*``, ``paired_*``), one of host code around the vendor's GEMM library (``blas``),
 and one library of host code (``runtime``: cache manager and scheduler).  A library's file name carries a hash of its sources and flags, so a
 changed source is never served by an old binary; what is missing is compiled on
 first use, with a progress line now and then.
@@ -41,6 +41,7 @@ CORE_SOURCES = ["kernels/errors.hip", "kernels/elementwise.hip", "kernels/sequen
                 "kernels/linear_scan.hip", "kernels/qkv_prepare.hip", "kernels/recurrent_rows.hip", "kernels/stream_rows.hip"]
 ATTN_SOURCES = ["kernels/errors.hip", "kernels/attention.hip"]
 LATENT_SOURCES = ["kernels/errors.hip", "kernels/latent_attention.hip"]
+PAIRED_SOURCES = ["kernels/errors.hip", "kernels/paired_attention.hip"]
 BLAS_SOURCES = ["kernels/errors.hip", "kernels/library_gemm.hip"]   # host code around the vendor's GEMM library
 RUNTIME_SOURCES = ["runtime/cache_manager.cpp", "runtime/scheduler.cpp", "runtime/c_api.cpp"]
 
@@ -50,6 +51,8 @@ PREBUILT_HEAD_DIMS = (16, 32, 48, 64, 80, 96, 128, 256)
 # (latent, rotated part) sizes of the latent attention library compiled ahead of time; others on first use.
 PREBUILT_LATENT_SIZES = ((16, 0), (16, 16), (16, 32), (32, 0), (32, 16), (32, 48), (48, 0), (48, 16), (64, 16), (64, 32),
                          (64, 64), (96, 16), (128, 16), (128, 32), (256, 32), (512, 32))
+# (key, value) sizes of the differential attention library compiled ahead of time; others on first use.
+PREBUILT_PAIRED_SIZES = ((16, 16), (16, 32), (32, 16), (32, 48), (32, 64), (48, 80), (64, 128), (128, 256))
 
 _lock = threading.Lock()
 
@@ -206,6 +209,15 @@ def latent_attention_library(kv_rank: int, rot_dim: int, force: bool = False) ->
                          defines={"LYP_LATENT_KV": str(kv_rank), "LYP_LATENT_RD": str(rot_dim)}, force=force)
 
 
+def paired_attention_library(key_dim: int, value_dim: int, force: bool = False) -> Path:
+    """The matrix-core differential attention for one pair of head sizes (compile-time constants there)."""
+    if key_dim % 16 or value_dim % 16 or not 16 <= key_dim <= 128 or not 16 <= value_dim <= 256:
+        raise ValueError(f"the differential attention kernels take keys of 16 to 128 values and values of up to 256, in "
+                         f"multiples of 16, not {key_dim} and {value_dim}")
+    return build_library(f"lyp_paired_k{key_dim}_v{value_dim}", PAIRED_SOURCES, hip=True,
+                         defines={"LYP_KEY_DIM": str(key_dim), "LYP_VALUE_DIM": str(value_dim)}, force=force)
+
+
 def blas_library(force: bool = False) -> Path:
     rocm = os.environ.get("ROCM_PATH", "/opt/rocm")
     return build_library("lyp_blas", BLAS_SOURCES, hip=True, force=force,
@@ -262,4 +274,6 @@ def build_all(force: bool = True) -> list[Path]:
         out.append(attention_library(hd, force))
     for kv, rd in PREBUILT_LATENT_SIZES:
         out.append(latent_attention_library(kv, rd, force))
+    for kd, vd in PREBUILT_PAIRED_SIZES:
+        out.append(paired_attention_library(kd, vd, force))
     return out

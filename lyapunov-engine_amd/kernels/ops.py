@@ -21,6 +21,7 @@ F32, BF16 = 0, 1
 _CODE = {torch.float32: F32, torch.bfloat16: BF16}
 
 STORE_ACT, STORE_F32, ACCUM_F32 = 0, 1, 2
+PAIRINGS = {"neighbours": 0, "halves": 1}   # which two values a rotation turns together: (2i, 2i + 1) or (i, i + half)
 
 
 class KernelError(RuntimeError):
@@ -100,26 +101,27 @@ def core() -> ctypes.CDLL:
         lib.lyp_mingru_scan_chunks.argtypes = [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                                c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_longlong, c_void_p]
         lib.lyp_latent_prep.argtypes = [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p,
-                                        c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p]
+                                        c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p]
         lib.lyp_latent_query_rotate.argtypes = [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int,
-                                                c_int, c_int, c_int, c_void_p]
+                                                c_int, c_int, c_int, c_int, c_void_p]
         lib.lyp_latent_attn_rows.argtypes = [c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p,
                                              c_int, c_void_p, c_float, c_void_p, c_int, c_int, c_int, c_int, c_int,
-                                             c_void_p]
+                                             c_int, c_void_p]
         lib.lyp_qk_norm_rope_kv.argtypes = [c_void_p, c_int, c_int, c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_int,
                                             c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
                                             c_void_p]
         lib.lyp_attn_rows.argtypes = [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p,
                                       c_void_p, c_int, c_void_p, c_float, c_int, c_int, c_void_p, c_int, c_int, c_int,
-                                      c_int, c_int, c_int, c_int, c_float, c_void_p, c_void_p]
+                                      c_int, c_int, c_int, c_int, c_float, c_void_p, c_int, c_int, c_int, c_void_p]
         lib.lyp_stream_add.argtypes = [c_void_p, c_void_p, c_int, c_int, c_void_p, c_longlong, c_void_p]
         lib.lyp_moe_route.argtypes = [c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p]
         lib.lyp_moe_route_splits.argtypes = [c_int, c_int]
         lib.lyp_moe_route_fused.argtypes = [c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
-                                            c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p]
+                                            c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_float, c_int,
+                                            c_void_p, c_void_p]
         lib.lyp_moe_route_sort.argtypes = [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_void_p,
                                            c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
-                                           c_void_p]
+                                           c_int, c_float, c_int, c_void_p, c_void_p]
         lib.lyp_moe_tile_rows.argtypes = [c_int, c_int]
         lib.lyp_moe_most_tiles.argtypes = [c_int, c_int, c_int]
         lib.lyp_moe_sort.argtypes = [c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
@@ -140,9 +142,9 @@ def core() -> ctypes.CDLL:
                                        c_void_p]
         lib.lyp_latent_direct_prep.argtypes = [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
                                                c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p]
-        lib.lyp_glu_clamped.argtypes = [c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_float, c_void_p]
-        lib.lyp_moe_combine.argtypes = [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int,
-                                        c_int, c_void_p]
+        lib.lyp_glu_clamped.argtypes = [c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_float, c_float, c_int, c_void_p]
+        lib.lyp_moe_combine.argtypes = [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
+                                        c_int, c_int, c_void_p]
         lib.lyp_group_rmsnorm.argtypes = [c_void_p, c_void_p, c_int, c_int, c_longlong, c_void_p, c_void_p, c_void_p, c_int,
                                           c_void_p, c_int, c_int, c_int, c_float, c_void_p]
         lib.lyp_add_sinusoid.argtypes = [c_void_p, c_void_p, c_int, c_int, c_double, c_void_p]
@@ -164,7 +166,14 @@ def core() -> ctypes.CDLL:
                                        c_void_p, c_float, c_int, c_int, c_int, c_void_p]
         lib.lyp_qkv_prepare.argtypes = [c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_float, c_void_p, c_void_p,
                                         c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p,
-                                        c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p]
+                                        c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
+                                        c_void_p]
+        lib.lyp_head_difference.argtypes = [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_float,
+                                            c_float, c_void_p]
+        lib.lyp_gemm_glu.argtypes = [c_void_p, c_void_p, c_int, c_int, c_float, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
+                                     c_int, c_int, c_int, c_float, c_float, c_float, c_void_p]
+        lib.lyp_gemm_normed.argtypes = [c_void_p, c_int, c_void_p, c_int, c_int, c_float, c_void_p, c_void_p, c_int, c_int,
+                                        c_int, c_int, c_int, c_int, c_int, c_void_p]
         lib.lyp_shift_mix.argtypes = [c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                       c_int, c_int, c_int, c_int, c_void_p]
         lib.lyp_skip_gate_group_norm.argtypes = [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
@@ -609,6 +618,28 @@ def linear_swiglu(x: torch.Tensor, w: torch.Tensor, interleave: int) -> torch.Te
     return swiglu(gate_up, out, interleave)
 
 
+def linear_glu(x: torch.Tensor, w: torch.Tensor, interleave: int, limit: float, slope: float, plus: float) -> torch.Tensor:
+    """g * sigmoid(slope * g) * (u + plus), g = min(x @ Wgate.T, limit), u = clamp(x @ Wup.T, -limit, limit), for the
+    fused matrix w [2 I, K] laid out as ``swiglu`` describes.  With few rows and interleave 8 it is one kernel;
+    ``x`` may be a ``PendingNorm``, which that kernel norms on its way."""
+    I, M = w.shape[0] // 2, x.shape[0]
+    p = x if isinstance(x, PendingNorm) else None
+    rows, dtype = (p.xs, p.dtype) if p is not None else (x, x.dtype)
+    if interleave == 8 and rows.shape[1] == w.shape[1] and _few_rows_product(M, w, dtype):
+        ssq = p.ssq_part if p is not None else None
+        _dev(rows, ssq, w)
+        out = torch.empty((M, I), dtype=dtype, device=w.device)
+        lib = core()
+        rc = lib.lyp_gemm_glu(_p(rows), _p(ssq), ssq.shape[0] if p is not None else 0, rows.shape[1], p.eps if p is not None else 0.0,
+                              _p(w), _p(out), _code(dtype), M, w.shape[0], w.shape[1], rows.stride(0), w.stride(0), I,
+                              float(limit), float(slope), float(plus), _stream())
+        if rc == 0:
+            return out
+        if rc < 0:
+            _check(rc, lib)
+    return glu_clamped(linear(p.run() if p is not None else x, w, out_dtype=dtype), limit, slope, plus, interleave)
+
+
 def cast(x: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
     if x.dtype == dtype:
         return x
@@ -825,8 +856,23 @@ def linear(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype | None = Non
     ``rmsnorm`` takes such a delta and adds the slices up, ``sum_parts`` does it
     for any other consumer.  With ``pending`` (the result will only be added to
     the residual stream) a product of few rows is not run at all but handed on
-    as a ``PendingLinear``."""
+    as a ``PendingLinear``.  ``x`` may be a ``PendingNorm``, which the product of few rows norms on its way."""
     out_dtype = out_dtype or x.dtype
+    if isinstance(x, PendingNorm):
+        p, M = x, x.shape[0]
+        if not pending and p.h.shape[1] == w.shape[1] and out_dtype in (p.dtype, torch.float32) and \
+                _few_rows_product(M, w, p.dtype):
+            _dev(p.xs, p.ssq_part, w)
+            out = torch.empty((M, w.shape[0]), dtype=out_dtype, device=w.device)
+            lib = core()
+            rc = lib.lyp_gemm_normed(_p(p.xs), p.xs.stride(0), _p(p.ssq_part), p.ssq_part.shape[0], p.h.shape[1], p.eps, _p(w),
+                                     _p(out), _code(p.dtype), int(out_dtype == torch.float32), M, w.shape[0], w.shape[1],
+                                     w.stride(0), out.stride(0), _stream())
+            if rc == 0:
+                return out
+            if rc < 0:
+                _check(rc, lib)
+        x = p.run()
     if pending and x.shape[0] <= PENDING_MAX_ROWS and _few_rows_product(x.shape[0], w, x.dtype):
         return PendingLinear(x, w, out_dtype)
     if w.dtype != x.dtype:
@@ -1097,10 +1143,11 @@ def mingru_scan_workspace(T: int, B: int, W: int) -> int:
 
 def latent_prep(d: torch.Tensor, wq: torch.Tensor, wkv: torch.Tensor, positions: torch.Tensor,
                 table: torch.Tensor | None, slot_map: torch.Tensor, cq: torch.Tensor, pages: torch.Tensor, *,
-                q_rank: int, kv_rank: int, rot_dim: int, eps: float) -> None:
+                q_rank: int, kv_rank: int, rot_dim: int, eps: float, pairing: str = "neighbours") -> None:
     """From the down-projections of a step's rows (d [T, q_rank + kv_rank + rot_dim]): the normed
     query latent into cq, and the normed key/value latent with the position-rotated shared key part
-    into each token's page slot (pages [pages, page size, kv_rank + rot_dim])."""
+    into each token's page slot (pages [pages, page size, kv_rank + rot_dim]).  ``pairing``: which two
+    values turn together, (2i, 2i + 1) ("neighbours") or (i, i + half) ("halves")."""
     _dev(d, wq, wkv, positions, table, slot_map, cq, pages)
     _f32(wq, wkv, table)
     T = d.shape[0]
@@ -1112,7 +1159,7 @@ def latent_prep(d: torch.Tensor, wq: torch.Tensor, wkv: torch.Tensor, positions:
     lib = core()
     _check(lib.lyp_latent_prep(_p(d), d.stride(0), _p(wq), _p(wkv), _p(positions), _p(table), dims, _p(slot_map),
                                _p(cq), _p(pages), _code(d.dtype), T, q_rank, kv_rank, rot_dim, float(eps),
-                               _stream()), lib)
+                               PAIRINGS[pairing], _stream()), lib)
 
 
 def latent_direct_prep(x: torch.Tensor, wkv: torch.Tensor, positions: torch.Tensor, table: torch.Tensor | None,
@@ -1136,9 +1183,10 @@ def latent_direct_prep(x: torch.Tensor, wkv: torch.Tensor, positions: torch.Tens
 
 
 def latent_query_rotate(q: torch.Tensor, positions: torch.Tensor, table: torch.Tensor | None, qa: torch.Tensor, *,
-                        num_heads: int, dim: int, rot_dim: int, kv_rank: int) -> None:
+                        num_heads: int, dim: int, rot_dim: int, kv_rank: int, pairing: str = "neighbours") -> None:
     """The rotated part of every query head (q [T, H (dim + rot_dim)], the last rot_dim of each head),
-    turned by the token's position, into qa[:, head, kv_rank:] (qa [T, H, kv_rank + rot_dim])."""
+    turned by the token's position, into qa[:, head, kv_rank:] (qa [T, H, kv_rank + rot_dim]).  ``pairing``: see
+    ``latent_prep``."""
     _dev(q, positions, table, qa)
     _f32(table)
     T = q.shape[0]
@@ -1148,15 +1196,16 @@ def latent_query_rotate(q: torch.Tensor, positions: torch.Tensor, table: torch.T
         raise KernelError(f"latent_query_rotate: q {tuple(q.shape)}, qa {tuple(qa.shape)}")
     lib = core()
     _check(lib.lyp_latent_query_rotate(_p(q), _p(positions), _p(table), dims, _p(qa), _code(q.dtype), T, num_heads,
-                                       dim, rot_dim, kv_rank, _stream()), lib)
+                                       dim, rot_dim, kv_rank, PAIRINGS[pairing], _stream()), lib)
 
 
 def latent_attn_rows(qa: torch.Tensor, pages: torch.Tensor, block_tables: torch.Tensor, q_start: torch.Tensor,
                      positions: torch.Tensor, ctx_len: torch.Tensor, sink: torch.Tensor | None, scale: float,
-                     out: torch.Tensor, *, kv_rank: int, rot_dim: int) -> torch.Tensor:
+                     out: torch.Tensor, *, kv_rank: int, rot_dim: int, window: int = 0) -> torch.Tensor:
     """Causal attention of every row over its request's latents in the pages, all heads sharing one
     key per token (the page row) whose first kv_rank values are also the value; the softmax's
-    denominator holds exp(sink[head]) as well (``sink`` None: nothing more).  Any sizes; a workgroup per (row, head)."""
+    denominator holds exp(sink[head]) as well (``sink`` None: nothing more).  ``window`` > 0: a row sees its own key and
+    the window - 1 before it.  Any sizes; a workgroup per (row, head)."""
     _dev(qa, pages, block_tables, q_start, positions, ctx_len, sink, out)
     _f32(sink)
     T, H, Dk = qa.shape
@@ -1169,7 +1218,7 @@ def latent_attn_rows(qa: torch.Tensor, pages: torch.Tensor, block_tables: torch.
     lib = core()
     _check(lib.lyp_latent_attn_rows(_p(qa), _p(pages), _p(block_tables), block_tables.shape[1], pages.shape[1],
                                     _p(q_start), _p(positions), _p(ctx_len), B, _p(sink), float(scale), _p(out),
-                                    _code(qa.dtype), T, H, kv_rank, rot_dim, _stream()), lib)
+                                    _code(qa.dtype), T, H, kv_rank, rot_dim, int(window), _stream()), lib)
     return out
 
 
@@ -1187,7 +1236,7 @@ def latent_lib(kv_rank: int, rot_dim: int) -> ctypes.CDLL:
         lib.lyp_latent_tile_keys.argtypes = [c_int]
         lib.lyp_latent_attn.argtypes = [c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int,
                                         c_void_p, c_float, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
-                                        c_void_p, c_void_p, c_int, c_void_p]
+                                        c_void_p, c_void_p, c_int, c_int, c_void_p]
         lib.lyp_latent_heads_out.argtypes = [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int,
                                              c_int, c_int, c_int, c_void_p]
         _latent[(kv_rank, rot_dim)] = lib
@@ -1201,14 +1250,18 @@ def latent_attn_fits_matrix_cores(kv_rank: int, rot_dim: int) -> bool:
 
 
 def latent_attn_launch(T: int, B: int, H: int, max_ctx: int, dtype: torch.dtype, kv_rank: int, rot_dim: int,
-                       n_parts: int | None = None) -> dict:
+                       n_parts: int | None = None, window: int = 0) -> dict:
     """The launch shape of ``latent_attn`` for a step of T rows of B requests with contexts of up
     to max_ctx: row groups, partitions of the keys, keys per partition, and the floats of the
-    partitions' workspaces (host values only)."""
+    partitions' workspaces (host values only).  With a window a row group's keys are at most those of the
+    window, of the group's tokens, and of the tile that the first of them stands in."""
     lib = latent_lib(kv_rank, rot_dim)
     code = _code(dtype)
     row_groups = -(-T * H // 64) + B
     tile = lib.lyp_latent_tile_keys(code)
+    if window:
+        tokens = min(T, (64 + H - 2) // H + 1)
+        max_ctx = min(max_ctx, window + tokens - 1 + tile - 1)
     if n_parts is None:
         n_parts = lib.lyp_latent_plan(row_groups, max_ctx, code)
     part_keys = max(tile, -(-(-(-max_ctx // n_parts)) // tile) * tile)
@@ -1220,12 +1273,13 @@ def latent_attn_launch(T: int, B: int, H: int, max_ctx: int, dtype: torch.dtype,
 def latent_attn(qa: torch.Tensor, pages: torch.Tensor, block_tables: torch.Tensor, q_start: torch.Tensor,
                 positions: torch.Tensor, ctx_len: torch.Tensor, sink: torch.Tensor | None, scale: float, out: torch.Tensor,
                 launch: dict, part_o: torch.Tensor | None = None, part_ml: torch.Tensor | None = None, *,
-                kv_rank: int, rot_dim: int, merge: bool = True) -> torch.Tensor:
+                kv_rank: int, rot_dim: int, merge: bool = True, window: int = 0) -> torch.Tensor:
     """``latent_attn_rows`` on the matrix cores (sizes in multiples of 16), a prompt's rows and
     single tokens alike; ``launch`` comes from ``latent_attn_launch`` for a bound on the step's
     contexts that the caller guarantees (keys beyond n_parts * part_keys would be left out).
     ``merge=False``: with several partitions ``out`` is left unwritten and the partitions' results
-    stay in ``part_o`` / ``part_ml`` for ``latent_heads_out`` to merge."""
+    stay in ``part_o`` / ``part_ml`` for ``latent_heads_out`` to merge.  ``window``: as for
+    ``latent_attn_rows``; the launch was made with the same."""
     _dev(qa, pages, block_tables, q_start, positions, ctx_len, sink, out, part_o, part_ml)
     _f32(sink, part_o, part_ml)
     T, H, Dk = qa.shape
@@ -1242,7 +1296,7 @@ def latent_attn(qa: torch.Tensor, pages: torch.Tensor, block_tables: torch.Tenso
     _check(lib.lyp_latent_attn(_p(qa), _p(pages), _p(block_tables), block_tables.shape[1], pages.shape[1], _p(q_start),
                                _p(positions), _p(ctx_len), B, _p(sink), float(scale), _p(out), _code(qa.dtype), T, H,
                                launch["row_groups"], launch["n_parts"], launch["part_keys"], _p(part_o), _p(part_ml),
-                               int(merge), _stream()), lib)
+                               int(merge), int(window), _stream()), lib)
     return out
 
 
@@ -1385,6 +1439,154 @@ def attn_decode(q: torch.Tensor, out: torch.Tensor, kpool: torch.Tensor, vpool: 
     return out
 
 
+# ------------------------------------------------------ two maps a head, one taken off the other
+_paired: dict = {}
+MAPS = 2
+
+
+def paired_lib(key_dim: int, value_dim: int) -> ctypes.CDLL:
+    lib = _paired.get((key_dim, value_dim))
+    if lib is None:
+        lib = _load(build.paired_attention_library(key_dim, value_dim))
+        lib.lyp_last_error.restype = ctypes.c_char_p
+        if (lib.lyp_paired_key_dim(), lib.lyp_paired_value_dim()) != (key_dim, value_dim):
+            raise KernelError(f"differential attention library for sizes {key_dim}, {value_dim} reports others")
+        lib.lyp_paired_decode_plan.argtypes = [c_int, c_int, c_int, c_int]
+        lib.lyp_paired_prefill_plan.argtypes = [c_int, c_int, c_int, c_int, c_int]
+        lib.lyp_paired_prefill.argtypes = [c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int,
+                                           c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
+                                           c_float, c_float, c_float, c_float, c_void_p, c_int, c_void_p, c_void_p, c_int,
+                                           c_void_p]
+        lib.lyp_paired_decode.argtypes = [c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int,
+                                          c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
+                                          c_int, c_int, c_int, c_float, c_float, c_float, c_float, c_void_p, c_int, c_void_p]
+        _paired[(key_dim, value_dim)] = lib
+    return lib
+
+
+def paired_attn_fits_matrix_cores(key_dim: int, value_dim: int) -> bool:
+    return key_dim % 16 == 0 and value_dim % 16 == 0 and 16 <= key_dim <= 128 and 16 <= value_dim <= 256
+
+
+def visible_keys(max_ctx: int, window: int, chunk: int, tokens: int = 1) -> int:
+    """Most keys that ``tokens`` neighbouring tokens of a request of up to ``max_ctx`` see between them, and the 15
+    before them that a block of 16 keys may begin with."""
+    reach = window or chunk
+    return min(max_ctx, reach + tokens - 1 + 15) if reach else max_ctx
+
+
+def paired_decode_launch(n_dec: int, max_ctx: int, *, num_heads: int, num_kv_heads: int, dim: int, vdim: int,
+                         window: int = 0, chunk: int = 0) -> dict:
+    """Keys per workgroup, the most partitions of a request and the floats of their workspaces."""
+    seen = max(1, visible_keys(max_ctx, window, chunk))
+    part = paired_lib(dim, vdim).lyp_paired_decode_plan(n_dec, seen, num_heads, num_kv_heads)
+    parts = max(1, -(-seen // part))
+    n = n_dec * num_heads * MAPS * parts if parts > 1 else 0
+    return dict(part_keys=part, max_parts=parts, part_o=n * vdim, part_ml=n * 2)
+
+
+def paired_prefill_launch(n_tiles: int, most_keys: int, dtype: torch.dtype, *, num_heads: int, num_kv_heads: int, dim: int,
+                          vdim: int, window: int = 0, chunk: int = 0) -> dict:
+    """In how many runs every tile's keys are cut and the floats of the runs' workspaces; ``most_keys``: what the
+    last of the tiles would see without a window or chunk."""
+    seen = visible_keys(most_keys, window, chunk, tokens=64)
+    parts = paired_lib(dim, vdim).lyp_paired_prefill_plan(n_tiles, seen, num_heads, num_kv_heads, _code(dtype))
+    n = n_tiles * 64 * num_heads * MAPS * parts if parts > 1 else 0
+    return dict(parts=parts, part_o=n * vdim, part_ml=n * 2)
+
+
+def _paired_check(q, out, kpool, vpool, block_tables, gate, H, G, dim, vdim) -> int:
+    _dev(out, kpool, vpool, block_tables)
+    n_pages, bs = kpool.shape[0], kpool.shape[2]
+    if not q.is_cuda or q.dim() != 2 or q.stride(1) != 1 or q.shape[1] != H * MAPS * dim or \
+            tuple(out.shape) != (q.shape[0], H * vdim) or tuple(kpool.shape) != (n_pages, MAPS * G, bs, dim) or \
+            tuple(vpool.shape) != (n_pages, G, vdim, bs) or len({q.dtype, out.dtype, kpool.dtype, vpool.dtype}) != 1 or \
+            block_tables.dtype != torch.int32 or block_tables.dim() != 2:
+        raise KernelError(f"differential attention: q {tuple(q.shape)}, out {tuple(out.shape)}, pools {tuple(kpool.shape)} / "
+                          f"{tuple(vpool.shape)} for {H}/{G} heads of {dim}/{vdim}")
+    if gate is not None:
+        _rows_view(gate, "differential attention")
+        _f32(gate)
+        if tuple(gate.shape) != tuple(out.shape):
+            raise KernelError(f"differential attention: gate {tuple(gate.shape)} beside {tuple(out.shape)}")
+    return bs
+
+
+def paired_prefill(q: torch.Tensor, out: torch.Tensor, kpool: torch.Tensor, vpool: torch.Tensor,
+                   block_tables: torch.Tensor, q_start: torch.Tensor, ctx_len: torch.Tensor, tile_seq: torch.Tensor,
+                   tile_q0: torch.Tensor, n_tiles: int, launch: dict, part_o: torch.Tensor | None = None,
+                   part_ml: torch.Tensor | None = None, *, num_heads: int, num_kv_heads: int, dim: int, vdim: int,
+                   scale: float, take_off: float, post: float, eps: float, gate: torch.Tensor | None = None,
+                   window: int = 0, chunk: int = 0) -> torch.Tensor:
+    """Differential attention of the step's tiles of 64 new tokens over the paged cache.  q [T, H 2 dim]: per head
+    the two maps' queries; keys in the pages likewise, [pages, 2 G, page, dim]; values [pages, G, vdim, page].
+    out [T, H vdim]: with a1, a2 the two maps' softmax sums, o = a1 - take_off * a2, o / rms(o) * post, times the
+    sigmoid of ``gate`` (float [T, H vdim], possibly a column range; None: not gated).  A token sees the keys
+    before it, those of a window, or those of its own chunk.  ``launch``: from ``paired_prefill_launch``."""
+    bs = _paired_check(q, out, kpool, vpool, block_tables, gate, num_heads, num_kv_heads, dim, vdim)
+    _dev(q_start, ctx_len, tile_seq, tile_q0, part_o, part_ml)
+    parts = launch["parts"]
+    if parts > 1 and (part_o is None or part_ml is None or part_o.dtype != torch.float32 or part_ml.dtype != torch.float32 or
+                      part_o.numel() < n_tiles * 64 * num_heads * MAPS * parts * vdim or
+                      part_ml.numel() < n_tiles * 64 * num_heads * MAPS * parts * 2):
+        raise KernelError("differential attention: the workspace for the runs of the keys is missing or too small")
+    if tile_seq.numel() < n_tiles or tile_q0.numel() < n_tiles:
+        raise KernelError(f"differential attention: {tile_seq.numel()} tiles listed, {n_tiles} asked for")
+    lib = paired_lib(dim, vdim)
+    _check(lib.lyp_paired_prefill(_p(q), q.stride(0), _p(out), out.stride(0), _p(kpool), _p(vpool), _code(q.dtype),
+                                  _p(block_tables), block_tables.shape[1], _p(q_start), _p(ctx_len), _p(tile_seq),
+                                  _p(tile_q0), n_tiles, num_heads, num_kv_heads, bs, int(window), int(chunk), float(scale),
+                                  float(take_off), float(eps), float(post), _p(gate), gate.stride(0) if gate is not None else 0,
+                                  _p(part_o), _p(part_ml), parts, _stream()), lib)
+    return out
+
+
+def paired_decode(q: torch.Tensor, out: torch.Tensor, kpool: torch.Tensor, vpool: torch.Tensor, block_tables: torch.Tensor,
+                  q_start: torch.Tensor, ctx_len: torch.Tensor, dec_seqs: torch.Tensor | None, n_seqs: int, launch: dict,
+                  part_o: torch.Tensor | None = None, part_ml: torch.Tensor | None = None, *, num_heads: int,
+                  num_kv_heads: int, dim: int, vdim: int, scale: float, take_off: float, post: float, eps: float,
+                  gate: torch.Tensor | None = None, window: int = 0, chunk: int = 0) -> torch.Tensor:
+    """``paired_prefill`` for requests that bring one new token each (``dec_seqs``; None: all of the step's
+    ``n_seqs``).  ``launch``: from ``paired_decode_launch`` for a bound on the contexts that the caller guarantees
+    (keys beyond max_parts * part_keys would be left out)."""
+    bs = _paired_check(q, out, kpool, vpool, block_tables, gate, num_heads, num_kv_heads, dim, vdim)
+    _dev(q_start, ctx_len, dec_seqs, part_o, part_ml)
+    parts = launch["max_parts"]
+    need = n_seqs * num_heads * MAPS * parts
+    if parts > 1 and (part_o is None or part_ml is None or part_o.dtype != torch.float32 or part_ml.dtype != torch.float32 or
+                      part_o.numel() < need * vdim or part_ml.numel() < need * 2):
+        raise KernelError("differential attention: the partitions' workspace is missing or too small")
+    if n_seqs > (dec_seqs.numel() if dec_seqs is not None else ctx_len.numel()):
+        raise KernelError(f"differential attention: {n_seqs} requests of one token asked for")
+    lib = paired_lib(dim, vdim)
+    _check(lib.lyp_paired_decode(_p(q), q.stride(0), _p(out), out.stride(0), _p(kpool), _p(vpool), _code(q.dtype),
+                                 _p(block_tables), block_tables.shape[1], _p(q_start), _p(ctx_len), _p(dec_seqs), n_seqs,
+                                 _p(part_o), _p(part_ml), parts, launch["part_keys"], num_heads, num_kv_heads, bs, int(window),
+                                 int(chunk), float(scale), float(take_off), float(eps), float(post), _p(gate),
+                                 gate.stride(0) if gate is not None else 0, _stream()), lib)
+    return out
+
+
+def head_difference(a: torch.Tensor, dtype: torch.dtype, *, num_heads: int, vdim: int, take_off: float, post: float, eps: float,
+                    gate: torch.Tensor | None = None) -> torch.Tensor:
+    """a float [T, H 2 vdim] (per head the two maps' sums) -> [T, H vdim] of ``dtype``, as ``paired_prefill`` finishes
+    a head."""
+    _dev(a)
+    _f32(a, gate)
+    T = a.shape[0]
+    if tuple(a.shape) != (T, num_heads * MAPS * vdim):
+        raise KernelError(f"head_difference: {tuple(a.shape)} for {num_heads} heads of {vdim}")
+    if gate is not None:
+        _rows_view(gate, "head_difference")
+        if tuple(gate.shape) != (T, num_heads * vdim):
+            raise KernelError(f"head_difference: gate {tuple(gate.shape)}")
+    out = torch.empty((T, num_heads * vdim), dtype=dtype, device=a.device)
+    lib = core()
+    _check(lib.lyp_head_difference(_p(a), _p(gate), gate.stride(0) if gate is not None else 0, _p(out), _code(dtype), T,
+                                   num_heads, vdim, float(take_off), float(eps), float(post), _stream()), lib)
+    return out
+
+
 # ------------------------------- normed projections, windows with kept tokens, sinks
 def qk_norm_rope_kv(qkv: torch.Tensor, q_norm: torch.Tensor | None, k_norm: torch.Tensor | None, eps: float,
                     positions: torch.Tensor, table: torch.Tensor | None, slots: torch.Tensor | None,
@@ -1419,11 +1621,15 @@ def qk_norm_rope_kv(qkv: torch.Tensor, q_norm: torch.Tensor | None, k_norm: torc
 def attn_rows(q: torch.Tensor, out: torch.Tensor, kpool: torch.Tensor, vpool: torch.Tensor, block_tables: torch.Tensor,
               q_start: torch.Tensor, positions: torch.Tensor, ctx_len: torch.Tensor, *, num_heads: int,
               num_kv_heads: int, dim: int, vdim: int, scale: float, window: int = 0, keep_first: int = 0,
-              sink: torch.Tensor | None = None, cap: float = 0.0, slopes: torch.Tensor | None = None) -> torch.Tensor:
+              sink: torch.Tensor | None = None, cap: float = 0.0, slopes: torch.Tensor | None = None, chunk: int = 0,
+              maps: int = 1) -> torch.Tensor:
     """Attention of every row of the step over its request's pages for any key and value size: q a
     view [T, >= H dim], out [T, H vdim].  A row at position p sees key j <= p when window == 0,
     p - j < window or j < keep_first.  ``cap`` > 0: scores become cap * tanh(score / cap);
-    ``slopes`` (float [H]): key j's score loses slopes[head] * (p - j)."""
+    ``slopes`` (float [H]): key j's score loses slopes[head] * (p - j).  ``chunk`` > 0 (no window): a row sees the
+    keys of its own run of ``chunk`` positions.  ``maps`` > 1: that many neighbouring query heads read as many
+    neighbouring key heads of their own and one value head together (``num_heads`` and ``num_kv_heads`` count query
+    and key heads; the value pool has num_kv_heads / maps).  ``out`` may be float beside 16-bit operands."""
     _sink_check(sink, num_heads)
     _sink_check(slopes, num_heads)
     _dev(slopes)
@@ -1431,8 +1637,10 @@ def attn_rows(q: torch.Tensor, out: torch.Tensor, kpool: torch.Tensor, vpool: to
     n_pages, bs = kpool.shape[0], kpool.shape[2]
     T = q.shape[0]
     if (not q.is_cuda or q.stride(1) != 1 or q.stride(0) < num_heads * dim
-            or tuple(kpool.shape) != (n_pages, num_kv_heads, bs, dim) or tuple(vpool.shape) != (n_pages, num_kv_heads, vdim, bs)
-            or tuple(out.shape) != (T, num_heads * vdim) or len({q.dtype, out.dtype, kpool.dtype, vpool.dtype}) != 1
+            or tuple(kpool.shape) != (n_pages, num_kv_heads, bs, dim) or maps < 1 or num_kv_heads % maps or num_heads % maps
+            or tuple(vpool.shape) != (n_pages, num_kv_heads // maps, vdim, bs)
+            or tuple(out.shape) != (T, num_heads * vdim) or len({q.dtype, kpool.dtype, vpool.dtype}) != 1
+            or out.dtype not in (q.dtype, torch.float32) or positions.numel() != T
             or block_tables.dtype != torch.int32 or block_tables.dim() != 2):
         raise KernelError(f"attn_rows: q {tuple(q.shape)}, out {tuple(out.shape)}, pools {tuple(kpool.shape)} / "
                           f"{tuple(vpool.shape)} for {num_heads}/{num_kv_heads} heads of {dim}/{vdim}")
@@ -1440,7 +1648,8 @@ def attn_rows(q: torch.Tensor, out: torch.Tensor, kpool: torch.Tensor, vpool: to
     _check(lib.lyp_attn_rows(_p(q), q.stride(0), _p(kpool), _p(vpool), _p(block_tables), block_tables.shape[1], bs,
                              _p(q_start), _p(positions), _p(ctx_len), q_start.numel() - 1, _p(sink), float(scale),
                              int(window), int(keep_first), _p(out), out.stride(0), _code(q.dtype), T, num_heads,
-                             num_kv_heads, dim, vdim, float(cap), _p(slopes), _stream()), lib)
+                             num_kv_heads, dim, vdim, float(cap), _p(slopes), int(chunk), int(maps),
+                             int(out.dtype == torch.float32), _stream()), lib)
     return out
 
 
@@ -1463,14 +1672,15 @@ def stream_add(h: torch.Tensor, a, b: torch.Tensor | None = None) -> None:
 
 
 # ------------------------------------------------------------ routed feed-forward
-def glu_clamped(gate_up: torch.Tensor, limit: float, alpha: float) -> torch.Tensor:
-    """[T, 2 I] (gates first) -> [T, I]: g = min(gate, limit), u = clamp(up, -limit, limit);
-    g * sigmoid(alpha * g) * (u + 1)."""
+def glu_clamped(gate_up: torch.Tensor, limit: float, alpha: float, plus: float = 1.0, interleave: int = 0) -> torch.Tensor:
+    """[T, 2 I] -> [T, I]: g = min(gate, limit), u = clamp(up, -limit, limit) (no limit: infinity);
+    g * sigmoid(alpha * g) * (u + plus).  ``interleave`` 0: gates first; n: runs of n gates and their n ups in turn."""
     _dev(gate_up)
     T, I = gate_up.shape[0], gate_up.shape[1] // 2
     out = torch.empty((T, I), dtype=gate_up.dtype, device=gate_up.device)
     lib = core()
-    _check(lib.lyp_glu_clamped(_p(gate_up), _p(out), _code(gate_up.dtype), T, I, float(limit), float(alpha), _stream()), lib)
+    _check(lib.lyp_glu_clamped(_p(gate_up), _p(out), _code(gate_up.dtype), T, I, float(limit), float(alpha), float(plus),
+                               int(interleave), _stream()), lib)
     return out
 
 
@@ -1493,16 +1703,19 @@ ROUTE_SORT_MAX_ROWS = 64     # steps of up to this many rows choose and sort in 
 
 
 def moe_route_from(x: torch.Tensor, router: torch.Tensor, bias: torch.Tensor | None, top: int, always: int = -1,
-                   sort_for: int = 0):
+                   sort_for: int = 0, over_all: bool = False, scale: float = 1.0, gated: bool = False):
     """As ``moe_route`` from the router's input: x [T, K] activations, ``router`` [E, K] float; the
     logits x @ router.T are formed in 32-bit in the same kernel.  ``sort_for`` > 0 (the number of
     expert matrices, the always-used one included): also returns the ``MoePlan`` of the choices, as
-    ``moe_sort`` makes it; with few rows the choice and the sort are one kernel."""
+    ``moe_sort`` makes it; with few rows the choice and the sort are one kernel.  ``over_all``: the weights are
+    the chosen experts' shares of the softmax over all experts; either kind is multiplied by ``scale``.
+    ``gated``: the router has one more row, whose logit's sigmoid is the token's share of what every token
+    uses: the always-used expert's weight, or, without one, returned last (float [T])."""
     _dev(x, router, bias)
     _f32(router, bias)
     T, K = x.shape
-    E = router.shape[0]
-    if router.shape[1] != K or x.stride(1) != 1:
+    E = router.shape[0] - int(gated)
+    if router.shape[1] != K or x.stride(1) != 1 or E < 1 or (bias is not None and bias.numel() != E):
         raise KernelError(f"moe_route_from: x {tuple(x.shape)}, router {tuple(router.shape)}")
     per = top + (1 if always >= 0 else 0)
     idx = torch.empty((T, per), dtype=torch.int32, device=x.device)
@@ -1510,13 +1723,16 @@ def moe_route_from(x: torch.Tensor, router: torch.Tensor, bias: torch.Tensor | N
     lib = core()
     # few rows: several workgroups share the inner dimension and leave partial sums
     splits = lib.lyp_moe_route_splits(T, K)
-    part = torch.empty((splits, T, E), dtype=torch.float32, device=x.device) if splits > 1 else None
+    part = torch.empty((splits, T, E + int(gated)), dtype=torch.float32, device=x.device) if splits > 1 else None
+    share = torch.empty(T, dtype=torch.float32, device=x.device) if gated and always < 0 else None
+    rule = (int(over_all), float(scale), int(gated), _p(share))
     together = sort_for > 0 and splits > 1 and T <= ROUTE_SORT_MAX_ROWS
     _check(lib.lyp_moe_route_fused(_p(x), x.stride(0), _code(x.dtype), _p(router), _p(bias), T, E, K, top, _p(idx),
-                                   _p(wgt), int(always), _p(part), splits, 0 if together else 1, _stream()), lib)
-    if not sort_for:
-        return idx, wgt
-    return idx, wgt, MoePlan(idx, sort_for, route=(part, bias, top, always, wgt) if together else None)
+                                   _p(wgt), int(always), _p(part), splits, 0 if together else 1, *rule, _stream()), lib)
+    out = (idx, wgt)
+    if sort_for:
+        out += (MoePlan(idx, sort_for, route=(part, bias, E, top, always, wgt, rule) if together else None),)
+    return out if share is None else out + (share,)
 
 
 class MoePlan:
@@ -1561,18 +1777,18 @@ class MoePlan:
         return plans
 
     def __init__(self, idx: torch.Tensor, E: int, route=None):
-        """``route`` (partial sums [parts, T, experts], bias, top, always, weights): the choices are not
-        made yet; the sort's kernel adds the router's partial sums up, chooses into ``idx`` and the
-        weights, and sorts."""
+        """``route`` (partial sums [parts, T, experts (+ 1)], bias, experts, top, always, weights, the rule's
+        arguments): the choices are not made yet; the sort's kernel adds the router's partial sums up, chooses
+        into ``idx`` and the weights, and sorts."""
         lib = core()
         sizes = self._place(idx.numel(), idx.shape[1], E)      # one allocation
         self._take(torch.empty(sum(sizes), dtype=torch.int32, device=idx.device), sizes)
         if route is not None:
-            part, bias, top, always, wgt = route
-            _check(lib.lyp_moe_route_sort(_p(part), part.shape[0], _p(bias), part.shape[1], part.shape[2], top, always,
+            part, bias, experts, top, always, wgt, rule = route
+            _check(lib.lyp_moe_route_sort(_p(part), part.shape[0], _p(bias), part.shape[1], experts, top, always,
                                           _p(idx), _p(wgt), E, self.tile_rows, _p(self.expert_off), _p(self.sorted_pair),
                                           _p(self.place_of), _p(self.tile_expert), _p(self.tile_row0), _p(self.n_tiles),
-                                          _stream()), lib)
+                                          *rule, _stream()), lib)
             return
         _check(lib.lyp_moe_sort(_p(idx), self.pairs, E, self.tile_rows, _p(self.expert_off), _p(self.sorted_pair),
                                 _p(self.place_of), _p(self.tile_expert), _p(self.tile_row0), _p(self.n_tiles),
@@ -1610,11 +1826,14 @@ def moe_gemm(a: torch.Tensor, w: torch.Tensor, plan: MoePlan, *, gated: bool, li
 
 
 def moe_combine(y: torch.Tensor, plan: MoePlan, weights: torch.Tensor | None, rows: int, addend: torch.Tensor | None = None,
-                shared: torch.Tensor | None = None) -> torch.Tensor:
-    """float [1, rows, H]: addend + shared + sum over a token's choices of weight * y[place of the
+                shared: torch.Tensor | None = None, share: torch.Tensor | None = None) -> torch.Tensor:
+    """float [1, rows, H]: addend + share * shared + sum over a token's choices of weight * y[place of the
     pair], added up in 32-bit in the order of the choices (one slice of partial sums, which a norm
-    adds to the residual stream)."""
-    _dev(y, weights, addend, shared)
+    adds to the residual stream).  ``share`` (float [rows]): a row's factor of ``shared`` (none: 1)."""
+    _dev(y, weights, addend, shared, share)
+    _f32(share)
+    if share is not None and (shared is None or share.numel() != rows):
+        raise KernelError(f"moe_combine: shares {tuple(share.shape)} for {rows} rows")
     H = y.shape[1]
     for t in (addend, shared):
         if t is not None and (tuple(t.shape) != (rows, H) or t.dtype != y.dtype):
@@ -1624,7 +1843,7 @@ def moe_combine(y: torch.Tensor, plan: MoePlan, weights: torch.Tensor | None, ro
         raise KernelError("moe_combine: weights do not fit the pairs")
     out = torch.empty((1, rows, H), dtype=torch.float32, device=y.device)
     lib = core()
-    _check(lib.lyp_moe_combine(_p(y), _p(plan.place_of), _p(weights), plan.top, _p(addend), _p(shared), _p(out),
+    _check(lib.lyp_moe_combine(_p(y), _p(plan.place_of), _p(weights), plan.top, _p(addend), _p(shared), _p(share), _p(out),
                                _code(y.dtype), rows, H, _stream()), lib)
     return out
 
@@ -2000,7 +2219,7 @@ def qkv_prepare(pre: torch.Tensor, dtype: torch.dtype, *, num_heads: int, num_kv
                 k_weight: torch.Tensor | None = None, eps: float = 0.0, positions: torch.Tensor | None = None,
                 table: torch.Tensor | None = None, pairing: str = "neighbours", values_from_keys: bool = False,
                 blend: torch.Tensor | None = None, other_values: torch.Tensor | None = None,
-                keep_values: bool = False):
+                keep_values: bool = False, value_heads: int | None = None):
     """From a float projection pre [T, >= (H + G) dim (+ G vdim)] (queries, keys and, unless the values
     are the keys, values side by side) to queries [T, H dim] of ``dtype`` (returned) and keys and
     values in the tokens' page slots: bias added; values taken (the biased key projection itself with
@@ -2009,35 +2228,37 @@ def qkv_prepare(pre: torch.Tensor, dtype: torch.dtype, *, num_heads: int, num_kv
     float [T, G vdim]; queries and keys RMS-normed per head (``norm`` "head"; weights [dim] shared by
     the heads, or none) or over the whole projection ("whole"; weights over all of it); the first
     table.shape[1] values of every head turned by the position, pairs (2i, 2i + 1) ("neighbours") or
-    (i, i + half) ("halves").  -> (q, kept values or None)."""
+    (i, i + half) ("halves").  ``value_heads``: how many heads the values have (None: as many as the keys; else a
+    divisor of that).  -> (q, kept values or None)."""
     _rows_view(pre, "qkv_prepare")
     _dev(bias, q_weight, k_weight, positions, table, slots, kpool, vpool, blend, other_values)
     _f32(pre, bias, q_weight, k_weight, table, blend, other_values)
     T, H, G = pre.shape[0], num_heads, num_kv_heads
-    n = (H + G) * dim + (0 if values_from_keys else G * vdim)
+    GV = G if value_heads is None else int(value_heads)
+    n = (H + G) * dim + (0 if values_from_keys else GV * vdim)
     modes = {"none": 0, "head": 1, "whole": 2}
-    pairings = {"neighbours": 0, "halves": 1}
+    pairings = PAIRINGS
     rot = table.shape[1] if table is not None else 0
     n_pages = kpool.shape[0]
     want_w = {0: (0, 0), 1: (dim, dim), 2: (H * dim, G * dim)}.get(modes.get(norm, -1))
-    if norm not in modes or pairing not in pairings or pre.shape[1] < n or (bias is not None and bias.numel() != n) or \
+    if norm not in modes or pairing not in pairings or GV < 1 or G % GV or pre.shape[1] < n or (bias is not None and bias.numel() != n) or \
             slots.numel() != T or slots.dtype != torch.int32 or (values_from_keys and vdim != dim) or \
             (rot and (positions is None or positions.numel() != T or positions.dtype != torch.int32)) or \
             any(w is not None and w.numel() != k for w, k in zip((q_weight, k_weight), want_w)) or \
-            (blend is not None and (other_values is None or tuple(other_values.shape) != (T, G * vdim) or
+            (blend is not None and (other_values is None or tuple(other_values.shape) != (T, GV * vdim) or
                                     other_values.stride(1) != 1)) or \
-            tuple(kpool.shape) != (n_pages, G, page_size, dim) or tuple(vpool.shape) != (n_pages, G, vdim, page_size) or \
+            tuple(kpool.shape) != (n_pages, G, page_size, dim) or tuple(vpool.shape) != (n_pages, GV, vdim, page_size) or \
             kpool.dtype != dtype or vpool.dtype != dtype:
         raise KernelError(f"qkv_prepare: pre {tuple(pre.shape)}, pools {tuple(kpool.shape)} / {tuple(vpool.shape)} "
                           f"{kpool.dtype} for {H}+{G} heads of {dim}/{vdim}, norm {norm!r}, pairing {pairing!r}, dtype {dtype}")
     q = torch.empty((T, H * dim), dtype=dtype, device=pre.device)
-    kept = torch.empty((T, G * vdim), dtype=torch.float32, device=pre.device) if keep_values else None
+    kept = torch.empty((T, GV * vdim), dtype=torch.float32, device=pre.device) if keep_values else None
     lib = core()
     _check(lib.lyp_qkv_prepare(_p(pre), pre.stride(0), _p(bias), modes[norm], _p(q_weight), _p(k_weight), float(eps),
                                _p(positions), _p(table), rot, pairings[pairing], int(values_from_keys), _p(blend),
                                _p(other_values), other_values.stride(0) if other_values is not None else 0, _p(kept),
                                _p(slots), _p(q), _p(kpool), _p(vpool), _code(dtype), T, H, G, dim, vdim, page_size,
-                               _stream()), lib)
+                               GV, _stream()), lib)
     return q, kept
 
 

@@ -150,9 +150,11 @@ class DecoderModel(Part):
                 if part_states.setdefault((call.cache, name), spec) != spec:
                     raise ValueError(f"state {name!r} of buffer {call.cache} is used with two shapes")
             if kv is not None:
-                if call.cache in by_cache and by_cache[call.cache] != kv:
-                    raise ValueError(f"cache buffer {call.cache} is used with two shapes: {by_cache[call.cache]} and {kv}")
-                by_cache.setdefault(call.cache, kv)
+                have = by_cache.get(call.cache)
+                if have is not None and have.tensors != kv.tensors:
+                    raise ValueError(f"cache buffer {call.cache} is used with two shapes: {have} and {kv}")
+                # calls that see different stretches of one buffer: it keeps what any of them needs
+                by_cache[call.cache] = kv if have is None else have.covering(kv)
             if st is not None:
                 if call.cache in states and states[call.cache] != st:
                     raise ValueError(f"state buffer {call.cache} is used with two shapes")

@@ -146,16 +146,38 @@ class PagedSpec:
     tensors: tuple         # of PageTensor
     window: int = 0        # 0: every token is kept; W: a token needs the last W tokens' entries, its own included
     keep_first: int = 0    # with a window: a token also needs the request's first keep_first entries
+    chunk: int = 0         # C (without a window): a token needs the entries of its own run of C positions, counted from 0
+
+    def __post_init__(self):
+        if self.window and self.chunk:
+            raise ValueError("what a token needs is a window or a chunk, not both")
+
+    @property
+    def keeps_all(self) -> bool:
+        return not self.window and not self.chunk
+
+    def covering(self, other: "PagedSpec") -> "PagedSpec":
+        """The spec of a buffer that calls with this reach and with ``other``'s both use: the same tensors,
+        kept for as long as either needs them (a chunk's entries all lie in a window of its length)."""
+        if self.tensors != other.tensors:
+            raise ValueError(f"one buffer with two contents: {self.tensors} and {other.tensors}")
+        if self == other:
+            return self
+        if self.keeps_all or other.keeps_all:
+            return PagedSpec(self.tensors)
+        return PagedSpec(self.tensors, max(self.window, self.chunk, other.window, other.chunk),
+                         max(self.keep_first, other.keep_first))
 
     @classmethod
     def keys_and_values(cls, num_kv_heads: int, head_dim: int, window: int = 0, value_dim: Optional[int] = None,
-                        keep_first: int = 0) -> "PagedSpec":
+                        keep_first: int = 0, chunk: int = 0, value_heads: Optional[int] = None) -> "PagedSpec":
         """The layout the attention kernels of this package read: keys
         [heads][slot][head_dim], values [heads][value_dim][slot] (``value_dim``
-        None: the keys' size)."""
+        None: the keys' size; ``value_heads`` None: as many as key heads)."""
         vd = head_dim if value_dim is None else int(value_dim)
-        return cls((PageTensor("k", (num_kv_heads, SLOT, head_dim)), PageTensor("v", (num_kv_heads, vd, SLOT))),
-                   int(window), int(keep_first) if window else 0)
+        vh = num_kv_heads if value_heads is None else int(value_heads)
+        return cls((PageTensor("k", (num_kv_heads, SLOT, head_dim)), PageTensor("v", (vh, vd, SLOT))),
+                   int(window), int(keep_first) if window else 0, int(chunk))
 
 
 @dataclass(frozen=True)

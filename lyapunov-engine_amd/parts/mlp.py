@@ -7,6 +7,7 @@ python/lyapunov_engine/ops.py:72-73).
 """
 from __future__ import annotations
 
+import math
 from typing import Optional
 
 import torch
@@ -82,6 +83,39 @@ class GatedDense(FeedForward):
     def forward(self, ctx: StepContext, x):
         act = ops.glu_act(ops.linear(x, self.gate_up_proj, out_dtype=ctx.dtype), self.activation)
         return ops.linear(act, self.down_proj, out_dtype=ctx.dtype)
+
+
+@FEED_FORWARDS.register("limited_glu")
+class LimitedGLU(FeedForward):
+    """down(g * sigmoid(gate_slope * g) * (u + plus)), no biases, with g = min(gate(x), limit) and
+    u = clamp(up(x), -limit, limit).  Gate and up are one matrix in tiles of 16 rows (eight gates, their eight ups)
+    where the width allows, which lets a step of few rows gate inside the product; other widths keep the plain
+    order, gates first."""
+
+    def __init__(self, hidden_size: int, intermediate_size: int, limit: float = math.inf, gate_slope: float = 1.0,
+                 plus: float = 0.0, names: Optional[dict] = None):
+        if not limit > 0:
+            raise ValueError(f"a gated feed-forward with a limit of {limit}")
+        self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
+        self.limit, self.gate_slope, self.plus = float(limit), float(gate_slope), float(plus)
+        n = dict(gate="gate", up="up", down="down")
+        n.update(names or {})
+        self.names = n
+        self.interleave = 8 if self.intermediate_size % 8 == 0 else 0
+        self.gate_up_proj: Optional[torch.Tensor] = None
+        self.down_proj: Optional[torch.Tensor] = None
+
+    def weight_specs(self):
+        n, shape = self.names, (self.intermediate_size, self.hidden_size)
+        return [WeightSpec("gate_up_proj", (WeightSource(n["gate"], shape), WeightSource(n["up"], shape)),
+                           interleave=self.interleave),
+                WeightSpec("down_proj", (WeightSource(n["down"], (self.hidden_size, self.intermediate_size)),))]
+
+    takes_pending_norm = True   # x may be an ops.PendingNorm: the gate/up product norms on its way in
+
+    def forward(self, ctx: StepContext, x):
+        act = ops.linear_glu(x, self.gate_up_proj, self.interleave, self.limit, self.gate_slope, self.plus)
+        return ops.linear(act, self.down_proj, out_dtype=ctx.dtype, may_split=True, pending=True)
 
 
 @FEED_FORWARDS.register("swiglu")

@@ -29,11 +29,14 @@ class RMSNorm(Norm):
         self.one_plus = bool(one_plus)
         self.weight: Optional[torch.Tensor] = None
         self._weight_f: Optional[torch.Tensor] = None
-        if self.one_plus:
-            self.can_defer = False     # the folded forms take the stored tensor as the multiplier
 
     def weight_specs(self):
         return [WeightSpec("weight", (WeightSource(self.tensor, (self.size,)),), init="normal" if self.one_plus else "ones")]
+
+    @property
+    def multiplier(self) -> torch.Tensor:
+        """What the kernels multiply by: the stored tensor, or one plus it as float."""
+        return self.weight_f if self.one_plus else self.weight
 
     @property
     def weight_f(self) -> torch.Tensor:
@@ -70,12 +73,12 @@ class RMSNorm(Norm):
             return ops.branch_join(h, delta.y, delta.weight, delta.mult, delta.eps, shift=delta.shift,
                                    next_weight=self.weight_f, eps_next=self.eps, out=out, rows=rows, conv=conv)
         if lazy and rows is None:
-            pending, delta = ops.rmsnorm_pending(h, self.weight, self.eps, ctx.dtype, delta)
+            pending, delta = ops.rmsnorm_pending(h, self.multiplier, self.eps, ctx.dtype, delta)
             if pending is not None:
                 return pending
         n = h.shape[0] if rows is None else rows.numel()
         out = torch.empty((n, self.size), dtype=ctx.dtype, device=h.device)
-        return ops.rmsnorm(h, self.weight_f if self.one_plus else self.weight, self.eps, out, delta=delta, rows=rows)
+        return ops.rmsnorm(h, self.multiplier, self.eps, out, delta=delta, rows=rows)
 
 
 @NORMS.register("group_rmsnorm")

@@ -1,12 +1,14 @@
 """A feed-forward that routes every token to a few of many small experts.
 
-    z = W_r x + b                       router logits, in 32-bit
-    the ``top`` experts with the largest z; their weights: the softmax over those z alone
+    z = W_r x (+ b)                     router logits, in 32-bit
+    the ``top`` experts with the largest z; their weights: the softmax over those z alone (``scores`` "chosen"),
+               or their shares of the softmax over all z ("all"); either times ``scale``
     expert e:  g = min(W_gate,e x, limit), u = clamp(W_up,e x, -limit, limit)
-               y_e = W_down,e (g * sigmoid(gate_slope * g) * (u + 1))
-    out = sum over the chosen e of weight_e * y_e   (+ a shared expert of the same form, run for every token)
+               y_e = W_down,e (g * sigmoid(gate_slope * g) * (u + plus))
+    out = sum over the chosen e of weight_e * y_e   (+ a shared expert of the same form, run for every token,
+               times sigmoid(W_s x), one number a token, with ``shared_gate``)
 
-No biases in the experts.  On the device nothing is counted on the host: the
+No biases in the experts.  The shared expert's gate is one more row of the router's matrix.  On the device nothing is counted on the host: the
 (token, choice) pairs are sorted by expert in one kernel, the two products walk
 a list of row tiles that kernel leaves (grids sized for the most tiles there can
 be), and the last kernel adds a token's weighted expert outputs, the shared
@@ -33,20 +35,26 @@ class RoutedExperts(FeedForward):
     choices_log: Optional[list] = None
 
     def __init__(self, hidden_size: int, num_experts: int, top: int, intermediate_size: int, limit: float,
-                 gate_slope: float = 1.702, shared_size: int = 0, shared_limit: float = 0.0,
+                 gate_slope: float = 1.702, shared_size: int = 0, shared_limit: float = 0.0, plus: float = 1.0,
+                 router_bias: bool = True, scores: str = "chosen", scale: float = 1.0, shared_gate: bool = False,
                  names: Optional[dict] = None):
         if not 1 <= top <= num_experts or intermediate_size <= 0 or shared_size < 0:
             raise ValueError(f"routed experts: {top} of {num_experts} experts of {intermediate_size}, shared {shared_size}")
         self.hidden_size, self.num_experts, self.top = int(hidden_size), int(num_experts), int(top)
         self.intermediate_size, self.limit, self.gate_slope = int(intermediate_size), float(limit), float(gate_slope)
+        if scores not in ("chosen", "all") or (shared_gate and not shared_size):
+            raise ValueError(f"routed experts: scores {scores!r}, a gate for a shared expert of {shared_size}")
         self.shared_size, self.shared_limit = int(shared_size), float(shared_limit)
+        self.plus, self.has_bias, self.scale = float(plus), bool(router_bias), float(scale)
+        self.over_all, self.shared_gate = scores == "all", bool(shared_gate)
         n = dict(router="router", router_bias="router.b", expert="e{j}.", shared="shared.", gate="gate", up="up",
-                 down="down")
+                 down="down", shared_gate="sg")
         n.update(names or {})
         self.names = n
         # A shared expert of the routed experts' size and limit is kept as one more matrix behind
         # theirs and rides in their products as an expert every token uses with weight 1.
         self.shared_folded = self.shared_size == self.intermediate_size and self.shared_limit == self.limit
+        self.shared_interleave = 8 if self.shared_size % 8 == 0 else 0      # as LimitedGLU keeps its matrix
         self.router = self.router_bias = self.gate_up = self.down = self.shared_gate_up = self.shared_down = None
         self.router_f = self.router_bias_f = None
 
@@ -61,12 +69,16 @@ class RoutedExperts(FeedForward):
             s = n["shared"]
             gate_up += [WeightSource(s + n["gate"], (I, H)), WeightSource(s + n["up"], (I, H))]
             down.append(WeightSource(s + n["down"], (H, I)))
-        specs = [WeightSpec("router", (WeightSource(n["router"], (E, H)),)),
-                 WeightSpec("router_bias", (WeightSource(n["router_bias"], (E,)),)),
-                 WeightSpec("gate_up", tuple(gate_up)), WeightSpec("down", tuple(down))]
+        router = (WeightSource(n["router"], (E, H)),)
+        if self.shared_gate:
+            router += (WeightSource(n["shared"] + n["shared_gate"], (1, H)),)
+        specs = [WeightSpec("router", router), WeightSpec("gate_up", tuple(gate_up)), WeightSpec("down", tuple(down))]
+        if self.has_bias:
+            specs.append(WeightSpec("router_bias", (WeightSource(n["router_bias"], (E,)),)))
         if self.shared_size and not self.shared_folded:
             s, S = n["shared"], self.shared_size
-            specs += [WeightSpec("shared_gate_up", (WeightSource(s + n["gate"], (S, H)), WeightSource(s + n["up"], (S, H)))),
+            specs += [WeightSpec("shared_gate_up", (WeightSource(s + n["gate"], (S, H)), WeightSource(s + n["up"], (S, H))),
+                                 interleave=self.shared_interleave),
                       WeightSpec("shared_down", (WeightSource(s + n["down"], (H, S)),))]
         return specs
 
@@ -74,7 +86,7 @@ class RoutedExperts(FeedForward):
         E, I, H = self.num_experts, self.intermediate_size, self.hidden_size
         # the router works in 32-bit whatever the activations are
         self.router_f = self.router.float().contiguous()
-        self.router_bias_f = self.router_bias.float().contiguous()
+        self.router_bias_f = self.router_bias.float().contiguous() if self.has_bias else None
         self.router = None
         stacked = E + (1 if self.shared_folded else 0)
         self.gate_up = self.gate_up.view(stacked, 2 * I, H)      # per expert: gate rows, then up rows
@@ -85,20 +97,20 @@ class RoutedExperts(FeedForward):
         shared expert's and ``addend`` (the other branch's output, activations [T, hidden])."""
         T = x.shape[0]
         always = self.num_experts if self.shared_folded else -1
-        idx, wgt, plan = ops.moe_route_from(x, self.router_f, self.router_bias_f, self.top, always,
-                                            sort_for=self.gate_up.shape[0])
+        idx, wgt, plan, *share = ops.moe_route_from(x, self.router_f, self.router_bias_f, self.top, always,
+                                                    sort_for=self.gate_up.shape[0], over_all=self.over_all, scale=self.scale,
+                                                    gated=self.shared_gate)
         if RoutedExperts.choices_log is not None:
             RoutedExperts.choices_log.append(idx[:, :self.top])
-        act = ops.moe_gemm(x, self.gate_up, plan, gated=True, limit=self.limit, alpha=self.gate_slope)
+        act = ops.moe_gemm(x, self.gate_up, plan, gated=True, limit=self.limit, alpha=self.gate_slope, plus=self.plus)
         y = ops.moe_gemm(act, self.down, plan, gated=False)
         shared = None
         if self.shared_size and not self.shared_folded:
-            gu = ops.linear(x, self.shared_gate_up, out_dtype=ctx.dtype)
-            shared = ops.linear(ops.glu_clamped(gu, self.shared_limit, self.gate_slope), self.shared_down,
-                                out_dtype=ctx.dtype)
+            gu = ops.linear_glu(x, self.shared_gate_up, self.shared_interleave, self.shared_limit, self.gate_slope, self.plus)
+            shared = ops.linear(gu, self.shared_down, out_dtype=ctx.dtype)
         if addend is not None:
             addend = ops.as_delta(addend, ctx.dtype)
-        return ops.moe_combine(y, plan, wgt, T, addend=addend, shared=shared)
+        return ops.moe_combine(y, plan, wgt, T, addend=addend, shared=shared, share=share[0] if share else None)
 
 
 @FEED_FORWARDS.register("group_routed_experts")

@@ -411,7 +411,10 @@ def test_routed_experts_against_the_plain_mixture(dtype, shape):
             t = torch.randn(src.shape, generator=g) * (1.0 if src.name.startswith("router") else 2.5 / math.sqrt(src.shape[-1]))
             w[src.name] = t.to(tdt(dtype))
             pieces.append(w[src.name])
-        setattr(part, ws.attr, torch.cat(pieces).to(DEV))
+        joined = torch.cat(pieces)
+        if ws.interleave:      # runs of the sources' rows in turn
+            joined = torch.stack([p.view(-1, ws.interleave, H) for p in pieces], dim=1).reshape(joined.shape)
+        setattr(part, ws.attr, joined.to(DEV))
     part.materialize(DEV, tdt(dtype))
     x = torch.randn(T, H, generator=g).to(tdt(dtype))
     addend = torch.randn(T, H, generator=g).to(tdt(dtype))
