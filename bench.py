@@ -218,7 +218,7 @@ VOBOTAR_SIZES = {
 # much again for their gates); the first four layers run twice.  Beside each stands the Faledra model of
 # equal width, depth, heads, latent and dense feed-forward: the closest design (attention over latents,
 # looped layers).
-def panodra_shape(width, heads, ff, layers, vocab, kv_rank, experts, top):
+def panodra_shape(width, heads, ff, layers, vocab, kv_rank, experts, top, expert_ff=None, loop=True):
     def mixer(scaling):
         rot = dict(base=500000.0, dims=32)
         if scaling:
@@ -230,10 +230,11 @@ def panodra_shape(width, heads, ff, layers, vocab, kv_rank, experts, top):
 
     def routed():
         return dict(type="latent_attention_2", mixer=mixer(False),
-                    mlp=dict(kind="moe", expert=dict(ff=ff * 3 // (2 * top)), router=dict(experts=experts, top=top)))
+                    mlp=dict(kind="moe", expert=dict(ff=expert_ff or ff * 3 // (2 * top)), router=dict(experts=experts, top=top)))
 
     return dict(architecture="Panodra", vocab=vocab, width=width, norm=dict(eps=1e-5), logit_scale=0.5, logit_softcap=30.0,
-                loop=dict(start=0, stop=4, times=2), layers=[routed() if i % 2 else dense() for i in range(layers)])
+                loop=dict(start=0, stop=4, times=2) if loop else None,
+                layers=[routed() if i % 2 else dense() for i in range(layers)])
 
 
 PANODRA_SIZES = {
@@ -241,8 +242,44 @@ PANODRA_SIZES = {
     "1b": (panodra_shape(2048, 32, 8192, 12, 128256, 256, 32, 4), DESIGN_SIZES["1b"][0]),
     "wide": (panodra_shape(4096, 32, 14336, 4, 128256, 512, 32, 4), DESIGN_SIZES["wide"][0]),
 }
+
+
+# Pudulorn models with layers of a real model's sizes: latent attention within a window of 1,024 tokens before a
+# limited gated feed-forward, in turn with differential attention in chunks of 1,024 (half as many heads of two maps
+# and twice the value size) before routed experts with a gated shared one, the experts a token uses having
+# together the dense layer's width; every other latent layer reads the latents of the one before it.  Beside
+# each stands the Panodra model of equal width, depth, latent heads and latent, whose feed-forwards have as
+# many weights (dense) and as many in a token's experts: the closest design (attention over latents, a dense
+# layer and routed experts in turn).
+def pudulorn_shape(width, heads, kv_heads, ff, layers, vocab, q_rank, kv_rank, experts, top, expert_ff, shared):
+    def latent(source):
+        m = dict(heads=heads, dim=64, rot_dim=32, vdim=64, q_rank=q_rank, kv_rank=kv_rank, scale=96 ** -0.5,
+                 rot=dict(base=500000.0, dims=32), mask=dict(size=1024))
+        if source is not None:
+            m["kv_from"] = source
+        return dict(type="latent_attention", mixer=m, mlp=dict(kind="dense", ff=ff, limit=7.0))
+
+    def differential():
+        return dict(type="attention",
+                    mixer=dict(heads=heads // 2, kv_heads=kv_heads // 2, dim=64, vdim=128, scale=0.125, diff=0.3,
+                               rot=dict(base=500000.0, dims=64), mask=dict(size=1024)),
+                    mlp=dict(kind="moe", router=dict(experts=experts, top=top, scale=2.5), expert=dict(ff=expert_ff),
+                             shared=dict(ff=shared)))
+
+    return dict(architecture="Pudulorn", vocab=vocab, width=width, norm=dict(eps=1e-5),
+                layers=[differential() if i % 2 else latent(i - 2 if i % 4 == 2 else None) for i in range(layers)])
+
+
+PUDULORN_SIZES = {
+    "small": (pudulorn_shape(1024, 16, 4, 4096, 8, 32000, 384, 128, 16, 3, 1024, 1024),
+              panodra_shape(1024, 16, 4096, 8, 32000, 128, 16, 4, expert_ff=1024, loop=False)),
+    "1b": (pudulorn_shape(2048, 32, 8, 8192, 16, 128256, 768, 256, 32, 4, 1536, 2048),
+           panodra_shape(2048, 32, 8192, 16, 128256, 256, 32, 4, expert_ff=2048, loop=False)),
+    "wide": (pudulorn_shape(4096, 32, 8, 14336, 8, 128256, 1536, 512, 32, 4, 3072, 2048),
+             panodra_shape(4096, 32, 14336, 8, 128256, 512, 32, 4, expert_ff=3584, loop=False)),
+}
 # what stands beside a design's sizes
-BESIDE = {"faledra": "llama", "ronupel": "llama", "tonilix": "faledra", "vobotar": "tonilix", "panodra": "faledra"}
+BESIDE = {"faledra": "llama", "ronupel": "llama", "tonilix": "faledra", "vobotar": "tonilix", "panodra": "faledra", "pudulorn": "panodra"}
 
 
 class _Vocab:
@@ -260,7 +297,7 @@ def run_design(args):
     context, block_size, out = 2304, 16, {}
     design = args.design
     sizes = {"faledra": DESIGN_SIZES, "ronupel": RONUPEL_SIZES, "tonilix": TONILIX_SIZES, "vobotar": VOBOTAR_SIZES,
-             "panodra": PANODRA_SIZES}[design]
+             "panodra": PANODRA_SIZES, "pudulorn": PUDULORN_SIZES}[design]
     beside = BESIDE[design]
     for size in (args.size.split(",") if args.size else sorted(sizes)):
         other, second = sizes[size]
@@ -504,8 +541,8 @@ def main():
                     help="mixed: the continuous batch of BASELINE.json configs[3] instead of the headline")
     ap.add_argument("--skip-points", action="store_true", help="only the headline decode and the prefill")
     ap.add_argument("--skip-check", action="store_true", help="no comparison of bfloat16 logits with a 32-bit run")
-    ap.add_argument("--design", default="llama", choices=["llama", "faledra", "ronupel", "tonilix", "vobotar", "panodra"],
-                    help="faledra, ronupel, tonilix, vobotar, panodra: that design's prefill and decode speed at a few "
+    ap.add_argument("--design", default="llama", choices=["llama", "faledra", "ronupel", "tonilix", "vobotar", "panodra", "pudulorn"],
+                    help="faledra, ronupel, tonilix, vobotar, panodra, pudulorn: that design's prefill and decode speed at a few "
                          "sizes, each beside the Llama shape (Tonilix and Panodra: the Faledra model; Vobotar: the Tonilix "
                          "model) of equal size, instead of the headline")
     ap.add_argument("--size", default="", help="with another --design: which sizes, with commas (default: all)")

@@ -14,9 +14,10 @@
 //   * paired_prefill: a workgroup takes up to 64 new tokens of one request and up to four query
 //     heads of one key/value head (a wave: one head, 16 tokens, both maps).  Key and value tiles pass
 //     through two LDS buffers, shared by the four waves; a value fragment read from LDS serves both maps.
+//     In launches of few workgroups two sets of four waves share a workgroup's keys, tile about.
 //   * paired_decode: a wave takes one request's single new token, all query heads of one
-//     key/value head (as the 16 columns of the tile), and a share of a partition of the keys;
-//     keys and values go from the pages straight to registers.
+//     key/value head (as the 16 columns of the tile), one map, and a share of a partition of the
+//     keys; keys and values go from the pages straight to registers.
 // With the keys in several partitions (few new tokens over many keys) the partitions' sums are
 // merged by paired_merge, which then finishes the heads.
 //
@@ -218,7 +219,8 @@ struct Tile {
   static constexpr size_t kBytes = 2 * kElems * sizeof(T);     // two buffers
   static constexpr int kKVecs = kKeys * kMaps * HD / kVec, kVVecs = VD * kKeys / kVec;
   static constexpr int kKPer = (kKVecs + 255) / 256, kVPer = (kVVecs + 255) / 256;
-  static_assert(kBytes <= 160 * 1024, "two tiles must fit the LDS");
+  static_assert(kBytes + 2 * kKeys * sizeof(int) <= 160 * 1024, "two tiles must fit the LDS");
+  static constexpr bool kMaySplit = sizeof(T) == 2 && 2 * (kBytes + 2 * kKeys * sizeof(int)) <= 160 * 1024 && VD <= 128;
 };
 
 // Where a value tile keeps key k: a lane reads its keys of a step (4 of each 16-key block) in one piece.
@@ -228,8 +230,11 @@ __device__ __forceinline__ constexpr int value_column(int k) {
   return k / (16 * NS) * (16 * NS) + k % 16 / 4 * (4 * NS) + k / 16 % NS * 4 + k % 4;
 }
 
-template <typename T, int GH>
-__global__ __launch_bounds__(256, (HD <= 64 && VD <= 128 && sizeof(T) == 2) ? 2 : 1) void paired_prefill_kernel(
+// KS = 2: two sets of four waves take the workgroup's tiles in turn, each through LDS buffers of its own,
+// and the second hands its sums to the first at the end: half as many tiles in a row, for launches whose
+// time is that of the workgroup with most keys.
+template <typename T, int GH, int KS>
+__global__ __launch_bounds__(256 * KS, (HD <= 64 && VD <= 128 && sizeof(T) == 2) ? 2 / KS : 1) void paired_prefill_kernel(
     const T* __restrict__ q, int q_stride, T* __restrict__ out, int out_stride, const T* __restrict__ kpool,
     const T* __restrict__ vpool, const int32_t* __restrict__ block_tables, int table_width,
     const int32_t* __restrict__ q_start, const int32_t* __restrict__ ctx_len, const int32_t* __restrict__ tile_seq,
@@ -241,11 +246,14 @@ __global__ __launch_bounds__(256, (HD <= 64 && VD <= 128 && sizeof(T) == 2) ? 2 
   constexpr int QW = (4 / GH) * 16;       // new tokens per workgroup
   constexpr int kSubs = 64 / QW;          // workgroups per 64-token tile of the host's list
   typedef T VecT __attribute__((ext_vector_type(VEC)));
+  constexpr int STRIDE = KS * KT;         // from one tile of a set to its next
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
-  __shared__ int s_page[2][KT];
-  T* lds = reinterpret_cast<T*>(smem);
+  __shared__ int s_page_all[KS][2][KT];
+  const int set = KS == 1 ? 0 : __builtin_amdgcn_readfirstlane(static_cast<int>(threadIdx.x) / 256);
+  int(*s_page)[KT] = s_page_all[set];
+  T* lds = reinterpret_cast<T*>(smem) + set * 2 * TL::kElems;
 
-  const int tid = threadIdx.x, lane = tid % kWave;
+  const int tid = threadIdx.x % 256, lane = tid % kWave;
   const int wave = __builtin_amdgcn_readfirstlane(tid / kWave);
   const int col = lane % 16, grp = lane / 16;
   const int g = H / G;
@@ -312,6 +320,9 @@ __global__ __launch_bounds__(256, (HD <= 64 && VD <= 128 && sizeof(T) == 2) ? 2 
   };
   VecT kreg[TL::kKPer], vreg[TL::kVPer];
   const bool v_vectors = bs % VEC == 0;
+  const size_t k_page_stride = static_cast<size_t>(kMaps * G) * bs * HD, v_page_stride = static_cast<size_t>(G) * VD * bs;
+  const T* k_heads = kpool + static_cast<size_t>(kMaps * kvh) * bs * HD;
+  const T* v_head = vpool + static_cast<size_t>(kvh) * VD * bs;
   auto zero_vec = [] {
     VecT z;
 #pragma unroll
@@ -321,6 +332,24 @@ __global__ __launch_bounds__(256, (HD <= 64 && VD <= 128 && sizeof(T) == 2) ? 2 
   // Keys outside [lo_wg, hi_wg) become zeros: what their slots hold may be anything.
   auto fetch = [&](int kt0, int buf) {
     const bool inside = kt0 >= lo_wg && kt0 + KT <= hi_wg;
+    if (inside && v_vectors) {     // the whole tile exists and is wanted: no tests
+#pragma unroll
+      for (int n = 0; n < TL::kKPer; ++n) {
+        const int piece = min(tid + n * 256, TL::kKVecs - 1);
+        const int row = piece / (kMaps * HD / VEC), d = piece % (kMaps * HD / VEC) * VEC;
+        kreg[n] = *reinterpret_cast<const VecT*>(k_heads + max(s_page[buf][row], 0) * k_page_stride +
+                                                 static_cast<size_t>((d / HD * bs + in_page(kt0 + row)) * HD + d % HD));
+      }
+#pragma unroll
+      for (int n = 0; n < TL::kVPer; ++n) {
+        const int piece = min(tid + n * 256, TL::kVVecs - 1);
+        const int blk = piece / (VD * (16 / VEC)), d = piece % (VD * (16 / VEC)) / (16 / VEC);
+        const int row = 16 * blk + piece % (16 / VEC) * VEC;
+        vreg[n] = *reinterpret_cast<const VecT*>(v_head + max(s_page[buf][row], 0) * v_page_stride +
+                                                 static_cast<size_t>(d * bs + in_page(kt0 + row)));
+      }
+      return;
+    }
 #pragma unroll
     for (int n = 0; n < TL::kKPer; ++n) {
       const int piece = tid + n * 256;
@@ -329,8 +358,8 @@ __global__ __launch_bounds__(256, (HD <= 64 && VD <= 128 && sizeof(T) == 2) ? 2 
       const int row = piece / (kMaps * HD / VEC), d = piece % (kMaps * HD / VEC) * VEC;
       const int key = kt0 + row, page = s_page[buf][row];
       if (page >= 0 && (inside || (key >= lo_wg && key < hi_wg)))
-        kreg[n] = *reinterpret_cast<const VecT*>(
-            kpool + ((static_cast<size_t>(page) * (kMaps * G) + kMaps * kvh + d / HD) * bs + in_page(key)) * HD + d % HD);
+        kreg[n] = *reinterpret_cast<const VecT*>(k_heads + page * k_page_stride +
+                                                 static_cast<size_t>((d / HD * bs + in_page(key)) * HD + d % HD));
     }
 #pragma unroll
     for (int n = 0; n < TL::kVPer; ++n) {
@@ -340,12 +369,11 @@ __global__ __launch_bounds__(256, (HD <= 64 && VD <= 128 && sizeof(T) == 2) ? 2 
       // 16-key blocks one after the other, inside a block dimension by dimension
       const int blk = piece / (VD * (16 / VEC)), d = piece % (VD * (16 / VEC)) / (16 / VEC);
       const int row = 16 * blk + piece % (16 / VEC) * VEC, key = kt0 + row;
-      const T* base = vpool + (static_cast<size_t>(kvh) * VD + d) * bs;
-      const size_t page_stride = static_cast<size_t>(G) * VD * bs;
+      const T* base = v_head + static_cast<size_t>(d) * bs;
       if (v_vectors) {
         const int page = s_page[buf][row];
         if (page < 0 || key >= hi_wg || key + VEC <= lo_wg) continue;
-        vreg[n] = *reinterpret_cast<const VecT*>(base + page * page_stride + in_page(key));
+        vreg[n] = *reinterpret_cast<const VecT*>(base + page * v_page_stride + in_page(key));
         if (!inside)
 #pragma unroll
           for (int e = 0; e < VEC; ++e)
@@ -354,7 +382,7 @@ __global__ __launch_bounds__(256, (HD <= 64 && VD <= 128 && sizeof(T) == 2) ? 2 
 #pragma unroll
         for (int e = 0; e < VEC; ++e) {
           const int page = s_page[buf][row + e];
-          if (page >= 0 && key + e >= lo_wg && key + e < hi_wg) vreg[n][e] = base[page * page_stride + in_page(key + e)];
+          if (page >= 0 && key + e >= lo_wg && key + e < hi_wg) vreg[n][e] = base[page * v_page_stride + in_page(key + e)];
         }
       }
     }
@@ -416,23 +444,60 @@ __global__ __launch_bounds__(256, (HD <= 64 && VD <= 128 && sizeof(T) == 2) ? 2 
   };
 
   if (k_begin < k_end) {     // (a run of a cut unit may be empty: the whole workgroup agrees on it)
-    locate(k_begin, 0);
-    locate(k_begin + KT, 1);
+    const int first = k_begin + set * KT;
+    locate(first, 0);
+    locate(first + STRIDE, 1);
     __syncthreads();
-    fetch(k_begin, 0);
-    stash(0);
+    if (first < k_end) {
+      fetch(first, 0);
+      stash(0);
+    }
     __syncthreads();
     int buf = 0;
-    for (int kt0 = k_begin; kt0 < k_end; kt0 += KT, buf ^= 1) {
-      const bool more = kt0 + KT < k_end;
+    // the bounds are those of set 0, so that every wave passes the same barriers
+    for (int kb = k_begin; kb < k_end; kb += STRIDE, buf ^= 1) {
+      const int kt0 = kb + set * KT;
+      const bool more = kt0 + STRIDE < k_end;
       if (more) {
-        fetch(kt0 + KT, buf ^ 1);
-        locate(kt0 + 2 * KT, buf);        // this tile's own entries were used a round ago
+        fetch(kt0 + STRIDE, buf ^ 1);
+        locate(kt0 + 2 * STRIDE, buf);        // this tile's own entries were used a round ago
       }
-      if (active && kt0 <= pos_last_w && kt0 + KT > lo_first_w) compute(buf, kt0);
+      if (active && kt0 < k_end && kt0 <= pos_last_w && kt0 + KT > lo_first_w) compute(buf, kt0);
       if (more) stash(buf ^ 1);
       __syncthreads();
     }
+  }
+
+  if constexpr (KS == 2) {
+    // set 1 hands maximum, sum and output of both maps to the same wave and lane of set 0, map by map
+    constexpr int kHand = 2 + 4 * kValueBlocks;
+    static_assert(256 * kHand * sizeof(float) <= KS * TL::kBytes, "the hand-over goes through the tile buffers");
+    float* hand = reinterpret_cast<float*>(smem) + tid;
+#pragma unroll
+    for (int mp = 0; mp < kMaps; ++mp) {
+      if (set == 1) {
+        hand[0] = run[mp].m;
+        hand[256] = run[mp].sum[0];
+#pragma unroll
+        for (int db = 0; db < kValueBlocks; ++db)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) hand[(2 + 4 * db + e) * 256] = o[mp][db][e];
+      }
+      __syncthreads();
+      if (set == 0) {
+        const float m_other = hand[0], m_new = fmaxf(run[mp].m, m_other);
+        const float m_safe = m_new == LYP_NEG_INF ? 0.f : m_new;
+        const float a0 = fast_exp2(run[mp].m - m_safe), a1 = fast_exp2(m_other - m_safe);   // 0 for a set that saw nothing
+        run[mp].sum[0] = run[mp].sum[0] * a0 + hand[256] * a1;
+#pragma unroll
+        for (int db = 0; db < kValueBlocks; ++db)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) o[mp][db][e] = o[mp][db][e] * a0 + hand[(2 + 4 * db + e) * 256] * a1;
+        run[mp].m = m_new;
+      }
+      __syncthreads();
+    }
+    if (set == 1) return;      // (no barrier follows)
   }
 
   if (n_parts > 1) {
@@ -458,60 +523,87 @@ __global__ __launch_bounds__(256, (HD <= 64 && VD <= 128 && sizeof(T) == 2) ? 2 
 }
 
 // ------------------------------------------------------- merging partitions
-// One wave: the partitions [0, n) of one token's head (their results at index base + map * most + p),
-// put together and finished.  `values(d)` and `store(d, v)` serve the lanes.
-template <typename T>
+constexpr int kPartsMost = 128;
+constexpr int kMergeThreads = 256;
+
+// A workgroup: the first count() partitions of one token's head (their results at index base + map * most + p),
+// put together and finished.  A thread a (map, value); the maxima, weights and denominators a wave a map, a lane
+// a partition.
+template <typename T, typename Count>
 __device__ __forceinline__ void merge_head(const float* __restrict__ part_o, const float* __restrict__ part_ml, size_t base,
-                                           int most, int n, const Finish& fin, size_t token, int head,
-                                           T* __restrict__ orow, int lane) {
-  constexpr int PER = (VD + kWave - 1) / kWave;
-  float v[kMaps][PER];
-  float inv[kMaps];
+                                           int most, Count count, const Finish& fin, size_t token, int head,
+                                           T* __restrict__ orow) {
+  __shared__ float s_w[kMaps][kPartsMost];
+  __shared__ float s_inv[kMaps];
+  __shared__ float s_v[kMaps][VD];
+  __shared__ float s_ss[kMergeThreads / kWave];
+  constexpr int PER = (kMaps * VD + kMergeThreads - 1) / kMergeThreads;
+  const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
+  // The first partitions' results are asked for before anything else is known (one that does not exist holds
+  // whatever the workspace held; it is dropped): the kernel is as long as its chain of loads.
+  constexpr int kFirst = 4;
+  float first[PER][kFirst];
 #pragma unroll
-  for (int mp = 0; mp < kMaps; ++mp) {
-    const size_t at = base + static_cast<size_t>(mp) * most;
-    const float2* ml = reinterpret_cast<const float2*>(part_ml) + at;
-    float m = LYP_NEG_INF;
-    for (int p = lane; p < n; p += kWave) m = fmaxf(m, ml[p].x);
+  for (int k = 0; k < PER; ++k) {
+    const int i = min(tid + k * kMergeThreads, kMaps * VD - 1);
+#pragma unroll
+    for (int p = 0; p < kFirst; ++p)
+      first[k][p] = part_o[(base + static_cast<size_t>(i / VD) * most + min(p, most - 1)) * VD + i % VD];
+  }
+  const int n = count();
+  if (wave < kMaps) {
+    const float2* ml = reinterpret_cast<const float2*>(part_ml) + base + static_cast<size_t>(wave) * most;
+    constexpr int EACH = kPartsMost / kWave;
+    float2 r[EACH];
+    float m = LYP_NEG_INF, l = 0.f;
+#pragma unroll
+    for (int e = 0; e < EACH; ++e) {
+      const int p = lane + e * kWave;
+      r[e] = p < n ? ml[p] : float2{LYP_NEG_INF, 0.f};
+      m = fmaxf(m, r[e].x);
+    }
     m = wave_max(m);
     const float m_safe = m == LYP_NEG_INF ? 0.f : m;
-    float l = 0.f;
 #pragma unroll
-    for (int k = 0; k < PER; ++k) v[mp][k] = 0.f;
-#pragma unroll 4
-    for (int p = 0; p < n; ++p) {
-      const float2 r = ml[p];
-      const float w = fast_exp2(r.x - m_safe);
-      l += w * r.y;
-#pragma unroll
-      for (int k = 0; k < PER; ++k) {
-        const int d = lane + kWave * k;
-        if (d < VD) v[mp][k] += w * part_o[(at + p) * VD + d];
-      }
+    for (int e = 0; e < EACH; ++e) {
+      const float w = fast_exp2(r[e].x - m_safe);
+      l += w * r[e].y;
+      s_w[wave][lane + e * kWave] = w;
     }
-    inv[mp] = l > 0.f ? 1.0f / l : 0.f;
+    l = wave_sum(l);
+    if (lane == 0) s_inv[wave] = l > 0.f ? 1.0f / l : 0.f;
   }
+  __syncthreads();
+#pragma unroll
+  for (int k = 0; k < PER; ++k) {
+    const int i = tid + k * kMergeThreads;
+    if (i >= kMaps * VD) continue;
+    const int mp = i / VD, d = i % VD;
+    float acc = 0.f;
+#pragma unroll
+    for (int p = 0; p < kFirst; ++p) acc += p < n ? s_w[mp][p] * first[k][p] : 0.f;
+    const float* src = part_o + (base + static_cast<size_t>(mp) * most) * VD + d;
+#pragma unroll 8
+    for (int p = kFirst; p < n; ++p) acc += s_w[mp][p] * src[static_cast<size_t>(p) * VD];
+    s_v[mp][d] = acc * s_inv[mp];
+  }
+  __syncthreads();
+  float o = 0.f;
+  if (tid < VD) o = s_v[0][tid] - fin.lambda * s_v[1][tid];
+  const float part = wave_sum(o * o);
+  if (lane == 0) s_ss[wave] = part;
+  __syncthreads();
+  if (tid >= VD) return;
   float ss = 0.f;
 #pragma unroll
-  for (int k = 0; k < PER; ++k) {
-    v[0][k] = v[0][k] * inv[0] - fin.lambda * (v[1][k] * inv[1]);
-    if (lane + kWave * k < VD) ss += v[0][k] * v[0][k];
-  }
-  ss = wave_sum(ss);
-  const float unit = fin.post / sqrtf(ss / static_cast<float>(VD) + fin.eps);
-  const float* gate = fin.gate != nullptr ? fin.gate + token * fin.gate_ld + static_cast<size_t>(head) * VD : nullptr;
-#pragma unroll
-  for (int k = 0; k < PER; ++k) {
-    const int d = lane + kWave * k;
-    if (d >= VD) continue;
-    const float y = v[0][k] * unit;
-    orow[d] = from_f32<T>(gate != nullptr ? gated(y, gate[d]) : y);
-  }
+  for (int w = 0; w < kMergeThreads / kWave; ++w) ss += s_ss[w];
+  const float y = o * (fin.post / sqrtf(ss / static_cast<float>(VD) + fin.eps));
+  orow[tid] = from_f32<T>(fin.gate != nullptr ? gated(y, fin.gate[token * fin.gate_ld + static_cast<size_t>(head) * VD + tid]) : y);
 }
 
-// grid (H, 64, tiles); one wave: the runs of one new token's head after a cut prefill.
+// grid (H, 64, tiles): the runs of one new token's head after a cut prefill.
 template <typename T>
-__global__ __launch_bounds__(64) void paired_merge_prefill_kernel(
+__global__ __launch_bounds__(kMergeThreads) void paired_merge_prefill_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml, int n_parts, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ tile_seq, const int32_t* __restrict__ tile_q0, T* __restrict__ out, int out_stride, int H,
     Finish fin) {
@@ -521,30 +613,35 @@ __global__ __launch_bounds__(64) void paired_merge_prefill_kernel(
   const int qi = tile_q0[tile] + in_tile;
   if (qi >= q_len) return;
   const size_t token = static_cast<size_t>(tok0) + qi;
-  merge_head<T>(part_o, part_ml, ((static_cast<size_t>(tile) * 64 + in_tile) * H + head) * kMaps * n_parts, n_parts, n_parts,
-                fin, token, head, out + token * out_stride + static_cast<size_t>(head) * VD, threadIdx.x);
+  merge_head<T>(part_o, part_ml, ((static_cast<size_t>(tile) * 64 + in_tile) * H + head) * kMaps * n_parts, n_parts,
+                [&] { return n_parts; }, fin, token, head, out + token * out_stride + static_cast<size_t>(head) * VD);
 }
 
 // ---------------------------------------------------------------------- decode
-constexpr int kDecodeWaves = VD <= 128 ? 4 : 2;
-constexpr int kDecodeLeast = kDecodeWaves * 32;     // keys of the smallest partition
+// Eight waves a workgroup: wave w takes map w % 2 and share w / 2 of the partition's keys.  (The two waves of a
+// share read the same values at the same time, the second from the cache; with both maps in one wave its
+// registers would hold half as many keys on their way.)
+constexpr int kDecodeWaves = 8;
+constexpr int kShares = kDecodeWaves / kMaps;
+constexpr int kShareKeys = VD <= 128 ? 64 : 32;     // the smallest share
+constexpr int kDecodeLeast = kShares * kShareKeys;  // keys of the smallest partition
 
 // The keys one workgroup takes of the n a request's token sees when a partition may hold `most` of
-// them: as many partitions as that needs, of even size, in whole blocks of 32 keys a wave.
+// them: as many partitions as that needs, of even size, in whole smallest shares.
 __device__ __forceinline__ int decode_part_keys(int n, int most) {
   const int parts = max(1, (n + most - 1) / most);
   const int per = (n + parts - 1) / parts;
   return max(kDecodeLeast, (per + kDecodeLeast - 1) / kDecodeLeast * kDecodeLeast);
 }
 
-// LDS of a workgroup: every wave's sums of both maps for the columns that hold a head, maxima and sums.
-constexpr size_t decode_lds_floats(int g) {
-  return static_cast<size_t>(kDecodeWaves) * ((g < 16 ? g : 16) * kMaps * VD + kMaps * 32);
-}
+// LDS of a workgroup: every wave's sums of its map for the columns that hold a head, maxima and sums.
+constexpr size_t decode_lds_floats(int g) { return static_cast<size_t>(kDecodeWaves) * ((g < 16 ? g : 16) * VD + 32); }
 
 // grid (partitions, G * column groups, requests).  WHOLE: one partition a request, which the workgroup
-// finishes by itself.
-template <typename T, bool WHOLE>
+// finishes by itself.  ALIGNED: pages of a multiple of 16 slots, so that a block of 16 keys lies in one page: its
+// address is then the same for the whole wave, and a block is read whole wherever a key of it is wanted (what the
+// other slots hold, NaN included, is dropped: scores by their mask, values by clear_unseen).
+template <typename T, bool WHOLE, bool ALIGNED>
 __global__ __launch_bounds__(kDecodeWaves* kWave) void paired_decode_kernel(
     const T* __restrict__ q, int q_stride, const T* __restrict__ kpool, const T* __restrict__ vpool,
     const int32_t* __restrict__ block_tables, int table_width, const int32_t* __restrict__ q_start,
@@ -552,42 +649,38 @@ __global__ __launch_bounds__(kDecodeWaves* kWave) void paired_decode_kernel(
     float* __restrict__ part_ml, int max_parts, int most_keys, int H, int G, int bs, int page_shift, int window, int chunk,
     float scale_log2, T* __restrict__ out, int out_stride, Finish fin) {
   using O = Operands<T>;
-  constexpr int NS = O::NS, STEP = 32, NB = STEP / 16, NSTEP = NB / NS;   // 32 keys a round
+  constexpr int NS = O::NS, STEP = sizeof(T) == 2 ? kShareKeys : (VD <= 128 ? 32 : 16), NB = STEP / 16, NSTEP = NB / NS;   // keys a round
   extern __shared__ float s_dec[];
   const int lane = threadIdx.x % kWave;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave);
+  const int mp = wave % kMaps, share = wave / kMaps;
   const int col = lane % 16, grp = lane / 16;
   const int g = H / G, cols_most = min(16, g);
-  float* s_o = s_dec;                                                     // [waves][cols_most][maps][VD]
-  float* s_m = s_o + kDecodeWaves * cols_most * kMaps * VD;               // [waves][maps][16]
-  float* s_l = s_m + kDecodeWaves * kMaps * 16;
+  float* s_o = s_dec;                                      // [waves][cols_most][VD]
+  float* s_m = s_o + kDecodeWaves * cols_most * VD;        // [waves][16]
+  float* s_l = s_m + kDecodeWaves * 16;
   const int col_groups = (g + 15) / 16;
   const int kvh = blockIdx.y / col_groups, h0 = (blockIdx.y % col_groups) * 16;
   const int slot = blockIdx.z, seq = dec_seqs != nullptr ? dec_seqs[slot] : slot;
   const int ctx = ctx_len[seq];
+  const size_t token = q_start[seq];
   const int pos = ctx - 1, lo = ctx > 0 ? first_seen(pos, window, chunk) : 0;
   const int lo16 = lo / 16 * 16;
   const int part_keys = decode_part_keys(ctx - lo16, most_keys);
   const int part_begin = lo16 + static_cast<int>(blockIdx.x) * part_keys;
   if (!WHOLE && part_begin >= ctx) return;        // the whole workgroup (the merge knows how many there are)
-  const int k_begin = part_begin + wave * (part_keys / kDecodeWaves);
-  const int k_end = min(ctx, k_begin + part_keys / kDecodeWaves);
+  const int k_begin = part_begin + share * (part_keys / kShares);
+  const int k_end = min(ctx, k_begin + part_keys / kShares);
 
   const bool col_valid = h0 + col < g;
   const int head = kvh * g + h0 + (col_valid ? col : 0);
-  const size_t token = q_start[seq];
-  RowFrag<T> qf[kMaps];
+  RowFrag<T> qf;
+  qf.zero();
+  if (col_valid) qf.load(q + token * q_stride + static_cast<size_t>(head) * (kMaps * HD) + mp * HD, grp);
+  f32x4 o[kValueBlocks];
+  Running run;
 #pragma unroll
-  for (int mp = 0; mp < kMaps; ++mp) {
-    qf[mp].zero();
-    if (col_valid) qf[mp].load(q + token * q_stride + static_cast<size_t>(head) * (kMaps * HD) + mp * HD, grp);
-  }
-  f32x4 o[kMaps][kValueBlocks];
-  Running run[kMaps];
-#pragma unroll
-  for (int mp = 0; mp < kMaps; ++mp)
-#pragma unroll
-    for (int db = 0; db < kValueBlocks; ++db) o[mp][db] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int db = 0; db < kValueBlocks; ++db) o[db] = f32x4{0.f, 0.f, 0.f, 0.f};
   typename O::WFrag ones;
 #pragma unroll
   for (int e = 0; e < O::KE; ++e) ones[e] = from_f32<T>(1.f);
@@ -598,63 +691,112 @@ __global__ __launch_bounds__(kDecodeWaves* kWave) void paired_decode_kernel(
     return at < table_width ? table[at] : -1;
   };
   auto in_page = [&](int key) { return page_shift >= 0 ? key & (bs - 1) : key % bs; };
-  RowFrag<T> kf[kMaps][NB];
+  const T* k_head = kpool + static_cast<size_t>(kMaps * kvh + mp) * bs * HD;
+  const T* v_head = vpool + (static_cast<size_t>(kvh) * VD + col) * bs;
+  const size_t k_page_stride = static_cast<size_t>(kMaps * G) * bs * HD, v_page_stride = static_cast<size_t>(G) * VD * bs;
+  RowFrag<T> kf[NB];
   typename O::WFrag vf[NSTEP][kValueBlocks];
   // pages of the round's keys: this lane's key of every 16-key block (keys), and the first of its four (values)
   int kpage[NB], vpage[NB];
   auto pages_of = [&](int kb0) {
+    if constexpr (ALIGNED) {
+#pragma unroll
+      for (int u = 0; u < NB; ++u)
+        kpage[u] = __builtin_amdgcn_readfirstlane(table[min(page_shift >= 0 ? (kb0 + 16 * u) >> page_shift : (kb0 + 16 * u) / bs,
+                                                            table_width - 1)]);
+      return;
+    }
 #pragma unroll
     for (int u = 0; u < NB; ++u) {
       kpage[u] = page_at(kb0 + 16 * u + col);
       vpage[u] = page_at(kb0 + 16 * u + 4 * grp);
     }
   };
+  auto wanted = [&](int u, int kb0) {     // ALIGNED: whether any key of a block is
+    return kb0 + 16 * u < k_end && kb0 + 16 * u + 16 > lo && kpage[u] >= 0;
+  };
   auto load_keys = [&](int kb0) {
+    if constexpr (ALIGNED) {
+#pragma unroll
+      for (int u = 0; u < NB; ++u) {
+        if (wanted(u, kb0))
+          kf[u].load(k_head + kpage[u] * k_page_stride + static_cast<size_t>(in_page(kb0 + 16 * u)) * HD + col * HD, grp);
+        else
+          kf[u].zero();
+      }
+      return;
+    }
 #pragma unroll
     for (int u = 0; u < NB; ++u) {
       const int key = kb0 + 16 * u + col;
-      const bool in = key >= lo && key < k_end && kpage[u] >= 0;
-#pragma unroll
-      for (int mp = 0; mp < kMaps; ++mp) {
-        if (in)
-          kf[mp][u].load(kpool + ((static_cast<size_t>(kpage[u]) * (kMaps * G) + kMaps * kvh + mp) * bs + in_page(key)) * HD, grp);
-        else
-          kf[mp][u].zero();
-      }
+      if (key >= lo && key < k_end && kpage[u] >= 0)
+        kf[u].load(k_head + kpage[u] * k_page_stride + static_cast<size_t>(in_page(key)) * HD, grp);
+      else
+        kf[u].zero();
     }
   };
   const bool v_quads = bs % 4 == 0;
-  const size_t v_page_stride = static_cast<size_t>(G) * VD * bs;
   auto load_values = [&](int kb0) {
+    if constexpr (ALIGNED) {
+#pragma unroll
+      for (int u = 0; u < NB; ++u) {
+        const bool in = wanted(u, kb0);
+        const T* at = vpool + max(kpage[u], 0) * v_page_stride + static_cast<size_t>(kvh) * VD * bs + in_page(kb0 + 16 * u);
+        const int mine = col * bs + 4 * grp;
+#pragma unroll
+        for (int db = 0; db < kValueBlocks; ++db) {
+          typename O::Frag f;
+          if (in) {
+            f = *reinterpret_cast<const typename O::Frag*>(at + db * 16 * bs + mine);
+          } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) f[e] = from_f32<T>(0.f);
+          }
+#pragma unroll
+          for (int e = 0; e < 4; ++e) vf[u / NS][db][4 * (u % NS) + e] = f[e];
+        }
+      }
+      return;
+    }
 #pragma unroll
     for (int u = 0; u < NB; ++u) {
       const int key0 = kb0 + 16 * u + 4 * grp;
-      const T* base = vpool + (static_cast<size_t>(kvh) * VD + col) * bs;
       if (v_quads) {
         const bool any = vpage[u] >= 0 && key0 < k_end && key0 + 3 >= lo;
-        const T* at = base + static_cast<size_t>(max(vpage[u], 0)) * v_page_stride + in_page(key0);
+        const T* at = v_head + max(vpage[u], 0) * v_page_stride + in_page(key0);
 #pragma unroll
         for (int db = 0; db < kValueBlocks; ++db) {
           typename O::Frag f;
 #pragma unroll
           for (int e = 0; e < 4; ++e) f[e] = from_f32<T>(0.f);
-          if (any) f = *reinterpret_cast<const typename O::Frag*>(at + static_cast<size_t>(db) * 16 * bs);
+          if (any) f = *reinterpret_cast<const typename O::Frag*>(at + db * 16 * bs);
 #pragma unroll
-          for (int e = 0; e < 4; ++e)
-            vf[u / NS][db][4 * (u % NS) + e] = key0 + e >= lo && key0 + e < k_end ? f[e] : from_f32<T>(0.f);
+          for (int e = 0; e < 4; ++e) vf[u / NS][db][4 * (u % NS) + e] = f[e];
         }
       } else {
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           const int key = key0 + e;
           const int page = key >= lo && key < k_end ? page_at(key) : -1;
-          const T* at = base + static_cast<size_t>(max(page, 0)) * v_page_stride + in_page(key);
+          const T* at = v_head + max(page, 0) * v_page_stride + in_page(key);
 #pragma unroll
           for (int db = 0; db < kValueBlocks; ++db)
-            vf[u / NS][db][4 * (u % NS) + e] = page >= 0 ? at[static_cast<size_t>(db) * 16 * bs] : from_f32<T>(0.f);
+            vf[u / NS][db][4 * (u % NS) + e] = page >= 0 ? at[db * 16 * bs] : from_f32<T>(0.f);
         }
       }
     }
+  };
+  // keys of a quad that nobody sees: whatever their slots hold becomes zero, where a round's edge makes that necessary
+  auto clear_unseen = [&](int kb0) {
+#pragma unroll
+    for (int u = 0; u < NB; ++u)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int key = kb0 + 16 * u + 4 * grp + e;
+        if (key >= lo && key < k_end) continue;
+#pragma unroll
+        for (int db = 0; db < kValueBlocks; ++db) vf[u / NS][db][4 * (u % NS) + e] = from_f32<T>(0.f);
+      }
   };
   if (k_begin < k_end) {
     pages_of(k_begin);
@@ -663,87 +805,77 @@ __global__ __launch_bounds__(kDecodeWaves* kWave) void paired_decode_kernel(
   }
   for (int kb0 = k_begin; kb0 < k_end; kb0 += STEP) {
     const bool more = kb0 + STEP < k_end;
-    f32x4 s[kMaps][NB];
+    if (more) pages_of(kb0 + STEP);
+    f32x4 s[NB];
 #pragma unroll
-    for (int mp = 0; mp < kMaps; ++mp)
-#pragma unroll
-      for (int u = 0; u < NB; ++u) s[mp][u] = score<T>(kf[mp][u], qf[mp]);
-    if (more) {
-      pages_of(kb0 + STEP);        // the values of the next round lie in the same pages
-      load_keys(kb0 + STEP);
-    }
-    typename O::WFrag p[kMaps][NSTEP];
-    const bool full = kb0 >= lo && kb0 + STEP <= k_end;
-#pragma unroll
-    for (int mp = 0; mp < kMaps; ++mp) {
-      if (full) weigh<T, NB, false>(s[mp], p[mp], scale_log2, kb0, lo, pos, run[mp], o[mp], grp);
-      else weigh<T, NB, true>(s[mp], p[mp], scale_log2, kb0, lo, k_end - 1, run[mp], o[mp], grp);
+    for (int u = 0; u < NB; ++u) s[u] = score<T>(kf[u], qf);
+    if (more) load_keys(kb0 + STEP);
+    typename O::WFrag p[NSTEP];
+    if (kb0 >= lo && kb0 + STEP <= k_end) {
+      weigh<T, NB, false>(s, p, scale_log2, kb0, lo, pos, run, o, grp);
+    } else {
+      weigh<T, NB, true>(s, p, scale_log2, kb0, lo, k_end - 1, run, o, grp);
+      clear_unseen(kb0);
     }
 #pragma unroll
-    for (int st = 0; st < NSTEP; ++st)
+    for (int st = 0; st < NSTEP; ++st) {
+      run.sum = O::MW::mma(ones, p[st], run.sum);
 #pragma unroll
-      for (int mp = 0; mp < kMaps; ++mp) {
-        run[mp].sum = O::MW::mma(ones, p[mp][st], run[mp].sum);
-#pragma unroll
-        for (int db = 0; db < kValueBlocks; ++db) o[mp][db] = O::MW::mma(vf[st][db], p[mp][st], o[mp][db]);
-      }
+      for (int db = 0; db < kValueBlocks; ++db) o[db] = O::MW::mma(vf[st][db], p[st], o[db]);
+    }
     if (more) load_values(kb0 + STEP);
   }
 
   if (col < cols_most) {
 #pragma unroll
-    for (int mp = 0; mp < kMaps; ++mp)
-#pragma unroll
-      for (int db = 0; db < kValueBlocks; ++db)
-        *reinterpret_cast<f32x4*>(&s_o[((wave * cols_most + col) * kMaps + mp) * VD + db * 16 + 4 * grp]) = o[mp][db];
+    for (int db = 0; db < kValueBlocks; ++db)
+      *reinterpret_cast<f32x4*>(&s_o[(wave * cols_most + col) * VD + db * 16 + 4 * grp]) = o[db];
   }
   if (lane < 16) {
-#pragma unroll
-    for (int mp = 0; mp < kMaps; ++mp) {
-      s_m[(wave * kMaps + mp) * 16 + col] = col_valid ? run[mp].m : LYP_NEG_INF;
-      s_l[(wave * kMaps + mp) * 16 + col] = run[mp].sum[0];
-    }
+    s_m[wave * 16 + col] = col_valid ? run.m : LYP_NEG_INF;
+    s_l[wave * 16 + col] = run.sum[0];
   }
   __syncthreads();
 
-  // a wave a column: the waves' results of both maps put together, in the order of the waves
+  // a wave a column: the shares' results of both maps put together, in the order of the shares
   constexpr int PER = (VD + kWave - 1) / kWave;
   const int ncols = min(16, g - h0);
   for (int c = wave; c < ncols; c += kDecodeWaves) {
     const int hh = kvh * g + h0 + c;
     float v[kMaps][PER], inv[kMaps];
 #pragma unroll
-    for (int mp = 0; mp < kMaps; ++mp) {
+    for (int m2 = 0; m2 < kMaps; ++m2) {
       float m = LYP_NEG_INF;
 #pragma unroll
-      for (int w = 0; w < kDecodeWaves; ++w) m = fmaxf(m, s_m[(w * kMaps + mp) * 16 + c]);
+      for (int w = 0; w < kShares; ++w) m = fmaxf(m, s_m[(w * kMaps + m2) * 16 + c]);
       const float m_safe = m == LYP_NEG_INF ? 0.f : m;
       float l = 0.f;
 #pragma unroll
-      for (int k = 0; k < PER; ++k) v[mp][k] = 0.f;
+      for (int k = 0; k < PER; ++k) v[m2][k] = 0.f;
 #pragma unroll
-      for (int w = 0; w < kDecodeWaves; ++w) {
-        const float wgt = fast_exp2(s_m[(w * kMaps + mp) * 16 + c] - m_safe);
-        l += wgt * s_l[(w * kMaps + mp) * 16 + c];
+      for (int w = 0; w < kShares; ++w) {
+        const int from = w * kMaps + m2;
+        const float wgt = fast_exp2(s_m[from * 16 + c] - m_safe);
+        l += wgt * s_l[from * 16 + c];
 #pragma unroll
         for (int k = 0; k < PER; ++k) {
           const int d = lane + kWave * k;
-          if (d < VD) v[mp][k] += wgt * s_o[((w * cols_most + c) * kMaps + mp) * VD + d];
+          if (d < VD) v[m2][k] += wgt * s_o[(from * cols_most + c) * VD + d];
         }
       }
       if constexpr (!WHOLE) {
-        const size_t at = ((static_cast<size_t>(slot) * H + hh) * kMaps + mp) * max_parts + blockIdx.x;
+        const size_t at = ((static_cast<size_t>(slot) * H + hh) * kMaps + m2) * max_parts + blockIdx.x;
 #pragma unroll
         for (int k = 0; k < PER; ++k) {
           const int d = lane + kWave * k;
-          if (d < VD) part_o[at * VD + d] = v[mp][k];
+          if (d < VD) part_o[at * VD + d] = v[m2][k];
         }
         if (lane == 0) {
           part_ml[at * 2] = m;
           part_ml[at * 2 + 1] = l;
         }
       }
-      inv[mp] = l > 0.f ? 1.0f / l : 0.f;
+      inv[m2] = l > 0.f ? 1.0f / l : 0.f;
     }
     if constexpr (WHOLE) {
       float ss = 0.f;
@@ -767,23 +899,26 @@ __global__ __launch_bounds__(kDecodeWaves* kWave) void paired_decode_kernel(
   }
 }
 
-// grid (H, requests); one wave: the partitions of one request's token and head.
+// grid (H, requests): the partitions of one request's token and head.
 template <typename T>
-__global__ __launch_bounds__(64) void paired_merge_decode_kernel(
+__global__ __launch_bounds__(kMergeThreads) void paired_merge_decode_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml, int max_parts, int most_keys,
     const int32_t* __restrict__ q_start, const int32_t* __restrict__ ctx_len, const int32_t* __restrict__ dec_seqs,
     T* __restrict__ out, int out_stride, int H, int window, int chunk, Finish fin) {
   const int head = blockIdx.x, slot = blockIdx.y, seq = dec_seqs != nullptr ? dec_seqs[slot] : slot;
   const int ctx = ctx_len[seq];
-  const int lo16 = ctx > 0 ? first_seen(ctx - 1, window, chunk) / 16 * 16 : 0;
-  const int part_keys = decode_part_keys(ctx - lo16, most_keys);
-  const int n = min(max_parts, (ctx - lo16 + part_keys - 1) / part_keys);
   const size_t token = q_start[seq];
-  merge_head<T>(part_o, part_ml, (static_cast<size_t>(slot) * H + head) * kMaps * max_parts, max_parts, n, fin, token, head,
-                out + token * out_stride + static_cast<size_t>(head) * VD, threadIdx.x);
+  auto live = [&] {
+    const int lo16 = ctx > 0 ? first_seen(ctx - 1, window, chunk) / 16 * 16 : 0;
+    const int part_keys = decode_part_keys(ctx - lo16, most_keys);
+    return min(max_parts, (ctx - lo16 + part_keys - 1) / part_keys);
+  };
+  merge_head<T>(part_o, part_ml, (static_cast<size_t>(slot) * H + head) * kMaps * max_parts, max_parts, live, fin, token, head,
+                out + token * out_stride + static_cast<size_t>(head) * VD);
 }
 
 constexpr int kPrefillPartsMost = 16;
+constexpr int kPartAlone = 256;    // partitions up to this size are merged in pairs where that leaves one
 
 static int shift_of(int bs) {
   if ((bs & (bs - 1)) != 0) return -1;
@@ -816,8 +951,7 @@ extern "C" {
 int lyp_paired_key_dim() { return HD; }
 int lyp_paired_value_dim() { return VD; }
 
-// Keys per workgroup at most for a decode launch over n_seqs requests whose tokens see up to max_keys keys.  Both
-// are rounded up to powers of two, so that a recorded launch (sized for a bucket) and a direct one choose alike.
+// Keys per workgroup at most for a decode launch over n_seqs requests whose tokens see up to max_keys keys.
 int lyp_paired_decode_plan(int n_seqs, int max_keys, int H, int G) {
   auto pow2 = [](int v, int least) {
     int p = least;
@@ -826,12 +960,12 @@ int lyp_paired_decode_plan(int n_seqs, int max_keys, int H, int G) {
   };
   const int g = H / std::max(G, 1);
   const long long base = static_cast<long long>(pow2(n_seqs, 1)) * G * ((g + 15) / 16);
-  const int keys = pow2(max_keys, 64);
   int part = kDecodeLeast;
+  while ((max_keys + part - 1) / part > kPartsMost) part *= 2;
   // partitions grow while the launch keeps a workgroup per compute unit
-  while (part < keys && base * ((keys + 2 * part - 1) / (2 * part)) >= compute_units()) part *= 2;
-  // two partitions a request are not worth the merge they need
-  if (2 * part >= keys && part < 2048) part = std::max(part, keys);
+  while (part < max_keys && base * ((max_keys + 2 * part - 1) / (2 * part)) >= compute_units()) part *= 2;
+  // two short partitions a request are not worth the merge they need
+  if (2 * part >= max_keys && part < max_keys && part <= kPartAlone) part *= 2;
   return part;
 }
 
@@ -845,7 +979,7 @@ int lyp_paired_prefill_plan(int n_tiles, int max_keys, int H, int G, int dtype) 
   const int kt = dtype == kF32 ? Tile<float>::kKeys : Tile<bf16_t>::kKeys;
   const int tiles = (max_keys + kt - 1) / kt;
   int parts = 1;
-  while (parts < kPrefillPartsMost && wgs * parts < compute_units() && tiles / (2 * parts) >= 4) parts *= 2;
+  while (parts < kPrefillPartsMost && wgs * parts < compute_units() && tiles / (2 * parts) >= 8) parts *= 2;
   return parts;
 }
 
@@ -866,18 +1000,31 @@ int lyp_paired_prefill(const void* q, int q_stride, void* out, int out_stride, c
   const Finish fin{lambda, eps, post, gate, gate_ld};
   const dim3 grid(G * ((g + gh - 1) / gh), n_tiles * gh, n_parts);
   const float scale_log2 = scale * kLog2e;
-#define LYP_PAIRED(T, GH)                                                                                              \
+  // Two sets of waves a workgroup while the launch has at most `kSplitBelow` workgroups per compute unit.
+  constexpr int kSplitBelow = 2;
+  const bool split = static_cast<long long>(grid.x) * grid.y * grid.z <= static_cast<long long>(kSplitBelow) * compute_units();
+#define LYP_PAIRED_KS(T, GH, KS)                                                                                       \
   do {                                                                                                                 \
     static bool asked = false;   /* the tiles may take more LDS than a kernel gets unasked */                          \
     if (!asked) {                                                                                                      \
-      (void)hipFuncSetAttribute(reinterpret_cast<const void*>(paired_prefill_kernel<T, GH>),                           \
-                                hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(Tile<T>::kBytes));        \
+      (void)hipFuncSetAttribute(reinterpret_cast<const void*>(paired_prefill_kernel<T, GH, KS>),                       \
+                                hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(KS * Tile<T>::kBytes));   \
       asked = true;                                                                                                    \
     }                                                                                                                  \
-    paired_prefill_kernel<T, GH><<<grid, 256, Tile<T>::kBytes, stream>>>(                                              \
+    paired_prefill_kernel<T, GH, KS><<<grid, 256 * KS, KS * Tile<T>::kBytes, stream>>>(                                \
         static_cast<const T*>(q), q_stride, static_cast<T*>(out), out_stride, static_cast<const T*>(kpool),            \
         static_cast<const T*>(vpool), block_tables, table_width, q_start, ctx_len, tile_seq, tile_q0, n_tiles, H, G,   \
         bs, shift_of(bs), window, chunk, scale_log2, fin, part_o, part_ml, n_parts);                                   \
+  } while (0)
+#define LYP_PAIRED(T, GH)                                   \
+  do {                                                      \
+    if constexpr (Tile<T>::kMaySplit) {                     \
+      if (split) {                                          \
+        LYP_PAIRED_KS(T, GH, 2);                            \
+        break;                                              \
+      }                                                     \
+    }                                                       \
+    LYP_PAIRED_KS(T, GH, 1);                                \
   } while (0)
 #define LYP_PAIRED_T(T)                   \
   do {                                    \
@@ -885,13 +1032,14 @@ int lyp_paired_prefill(const void* q, int q_stride, void* out, int out_stride, c
     else if (gh == 2) LYP_PAIRED(T, 2);   \
     else LYP_PAIRED(T, 1);                \
     if (n_parts > 1)                      \
-      paired_merge_prefill_kernel<T><<<dim3(H, 64, n_tiles), 64, 0, stream>>>(                       \
+      paired_merge_prefill_kernel<T><<<dim3(H, 64, n_tiles), kMergeThreads, 0, stream>>>(            \
           part_o, part_ml, n_parts, q_start, tile_seq, tile_q0, static_cast<T*>(out), out_stride, H, fin); \
   } while (0)
   if (dtype == kF32) LYP_PAIRED_T(float);
   else LYP_PAIRED_T(bf16_t);
 #undef LYP_PAIRED_T
 #undef LYP_PAIRED
+#undef LYP_PAIRED_KS
   LYP_LAUNCH_CHECK("paired_prefill");
   return 0;
 }
@@ -907,7 +1055,8 @@ int lyp_paired_decode(const void* q, int q_stride, void* out, int out_stride, co
   if (check_common("paired_decode", H, G, bs, table_width, q_stride, out_stride, window, chunk, q, kpool, vpool, gate, gate_ld))
     return -1;
   LYP_REQUIRE(scale > 0.f, "paired_decode: a scale of %g", static_cast<double>(scale));
-  LYP_REQUIRE(n_seqs >= 0 && n_seqs <= 65535 && max_parts > 0 && part_keys > 0 && part_keys % kDecodeLeast == 0,
+  LYP_REQUIRE(n_seqs >= 0 && n_seqs <= 65535 && max_parts > 0 && max_parts <= kPartsMost && part_keys > 0 &&
+                  part_keys % kDecodeLeast == 0,
               "paired_decode: %d requests, %d partitions of %d keys", n_seqs, max_parts, part_keys);
   LYP_REQUIRE(max_parts == 1 || (part_o && part_ml), "paired_decode: no workspace");
   LYP_REQUIRE(dtype == kF32 || dtype == kBF16, "paired_decode: unknown dtype %d", dtype);
@@ -918,21 +1067,26 @@ int lyp_paired_decode(const void* q, int q_stride, void* out, int out_stride, co
   const size_t lds = decode_lds_floats(g) * sizeof(float);
   const dim3 grid(max_parts, G * col_groups, n_seqs);
   const float scale_log2 = scale * kLog2e;
-#define LYP_PAIRED_DEC(T, WHOLE)                                                                                       \
+#define LYP_PAIRED_DEC_A(T, WHOLE, ALIGNED)                                                                            \
   do {                                                                                                                 \
     if (lds > 48 * 1024) {                                                                                             \
       static bool asked = false;                                                                                       \
       if (!asked) {                                                                                                    \
-        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(paired_decode_kernel<T, WHOLE>),                       \
+        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(paired_decode_kernel<T, WHOLE, ALIGNED>),              \
                                   hipFuncAttributeMaxDynamicSharedMemorySize,                                          \
                                   static_cast<int>(decode_lds_floats(16) * sizeof(float)));                            \
         asked = true;                                                                                                  \
       }                                                                                                                \
     }                                                                                                                  \
-    paired_decode_kernel<T, WHOLE><<<grid, kDecodeWaves * kWave, lds, stream>>>(                                       \
+    paired_decode_kernel<T, WHOLE, ALIGNED><<<grid, kDecodeWaves * kWave, lds, stream>>>(                              \
         static_cast<const T*>(q), q_stride, static_cast<const T*>(kpool), static_cast<const T*>(vpool), block_tables,  \
         table_width, q_start, ctx_len, dec_seqs, part_o, part_ml, max_parts, part_keys, H, G, bs, shift_of(bs), window, \
         chunk, scale_log2, static_cast<T*>(out), out_stride, fin);                                                     \
+  } while (0)
+#define LYP_PAIRED_DEC(T, WHOLE)                             \
+  do {                                                       \
+    if (bs % 16 == 0) LYP_PAIRED_DEC_A(T, WHOLE, true);      \
+    else LYP_PAIRED_DEC_A(T, WHOLE, false);                  \
   } while (0)
 #define LYP_PAIRED_DEC_T(T)                                                                                            \
   do {                                                                                                                 \
@@ -940,7 +1094,8 @@ int lyp_paired_decode(const void* q, int q_stride, void* out, int out_stride, co
       LYP_PAIRED_DEC(T, true);                                                                                         \
     } else {                                                                                                           \
       LYP_PAIRED_DEC(T, false);                                                                                        \
-      paired_merge_decode_kernel<T><<<dim3(H, n_seqs), 64, 0, stream>>>(part_o, part_ml, max_parts, part_keys, q_start, \
+      paired_merge_decode_kernel<T><<<dim3(H, n_seqs), kMergeThreads, 0, stream>>>(part_o, part_ml, max_parts,         \
+                                                                        part_keys, q_start,                            \
                                                                         ctx_len, dec_seqs, static_cast<T*>(out),       \
                                                                         out_stride, H, window, chunk, fin);            \
     }                                                                                                                  \
@@ -949,6 +1104,7 @@ int lyp_paired_decode(const void* q, int q_stride, void* out, int out_stride, co
   else LYP_PAIRED_DEC_T(bf16_t);
 #undef LYP_PAIRED_DEC_T
 #undef LYP_PAIRED_DEC
+#undef LYP_PAIRED_DEC_A
   LYP_LAUNCH_CHECK("paired_decode");
   return 0;
 }

@@ -1469,10 +1469,10 @@ def paired_attn_fits_matrix_cores(key_dim: int, value_dim: int) -> bool:
 
 
 def visible_keys(max_ctx: int, window: int, chunk: int, tokens: int = 1) -> int:
-    """Most keys that ``tokens`` neighbouring tokens of a request of up to ``max_ctx`` see between them, and the 15
-    before them that a block of 16 keys may begin with."""
+    """Most keys that ``tokens`` neighbouring tokens of a request of up to ``max_ctx`` see between them, and those
+    before them that a block of 16 keys begins with (none before a chunk of a multiple of 16)."""
     reach = window or chunk
-    return min(max_ctx, reach + tokens - 1 + 15) if reach else max_ctx
+    return min(max_ctx, reach + tokens - 1 + (15 if window or chunk % 16 else 0)) if reach else max_ctx
 
 
 def paired_decode_launch(n_dec: int, max_ctx: int, *, num_heads: int, num_kv_heads: int, dim: int, vdim: int,

@@ -157,7 +157,7 @@ def test_differential_attention_of_single_tokens(dtype, mask, heads, dims):
     rows = [int(pg.q_start[b]) for b in (0, 1, 4, 5, 6)]
     sizes = dict(num_heads=H, num_kv_heads=G, dim=D, vdim=V, window=window, chunk=chunk)
     bound = ops.visible_keys(411, window, chunk)
-    least = 4 * 32 if V <= 128 else 2 * 32
+    least = 8 * 32 if V <= 128 else 4 * 32
     for launch in (ops.paired_decode_launch(6, 411, **sizes), dict(part_keys=least, max_parts=-(-bound // least)),
                    dict(part_keys=512, max_parts=1)):
         n = 6 * H * 2 * launch["max_parts"]
@@ -185,7 +185,7 @@ def test_differential_attention_at_other_page_sizes_and_without_a_gate(dtype, bs
     out = torch.full((pg.T, H * V), float("nan"), dtype=tdt(dtype), device=DEV)
     ops.paired_prefill(q, out, kpool, vpool, bt, q_start, ctx, ints([b for _, b, _ in tiles]), ints([q0 for _, _, q0 in tiles]),
                        len(tiles), dict(parts=1), scale=scale, **sizes, **opts)
-    ops.paired_decode(q, out, kpool, vpool, bt, q_start, ctx, ints([1]), 1, dict(part_keys=128, max_parts=1), scale=scale, **sizes, **opts)
+    ops.paired_decode(q, out, kpool, vpool, bt, q_start, ctx, ints([1]), 1, dict(part_keys=256, max_parts=1), scale=scale, **sizes, **opts)
     close(out, want, dtype, f"pages of {bs}", tol=3e-5 if dtype == "float32" else 2.5e-2)
 
 
@@ -207,7 +207,7 @@ def test_one_key_among_many_stands_out():
             q, kpool, vpool, scale, opts, want = paired_case(pg, H, G, D, V, "float32", seed=3, window=window, chunk=chunk, spike=spike)
             bt, q_start, _, ctx = pg.device()
             sizes = dict(num_heads=H, num_kv_heads=G, dim=D, vdim=V, window=window, chunk=chunk)
-            for most in (128, 256, 1024):
+            for most in (256, 512, 1024):
                 parts = -(-ops.visible_keys(L, window, chunk) // most)
                 n = H * 2 * parts
                 out = torch.empty(1, H * V, device=DEV)
@@ -247,7 +247,7 @@ def test_mismatches_are_errors():
         with pytest.raises(ops.KernelError):
             ops.paired_prefill(*args, scale=scale, **{**sizes, **kw}, **opts)
     with pytest.raises(ops.KernelError):
-        ops.paired_decode(q, out, kpool, vpool, bt, q_start, ctx, None, 2, dict(part_keys=128, max_parts=1), scale=scale, **sizes, **opts)
+        ops.paired_decode(q, out, kpool, vpool, bt, q_start, ctx, None, 2, dict(part_keys=256, max_parts=1), scale=scale, **sizes, **opts)
 
 
 # --------------------------------------------------------------- latent windows
