@@ -959,6 +959,96 @@ __global__ void moe_combine_kernel(const T* __restrict__ y, const int32_t* __res
   }
 }
 
+// The weighted sum straight onto the residual stream, and the RMS norm of the stream's new row: as
+// moe_combine_kernel, v = h[row] + share[row] * shared + sum_k wgt[row, k] * y[place], v to h, and
+// v / sqrt(mean(v^2) + eps) * w to out.  One workgroup a row, the row in registers: G groups of 4 values a thread.
+constexpr int kCombineNormThreads = 256;
+constexpr int kCombineNormMost = 8;     // groups a thread may hold: rows of up to 8,192 values
+
+template <typename T, typename TW, int G>
+__global__ __launch_bounds__(kCombineNormThreads) void moe_combine_norm_kernel(
+    const T* __restrict__ y, const int32_t* __restrict__ place_of, const float* __restrict__ wgt, int top,
+    const T* __restrict__ shared, const float* __restrict__ share, float* __restrict__ h, const TW* __restrict__ w, float eps,
+    T* __restrict__ out, int H) {
+  __shared__ int32_t s_at[kMostTop];
+  __shared__ float s_w[kMostTop];
+  __shared__ float s_ss[kCombineNormThreads / kWave];
+  typedef T VecT __attribute__((ext_vector_type(4)));
+  typedef TW VecW __attribute__((ext_vector_type(4)));
+  const int row = blockIdx.x;
+  const size_t at = static_cast<size_t>(row) * H;
+  if (threadIdx.x < top) {
+    s_at[threadIdx.x] = place_of[static_cast<size_t>(row) * top + threadIdx.x];
+    s_w[threadIdx.x] = wgt != nullptr ? wgt[static_cast<size_t>(row) * top + threadIdx.x] : 1.0f / static_cast<float>(top);
+  }
+  f32x4 v[G];
+  VecW wv[G];
+#pragma unroll
+  for (int u = 0; u < G; ++u) {
+    const int c = (threadIdx.x + u * kCombineNormThreads) * 4;
+    v[u] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (c < H) {
+      v[u] = *reinterpret_cast<const f32x4*>(h + at + c);
+      wv[u] = *reinterpret_cast<const VecW*>(w + c);
+    }
+  }
+  // the same sums in the same order as the combining kernel's, added to the stream as a whole
+  const float part = share != nullptr ? share[row] : 1.0f;
+  f32x4 sum[G];
+#pragma unroll
+  for (int u = 0; u < G; ++u) {
+    const int c = (threadIdx.x + u * kCombineNormThreads) * 4;
+    sum[u] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (shared != nullptr && c < H) {
+      const VecT s = *reinterpret_cast<const VecT*>(shared + at + c);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) sum[u][i] = part * to_f32(s[i]);
+    }
+  }
+  __syncthreads();
+#pragma unroll 4
+  for (int k = 0; k < top; ++k) {
+    const T* src = y + static_cast<size_t>(s_at[k]) * H;
+    const float wk = s_w[k];
+#pragma unroll
+    for (int u = 0; u < G; ++u) {
+      const int c = (threadIdx.x + u * kCombineNormThreads) * 4;
+      if (c >= H) continue;
+      const VecT s = *reinterpret_cast<const VecT*>(src + c);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) sum[u][i] += wk * to_f32(s[i]);
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int u = 0; u < G; ++u) {
+    const int c = (threadIdx.x + u * kCombineNormThreads) * 4;
+    if (c >= H) continue;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      v[u][i] += sum[u][i];
+      ss += v[u][i] * v[u][i];
+    }
+    *reinterpret_cast<f32x4*>(h + at + c) = v[u];
+  }
+  ss = wave_sum(ss);
+  if (threadIdx.x % kWave == 0) s_ss[threadIdx.x / kWave] = ss;
+  __syncthreads();
+  ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < kCombineNormThreads / kWave; ++i) ss += s_ss[i];
+  const float inv = 1.0f / sqrtf(ss / static_cast<float>(H) + eps);
+#pragma unroll
+  for (int u = 0; u < G; ++u) {
+    const int c = (threadIdx.x + u * kCombineNormThreads) * 4;
+    if (c >= H) continue;
+    VecT o;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) o[i] = from_f32<T>(v[u][i] * inv * to_f32(wv[u][i]));
+    *reinterpret_cast<VecT*>(out + at + c) = o;
+  }
+}
+
 // The weighted sum straight onto the residual stream, with what the next branch reads of it
 // (stream_map.h): v = base[row] + sum_k wgt[row, k] * y[place_of[row * top + k]], v to h (where given),
 // map(v) to out.  A thread takes V neighbouring columns; blockIdx.y walks the row.
@@ -1299,6 +1389,40 @@ int lyp_moe_combine(const void* y, const int32_t* place_of, const float* wgt, in
   }
 #undef LYP_COMBINE
   LYP_LAUNCH_CHECK("moe_combine");
+  return 0;
+}
+
+// As lyp_moe_combine, but h [rows, H] float += the sum, and out [rows, H] of dtype = its RMS norm times w [H] (float or
+// bfloat16).  Returns 1 (and does nothing) for rows that the kernel does not take.
+int lyp_moe_combine_norm(const void* y, const int32_t* place_of, const float* wgt, int top, const void* shared,
+                         const float* share, float* h, const void* w, int w_f32, float eps, void* out, int dtype, int rows,
+                         int H, hipStream_t stream) {
+  LYP_REQUIRE(rows >= 0 && H > 0 && top > 0 && top <= kMostTop && (share == nullptr || shared != nullptr) && h && w && out,
+              "moe_combine_norm: %d rows of %d, %d choices", rows, H, top);
+  LYP_REQUIRE(dtype == kF32 || dtype == kBF16, "moe_combine_norm: unknown dtype %d", dtype);
+  auto aligned = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+  const int groups = (H + 4 * kCombineNormThreads - 1) / (4 * kCombineNormThreads);
+  if (H % 4 != 0 || groups > kCombineNormMost || !aligned(y) || !aligned(shared) || !aligned(h) || !aligned(w) || !aligned(out))
+    return 1;
+  if (rows == 0) return 0;
+#define LYP_CN(T, TW, G)                                                                                               \
+  moe_combine_norm_kernel<T, TW, G><<<rows, kCombineNormThreads, 0, stream>>>(                                         \
+      static_cast<const T*>(y), place_of, wgt, top, static_cast<const T*>(shared), share, h, static_cast<const TW*>(w), eps, \
+      static_cast<T*>(out), H)
+#define LYP_CN_W(T, TW)                     \
+  do {                                      \
+    if (groups == 1) LYP_CN(T, TW, 1);      \
+    else if (groups == 2) LYP_CN(T, TW, 2); \
+    else if (groups <= 4) LYP_CN(T, TW, 4); \
+    else LYP_CN(T, TW, kCombineNormMost);   \
+  } while (0)
+  if (dtype == kF32 && w_f32) LYP_CN_W(float, float);
+  else if (dtype == kF32) LYP_CN_W(float, bf16_t);
+  else if (w_f32) LYP_CN_W(bf16_t, float);
+  else LYP_CN_W(bf16_t, bf16_t);
+#undef LYP_CN_W
+#undef LYP_CN
+  LYP_LAUNCH_CHECK("moe_combine_norm");
   return 0;
 }
 

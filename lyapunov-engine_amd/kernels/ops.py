@@ -145,6 +145,8 @@ def core() -> ctypes.CDLL:
         lib.lyp_glu_clamped.argtypes = [c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_float, c_float, c_int, c_void_p]
         lib.lyp_moe_combine.argtypes = [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
                                         c_int, c_int, c_void_p]
+        lib.lyp_moe_combine_norm.argtypes = [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
+                                             c_float, c_void_p, c_int, c_int, c_int, c_void_p]
         lib.lyp_group_rmsnorm.argtypes = [c_void_p, c_void_p, c_int, c_int, c_longlong, c_void_p, c_void_p, c_void_p, c_int,
                                           c_void_p, c_int, c_int, c_int, c_float, c_void_p]
         lib.lyp_add_sinusoid.argtypes = [c_void_p, c_void_p, c_int, c_int, c_double, c_void_p]
@@ -1849,14 +1851,36 @@ def moe_combine(y: torch.Tensor, plan: MoePlan, weights: torch.Tensor | None, ro
 
 
 class PendingExperts:
-    """The weighted sum over a token's experts, not carried out yet: ``stream_next`` puts it straight
-    onto the residual stream; ``run()`` gives it as ``moe_combine`` does."""
+    """The weighted sum over a token's experts (and what every token uses), not carried out yet: ``stream_next``
+    and ``experts_rmsnorm`` put it straight onto the residual stream; ``run()`` gives it as ``moe_combine``
+    does."""
 
-    def __init__(self, y: torch.Tensor, plan: MoePlan, weights: torch.Tensor | None, rows: int):
-        self.y, self.plan, self.weights, self.rows = y, plan, weights, rows
+    def __init__(self, y: torch.Tensor, plan: MoePlan, weights: torch.Tensor | None, rows: int,
+                 shared: torch.Tensor | None = None, share: torch.Tensor | None = None):
+        self.y, self.plan, self.weights, self.rows, self.shared, self.share = y, plan, weights, rows, shared, share
 
     def run(self) -> torch.Tensor:
-        return moe_combine(self.y, self.plan, self.weights, self.rows)
+        return moe_combine(self.y, self.plan, self.weights, self.rows, shared=self.shared, share=self.share)
+
+
+def experts_rmsnorm(h: torch.Tensor, pending: PendingExperts, weight: torch.Tensor, eps: float, out: torch.Tensor) -> bool:
+    """h += the pending sum, out = rmsnorm(h) * weight, in one kernel; False (nothing done) for rows it does not take."""
+    p = pending
+    _dev(h, p.y, p.weights, p.shared, p.share, weight, out)
+    _f32(h, p.weights, p.share)
+    T, H = h.shape
+    if tuple(out.shape) != (T, H) or p.y.shape[1] != H or out.dtype != p.y.dtype or weight.numel() != H or p.rows != T or \
+            T * p.plan.top != p.plan.pairs or (p.weights is not None and p.weights.numel() != p.plan.pairs) or \
+            (p.shared is not None and (tuple(p.shared.shape) != (T, H) or p.shared.dtype != p.y.dtype)) or \
+            (p.share is not None and p.share.numel() != T):
+        raise KernelError(f"experts_rmsnorm: h {tuple(h.shape)}, experts' rows {tuple(p.y.shape)} {p.y.dtype}, out {tuple(out.shape)}")
+    lib = core()
+    rc = lib.lyp_moe_combine_norm(_p(p.y), _p(p.plan.place_of), _p(p.weights), p.plan.top, _p(p.shared), _p(p.share), _p(h),
+                                  _p(weight), int(_code(weight.dtype) == F32), float(eps), _p(out), _code(out.dtype), T, H,
+                                  _stream())
+    if rc < 0:
+        _check(rc, lib)
+    return rc == 0
 
 
 # ------------------------------------ a residual stream read feature by feature
@@ -1941,7 +1965,7 @@ def stream_next(h: torch.Tensor, delta, smap: StreamMap, dtype: torch.dtype, row
                     _check(rc, lib)
                 if rc == 0:
                     return out
-        elif delta.y.dtype == dtype and delta.y.shape[1] == H and delta.rows == T:
+        elif delta.y.dtype == dtype and delta.y.shape[1] == H and delta.rows == T and delta.shared is None:
             _dev(delta.y, delta.weights)
             _check(lib.lyp_moe_combine_stream(_p(delta.y), _p(delta.plan.place_of), _p(delta.weights), delta.plan.top,
                                               _p(keeps), _p(base), smap.kind, smap.alpha, _p(smap.weight), _p(smap.bias),

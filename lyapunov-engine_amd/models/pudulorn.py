@@ -81,7 +81,7 @@ def pudulorn_spec(cfg: PudulornConfig) -> ModelSpec:
                 "intermediate_size": int(lc.mlp["expert"]["ff"]), "limit": math.inf, "gate_slope": 1.0, "plus": 0.0,
                 "router_bias": False, "scores": "all", "scale": float(lc.mlp["router"]["scale"]),
                 "shared_size": int(shared["ff"]) if shared is not None else 0, "shared_limit": math.inf,
-                "shared_gate": shared is not None})
+                "shared_gate": shared is not None, "pending": True})
         layers.append(LayerSpec(block="prenorm", mixer=mixer, ffn=ffn, norm1=norm(), norm2=norm(), names=LAYER_NAMES))
     return ModelSpec(
         vocab_size=cfg.vocab, hidden_size=cfg.width, layers=tuple(layers), schedule=running_order(cfg),

@@ -229,7 +229,8 @@ def settled(norm, h, delta):
         delta = delta.join(h)
     if isinstance(delta, ops.Restart) and not getattr(norm, "takes_any_delta", False):
         delta = delta.join(h)
-    if isinstance(delta, ops.PendingExperts) and not getattr(norm, "takes_any_delta", False):
+    if isinstance(delta, ops.PendingExperts) and not (getattr(norm, "takes_any_delta", False) or
+                                                      getattr(norm, "takes_experts", False)):
         delta = delta.run()
     if isinstance(delta, ops.PendingLinear) and not getattr(norm, "can_defer", False):
         delta = delta.run()

@@ -54,8 +54,9 @@ class RMSNorm(Norm):
             y = y[0] if y.shape[0] == 1 else ops.sum_parts(y, torch.float32)     # one slice: nothing to add up
         return ops.JoiningBranch(y, self.weight_f, self.eps, mult)
 
-    # A delta may be an ops.JoiningBranch: the sum and this norm are then one kernel.
+    # A delta may be an ops.JoiningBranch or an ops.PendingExperts: the sum and this norm are then one kernel.
     joins_branches = True
+    takes_experts = True
 
     # With ``lazy`` the norm may add the delta and hand the rows on as an
     # ops.PendingNorm for the consumer's kernel to norm on its way in.
@@ -72,6 +73,11 @@ class RMSNorm(Norm):
                                        rows=rows, conv=conv)
             return ops.branch_join(h, delta.y, delta.weight, delta.mult, delta.eps, shift=delta.shift,
                                    next_weight=self.weight_f, eps_next=self.eps, out=out, rows=rows, conv=conv)
+        if isinstance(delta, ops.PendingExperts):
+            out = torch.empty((h.shape[0], self.size), dtype=ctx.dtype, device=h.device)
+            if rows is None and ops.experts_rmsnorm(h, delta, self.multiplier, self.eps, out):
+                return out
+            delta = delta.run()
         if lazy and rows is None:
             pending, delta = ops.rmsnorm_pending(h, self.multiplier, self.eps, ctx.dtype, delta)
             if pending is not None:

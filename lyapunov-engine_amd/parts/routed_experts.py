@@ -37,7 +37,9 @@ class RoutedExperts(FeedForward):
     def __init__(self, hidden_size: int, num_experts: int, top: int, intermediate_size: int, limit: float,
                  gate_slope: float = 1.702, shared_size: int = 0, shared_limit: float = 0.0, plus: float = 1.0,
                  router_bias: bool = True, scores: str = "chosen", scale: float = 1.0, shared_gate: bool = False,
-                 names: Optional[dict] = None):
+                 pending: bool = False, names: Optional[dict] = None):
+        """``pending``: without another branch to add, the weighted sum is left to the norm that follows
+        (ops.PendingExperts), for one that takes it."""
         if not 1 <= top <= num_experts or intermediate_size <= 0 or shared_size < 0:
             raise ValueError(f"routed experts: {top} of {num_experts} experts of {intermediate_size}, shared {shared_size}")
         self.hidden_size, self.num_experts, self.top = int(hidden_size), int(num_experts), int(top)
@@ -46,7 +48,7 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"routed experts: scores {scores!r}, a gate for a shared expert of {shared_size}")
         self.shared_size, self.shared_limit = int(shared_size), float(shared_limit)
         self.plus, self.has_bias, self.scale = float(plus), bool(router_bias), float(scale)
-        self.over_all, self.shared_gate = scores == "all", bool(shared_gate)
+        self.over_all, self.shared_gate, self.pending = scores == "all", bool(shared_gate), bool(pending)
         n = dict(router="router", router_bias="router.b", expert="e{j}.", shared="shared.", gate="gate", up="up",
                  down="down", shared_gate="sg")
         n.update(names or {})
@@ -93,8 +95,8 @@ class RoutedExperts(FeedForward):
         self.down = self.down.view(stacked, H, I)
 
     def forward(self, ctx: StepContext, x, addend=None):
-        """-> float [1, T, hidden] (one slice of partial sums): the experts' weighted outputs, the
-        shared expert's and ``addend`` (the other branch's output, activations [T, hidden])."""
+        """-> float [1, T, hidden] (one slice of partial sums; or see ``pending``): the experts' weighted outputs,
+        the shared expert's and ``addend`` (the other branch's output, activations [T, hidden])."""
         T = x.shape[0]
         always = self.num_experts if self.shared_folded else -1
         idx, wgt, plan, *share = ops.moe_route_from(x, self.router_f, self.router_bias_f, self.top, always,
@@ -110,6 +112,8 @@ class RoutedExperts(FeedForward):
             shared = ops.linear(gu, self.shared_down, out_dtype=ctx.dtype)
         if addend is not None:
             addend = ops.as_delta(addend, ctx.dtype)
+        elif self.pending:
+            return ops.PendingExperts(y, plan, wgt, T, shared, share[0] if share else None)
         return ops.moe_combine(y, plan, wgt, T, addend=addend, shared=shared, share=share[0] if share else None)
 
 

@@ -473,6 +473,45 @@ def test_weights_are_shares_of_all_scores(dtype, T, E, top, K):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H", [64, 320, 1024, 2052, 4096, 8192, 70, 8196])     # the last two: sum and norm apart
+@pytest.mark.parametrize("T", [1, 33])
+def test_the_experts_sum_that_ends_in_the_norm(dtype, H, T):
+    """The weighted sum with and without a shared expert and its share, weights given and equal, onto the stream and
+    through a norm in one kernel; picked rows leave the stream alone."""
+    from lyapunov_engine_amd.kernels import ops
+    from lyapunov_engine_amd.parts.base import StepContext
+    from lyapunov_engine_amd.parts.norm import RMSNorm
+
+    top, E = 3, 5
+    g = torch.Generator().manual_seed(H + T)
+    idx = torch.stack([torch.randperm(E, generator=g)[:top] for _ in range(T)]).int().to(DEV)
+    plan = ops.moe_sort(idx, E)
+    y = torch.randn(T * top, H, generator=g).to(tdt(dtype))
+    place = plan.place_of.long().cpu().view(T, top)
+    wgt, share = torch.rand(T, top, generator=g), torch.rand(T, generator=g)
+    shared = torch.randn(T, H, generator=g).to(tdt(dtype))
+    h0 = torch.randn(T, H, generator=g) * 2
+    norm = RMSNorm(H, 1e-5, tensor="", one_plus=True)
+    norm.weight = (0.3 * torch.randn(H, generator=g)).to(tdt(dtype)).to(DEV)
+    ctx = StepContext(device=torch.device(DEV), dtype=tdt(dtype), T=T, B=1, token_ids=None, positions=None, q_start=None, ctx_len=None,
+                      state_slots=None, logit_rows=None, R=0, groups=[])
+    for w, s, f in ((wgt, shared, share), (wgt, None, None), (None, None, None), (wgt, shared, None)):
+        want = h0.double() + ((torch.full((T, top), 1 / top) if w is None else w).double()[..., None] * y.double()[place]).sum(1)
+        if s is not None:
+            want = want + s.double() * (1.0 if f is None else f.double()[:, None])
+        dev = lambda t: None if t is None else t.to(DEV)
+        pending = lambda: ops.PendingExperts(y.to(DEV), plan, dev(w), T, dev(s), dev(f))
+        h = h0.to(DEV)
+        out = norm.forward(ctx, h, pending(), lazy=True)
+        close(h, want, "float32", "the stream")
+        normed = DP.shifted_rms_norm(want, norm.weight.double().cpu(), 1e-5)
+        close(out, normed, dtype, "the norm")
+        h = h0.to(DEV)
+        close(norm.forward(ctx, h, pending(), rows=ints([T - 1, 0])), normed[[T - 1, 0]], dtype, "picked rows")
+        assert torch.equal(h.cpu(), h0)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("shape", [(1, 16, 4, 128, 64, 128), (9, 5, 2, 72, 28, 28), (70, 12, 3, 128, 64, 96), (300, 6, 2, 256, 512, 512),
                                    (600, 3, 3, 64, 40, 20), (40, 7, 2, 512, 32, 0), (3, 1, 1, 40, 48, 50)])
 def test_the_routed_part_against_the_plain_one(dtype, shape):
