@@ -2004,7 +2004,7 @@ def moe_route_grouped(x: torch.Tensor, router: torch.Tensor, correction: torch.T
     splits = max(2, lib.lyp_moe_route_splits(T, K))      # two shares at the least: the product then leaves its sums
     part = torch.empty((splits, T, E), dtype=torch.float32, device=x.device)
     _check(lib.lyp_moe_route_fused(_p(x), x.stride(0), _code(x.dtype), _p(router), None, T, E, K, top, _p(idx), _p(wgt), -1,
-                                   _p(part), splits, 0, _stream()), lib)
+                                   _p(part), splits, 0, 0, 1.0, 0, 0, _stream()), lib)
     _check(lib.lyp_moe_choose_grouped(_p(part), splits, _p(correction), T, E, top, int(groups), int(keep), float(scale),
                                       _p(idx), _p(wgt), _stream()), lib)
     return idx, wgt
