@@ -544,7 +544,7 @@ def main():
     ap.add_argument("--design", default="llama", choices=["llama", "faledra", "ronupel", "tonilix", "vobotar", "panodra", "pudulorn"],
                     help="faledra, ronupel, tonilix, vobotar, panodra, pudulorn: that design's prefill and decode speed at a few "
                          "sizes, each beside the Llama shape (Tonilix and Panodra: the Faledra model; Vobotar: the Tonilix "
-                         "model) of equal size, instead of the headline")
+                         "model; Pudulorn: the Panodra model) of equal size, instead of the headline")
     ap.add_argument("--size", default="", help="with another --design: which sizes, with commas (default: all)")
     args = ap.parse_args()
     if args.gpus != 1:

@@ -303,7 +303,7 @@ def test_position_reach_of_a_model_that_forgets():
 def test_bounds_of_what_is_seen():
     from lyapunov_engine_amd.kernels import ops
 
-    for window, chunk in ((0, 0), (10, 0), (0, 10), (1, 0), (0, 1)):
+    for window, chunk in ((0, 0), (10, 0), (0, 10), (1, 0), (0, 1), (0, 32)):
         for tokens in (1, 64):
             most = 0
             for first in range(0, 150):
